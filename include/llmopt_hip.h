@@ -150,6 +150,8 @@ int llmopt_hip_buffer_argmax_f16(llmopt_hip_buffer *buffer, int64_t vocabulary, 
 /* caml_llmopt_f16_argmax (native/ocaml_metal_stubs.m:2565-2579): index of the
  * first maximum of `count` fp16 logits in host memory (0 for an empty row). */
 int llmopt_hip_f16_argmax(const uint16_t *logits, int64_t count, int64_t *out_index);
+/* The same over a float32 row (no reference counterpart). */
+int llmopt_hip_f32_argmax(const float *logits, int64_t count, int64_t *out_index);
 /* caml_llmopt_sample_f16_native (native/ocaml_metal_stubs.m:2629-2765; called by
  * Sampling.sample, lib/sampling.ml:193-207, on the last logits row in host memory):
  * greedy when temperature <= 1e-4 or top_k == 1; else top-k (0 -> 64, at most 256)
@@ -157,6 +159,9 @@ int llmopt_hip_f16_argmax(const uint16_t *logits, int64_t count, int64_t *out_in
  * draw from xoroshiro128+ seeded with `seed` (0 = from the clock).  Same float32
  * operation order and tie handling as the reference: a seed gives the same token. */
 int llmopt_hip_sample_f16(const uint16_t *logits, int64_t count, double temperature, int64_t top_k,
+                          double top_p, double min_p, int64_t seed, int64_t *out_token);
+/* The same over a float32 row (no reference counterpart). */
+int llmopt_hip_sample_f32(const float *logits, int64_t count, double temperature, int64_t top_k,
                           double top_p, double min_p, int64_t seed, int64_t *out_token);
 
 /* ---- dispatch ------------------------------------------------------------ */
@@ -241,6 +246,14 @@ void llmopt_hip_release_prebaked(llmopt_hip_prebaked *plan);
  * returns LLMOPT_ERR_FAILURE (the reference exits the process there). */
 int llmopt_hip_prebaked_execute(llmopt_hip_prebaked *plan, int64_t token, int64_t past_tokens,
                                 int64_t checkpoint, int64_t *out_token);
+/* No reference counterpart.  The plan's records read their step words - u32
+ * position, u32 state slot - from `step_words` (a buffer the records bind):
+ * every execute writes its past_tokens and checkpoint arguments there first.
+ * past_tokens beyond max_past_tokens or a checkpoint outside [0, slots) is
+ * LLMOPT_ERR_INVALID.  Once per plan, and only for plans without paged
+ * attention or checkpoint records (those keep their own words). */
+int llmopt_hip_prebaked_bind_step(llmopt_hip_prebaked *plan, llmopt_hip_buffer *step_words,
+                                  int64_t max_past_tokens, int64_t slots);
 /* 1 when execute replays one HIP graph, 0 when it launches record by record
  * (no reference counterpart; for diagnostics and tests). */
 int llmopt_hip_prebaked_is_single_submission(llmopt_hip_prebaked *plan);

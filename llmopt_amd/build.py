@@ -92,5 +92,10 @@ def build(force: bool = False, host_ubsan: bool = False) -> str:
     return library
 
 
+def ensure() -> str:
+    """Builds the library if it is missing; a library that is there is taken as it is."""
+    return LIBRARY if os.path.exists(LIBRARY) else build()
+
+
 if __name__ == "__main__":
     print(build(force="--force" in sys.argv, host_ubsan="--host-ubsan" in sys.argv))

@@ -49,13 +49,16 @@ float half_to_float(uint16_t bits) {
   return value;
 }
 
-// a > b in IEEE comparison order (false when either is NaN); fp16 -> fp32 is exact and monotonic
-bool half_greater(uint16_t a, uint16_t b) { return half_to_float(a) > half_to_float(b); }
+// fp16 -> fp32 is exact and monotonic: comparisons of the values are IEEE comparisons of the halves
+float logit_value(uint16_t bits) { return half_to_float(bits); }
+float logit_value(float value) { return value; }
 
-int64_t first_maximum(const uint16_t *logits, int64_t count) {
+// false when either is NaN
+template <typename Logit>
+int64_t first_maximum(const Logit *logits, int64_t count) {
   int64_t best = 0;
   for (int64_t i = 1; i < count; ++i)
-    if (half_greater(logits[i], logits[best])) best = i;
+    if (logit_value(logits[i]) > logit_value(logits[best])) best = i;
   return best;
 }
 
@@ -133,21 +136,21 @@ struct Generator {
   float uniform() { return (float)(next() >> 11) * (1.0f / 9007199254740992.0f); }
 };
 
-}  // namespace
-
-extern "C" int llmopt_hip_f16_argmax(const uint16_t *logits, int64_t count, int64_t *out_index) {
-  if (out_index == nullptr) return llmopt::fail(LLMOPT_ERR_INVALID, "f16 argmax needs an output");
+template <typename Logit>
+int argmax_row(const Logit *logits, int64_t count, int64_t *out_index, const char *type) {
+  if (out_index == nullptr) return llmopt::fail(LLMOPT_ERR_INVALID, "%s argmax needs an output", type);
   if (count < 0 || (count > 0 && logits == nullptr))
-    return llmopt::fail(LLMOPT_ERR_INVALID, "f16 argmax needs %lld logits", (long long)count);
+    return llmopt::fail(LLMOPT_ERR_INVALID, "%s argmax needs %lld logits", type, (long long)count);
   *out_index = count == 0 ? 0 : first_maximum(logits, count);
   return LLMOPT_OK;
 }
 
-extern "C" int llmopt_hip_sample_f16(const uint16_t *logits, int64_t count, double temperature, int64_t top_k,
-                                     double top_p, double min_p, int64_t seed, int64_t *out_token) {
-  if (out_token == nullptr) return llmopt::fail(LLMOPT_ERR_INVALID, "f16 sampling needs an output");
+template <typename Logit>
+int sample_row(const Logit *logits, int64_t count, double temperature, int64_t top_k, double top_p, double min_p,
+               int64_t seed, int64_t *out_token, const char *type) {
+  if (out_token == nullptr) return llmopt::fail(LLMOPT_ERR_INVALID, "%s sampling needs an output", type);
   if (count < 0 || (count > 0 && logits == nullptr))
-    return llmopt::fail(LLMOPT_ERR_INVALID, "f16 sampling needs %lld logits", (long long)count);
+    return llmopt::fail(LLMOPT_ERR_INVALID, "%s sampling needs %lld logits", type, (long long)count);
   if (count == 0) {
     *out_token = 0;
     return LLMOPT_OK;
@@ -164,7 +167,7 @@ extern "C" int llmopt_hip_sample_f16(const uint16_t *logits, int64_t count, doub
   const int keep = requested <= 0 ? 64 : requested <= 256 ? requested : 256;
   BoundedHeap heap;
   for (int64_t i = 0; i < count; ++i) {
-    const float value = half_to_float(logits[i]);
+    const float value = logit_value(logits[i]);
     if (heap.size() < keep)
       heap.push({(uint32_t)i, value});
     else if (value > heap.root().logit)
@@ -233,4 +236,24 @@ extern "C" int llmopt_hip_sample_f16(const uint16_t *logits, int64_t count, doub
   }
   *out_token = (int64_t)chosen;
   return LLMOPT_OK;
+}
+
+}  // namespace
+
+extern "C" int llmopt_hip_f16_argmax(const uint16_t *logits, int64_t count, int64_t *out_index) {
+  return argmax_row(logits, count, out_index, "f16");
+}
+
+extern "C" int llmopt_hip_f32_argmax(const float *logits, int64_t count, int64_t *out_index) {
+  return argmax_row(logits, count, out_index, "f32");
+}
+
+extern "C" int llmopt_hip_sample_f16(const uint16_t *logits, int64_t count, double temperature, int64_t top_k,
+                                     double top_p, double min_p, int64_t seed, int64_t *out_token) {
+  return sample_row(logits, count, temperature, top_k, top_p, min_p, seed, out_token, "f16");
+}
+
+extern "C" int llmopt_hip_sample_f32(const float *logits, int64_t count, double temperature, int64_t top_k,
+                                     double top_p, double min_p, int64_t seed, int64_t *out_token) {
+  return sample_row(logits, count, temperature, top_k, top_p, min_p, seed, out_token, "f32");
 }

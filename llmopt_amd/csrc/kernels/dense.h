@@ -1,0 +1,213 @@
+// Host-visible launch interface of the kernels over bfloat16 weights: linears with the epilogues a
+// layered decoder needs, chunked attention with a softmax sink, the Mamba-2 recurrence, and routed
+// experts.  Plain structs and device pointers; launchers are asynchronous on the stream and assume
+// validated sizes.  `f32` selects float activations (else bfloat16); weights are bfloat16 in both.
+#pragma once
+
+#include <hip/hip_runtime.h>
+#include <stdint.h>
+
+namespace llmopt {
+
+// The step words in device memory every stateful kernel reads: the position of the first token of the
+// step in its sequence, and the sequence's state slot.
+constexpr uint32_t kStatePosition = 0, kStateSlot = 1, kStateWords = 2;
+
+enum class DenseEpilogue : uint32_t {
+  kStore = 0,     // out[r, c] (activation type)
+  kStoreF32 = 1,  // out_f32[r, c]
+  kAdd = 2,       // stream[r, c] += result * (row_gate ? sigmoid(row_gate[r * row_gate_stride]) : 1)
+  kGated = 3,     // out[r, c] = act(gate) * up
+  kQkv = 4,       // kStore, with the value columns mixed with another layer's values
+  kSplit = 5,     // columns below `split` to out, the rest to out_f32 as float32
+};
+
+// Values of a layer, mixed per token with those of the first mixing layer.
+// mode 0: as they are; 1: this is the first such layer, its values are kept in v_first;
+// 2: (1 - lambda) v + lambda v_first.
+struct ValueMix {
+  uint32_t mode;
+  float lambda;
+  float *v_first;  // f32 [m, n_v]
+};
+
+struct DenseLinearArgs {
+  bool f32;
+  const void *x;         // activations [m, k], row stride ldx
+  const uint16_t *w;     // bf16 [n, k]
+  const uint16_t *w_up;  // kGated: the second matrix
+  uint32_t m, n, k, ldx;
+  DenseEpilogue epilogue;
+  uint32_t activation;
+  void *out;
+  float *out_f32;        // kStoreF32, kSplit, and the stream of kAdd
+  uint32_t ld_out, ld_f32;
+  const float *row_gate;
+  uint32_t row_gate_stride;
+  uint32_t split;        // kSplit; kQkv: first value column
+  ValueMix mix;
+  // routed rows (null: the plain product): see RoutePlan
+  const uint32_t *tile_expert, *tile_first, *tile_rows, *row_source;
+  uint32_t tiles;
+};
+// Rows of a product tile of the routed form (what RoutePlan cuts experts into).
+constexpr uint32_t kRoutedTileRows = 64;
+hipError_t launch_dense_gemm(const DenseLinearArgs &args, hipStream_t stream);
+
+// out[r, :] = x[row, :] / rms * weight with row = rows ? rows[r] : r; `groups` equal parts normalised each
+// by its own root mean square.  gate != null: the input is x * silu(gate) (x, gate in the activation type).
+struct DenseNormArgs {
+  bool f32;
+  const float *x;        // f32 [*, width], when x_act is null
+  const void *x_act;     // activation type [rows, width]
+  const void *gate;      // activation type, row stride ld_gate
+  uint32_t ld_gate;
+  const uint16_t *weight;  // bf16 [width]
+  void *out;             // activation type [rows, width]
+  const uint32_t *rows_index;
+  uint32_t rows, width, groups;
+  float epsilon;
+};
+hipError_t launch_dense_norm(const DenseNormArgs &args, hipStream_t stream);
+
+struct DenseEmbeddingArgs {
+  const int64_t *tokens;
+  const uint16_t *embed;  // bf16 [vocabulary, width]
+  float *stream;          // f32 [m, width]
+  uint32_t m, vocabulary, width;
+  float scale;
+};
+hipError_t launch_dense_embedding(const DenseEmbeddingArgs &args, hipStream_t stream);
+
+// ---- one token: matrix-vector products ----------------------------------------------------------
+
+enum class GemvEpilogue : uint32_t {
+  kStore = 0, kStoreF32 = 1, kAdd = 2, kGated = 3,
+  kQkv = 4,    // q to out; mixed k, v straight to their cache rows
+  kSsmIn = 5,  // z as it is, x | B | C through the convolution and silu, dt through softplus: all to out_f32
+};
+
+struct ChunkCache {
+  void *keys, *values;  // [slot][kv_heads][capacity][dim] / [...][vdim], activation type
+  uint32_t capacity;    // rows per head; position p lives in row p % capacity
+  uint32_t chunk;       // positions of one chunk (capacity >= chunk); 0: no chunks
+};
+
+struct DenseGemvArgs {
+  bool f32;
+  // input: norm_weight == null: activation-type row, or f32 (x_is_f32); else the f32 row normalised on the way in
+  const void *x;
+  bool x_is_f32;
+  const uint16_t *norm_weight;
+  uint32_t norm_groups;
+  float epsilon;
+  const uint16_t *w, *w_up;
+  uint32_t n, k;
+  GemvEpilogue epilogue;
+  uint32_t activation;
+  void *out;
+  float *out_f32;
+  // kQkv
+  const uint32_t *state;
+  uint32_t n_q, n_k, dim, vdim, kv_heads;
+  ChunkCache cache;
+  ValueMix mix;
+  // kSsmIn
+  const uint16_t *conv, *conv_bias, *dt_bias;
+  float *conv_state;  // f32 [slot][taps][channels], position p in row p % taps
+  uint32_t inner, channels, taps;
+};
+bool dense_gemv_ok(const DenseGemvArgs &args);
+hipError_t launch_dense_gemv(const DenseGemvArgs &args, hipStream_t stream);
+
+// ---- attention ---------------------------------------------------------------------------------------
+
+// q | k | v rows of m new tokens at positions state[0] .. + m - 1; earlier keys of the first token's
+// chunk come from the cache.  score = cap tanh(scale q k / cap); the sink joins the denominator only.
+struct ChunkAttentionArgs {
+  bool f32;
+  const void *qkv;  // [m, heads * dim + kv_heads * (dim + vdim)]; one token: only q is read
+  ChunkCache cache;
+  const uint16_t *sink;  // bf16 [heads], may be null
+  const uint32_t *state;
+  void *out;  // [m, heads * vdim]
+  uint32_t m, heads, kv_heads, dim, vdim;
+  float scale, softcap;  // softcap 0: none
+  void *workspace;
+  size_t workspace_bytes;
+};
+size_t chunk_attention_workspace_bytes(const ChunkAttentionArgs &args);
+bool chunk_attention_ok(const ChunkAttentionArgs &args);
+hipError_t launch_chunk_attention(const ChunkAttentionArgs &args, hipStream_t stream);
+// k, v of the step's tokens into their cache rows (those that the ring still holds afterwards).
+hipError_t launch_chunk_cache_write(const ChunkAttentionArgs &args, hipStream_t stream);
+
+// ---- Mamba-2 ------------------------------------------------------------------------------------------
+
+struct SsmArgs {
+  bool f32;
+  uint32_t m, heads, vdim, groups, state_size, taps;
+  const uint32_t *step;  // state words
+  const void *projected;  // [m, inner + channels] z | x B C, activation type
+  const float *dt;        // f32 [m, heads], before softplus
+  const uint16_t *conv, *conv_bias, *dt_bias, *a_log, *d_skip;
+  float *conv_state;      // [slot][taps][channels]
+  float *ssm_state;       // [slot][heads][vdim][state_size]
+  void *y;                // m > 1: activation type [m, inner], without the gate
+  // one token: the row kSsmIn left, and y * silu(z) as f32 [inner]
+  const float *row;
+  float *gated;
+  void *workspace;
+  size_t workspace_bytes;
+};
+constexpr uint32_t kSsmChunk = 64;
+size_t ssm_workspace_bytes(const SsmArgs &args);
+hipError_t launch_ssm_step(const SsmArgs &args, hipStream_t stream);
+hipError_t launch_ssm_prefill(const SsmArgs &args, hipStream_t stream);
+
+// ---- routed experts -------------------------------------------------------------------------------------
+
+struct RoutePlan {
+  uint32_t m, experts, top;
+  const float *logits;  // f32 [m, ld_logits]
+  uint32_t ld_logits;
+  uint32_t *expert;     // [m, top]
+  float *weight;        // [m, top]
+  uint32_t *position;   // [m, top]: row of the sorted order
+  uint32_t *row_token;  // [m * top]
+  uint32_t *tile_expert, *tile_first, *tile_rows;  // [max_tiles]
+  uint32_t max_tiles;
+};
+uint32_t route_max_tiles(uint32_t m, uint32_t experts, uint32_t top);
+// The `top` largest logits of every token (ties to the lower index), the softmax over them, the
+// (token, choice) pairs sorted by expert and cut into product tiles of one expert.
+hipError_t launch_route(const RoutePlan &plan, hipStream_t stream);
+// stream[t, :] += sum_s weight[t, s] rows[position[t, s], :]
+struct RouteCombineArgs {
+  bool f32;
+  const RoutePlan *plan;
+  const void *rows;  // activation type [m * top, width]
+  float *stream;
+  uint32_t width;
+};
+hipError_t launch_route_combine(const RouteCombineArgs &args, hipStream_t stream);
+
+// One token: every workgroup selects the experts from the logits itself.
+struct MoeGemvArgs {
+  bool f32;
+  const float *logits;  // f32 [experts (+ 1: the shared expert's gate)]
+  uint32_t experts, top, width, ff, shared_ff;
+  const float *x;                 // f32 [width]
+  const uint16_t *norm_weight;
+  float epsilon;
+  const uint16_t *gate, *up;      // bf16 [experts][ff, width]
+  const uint16_t *down;           // bf16 [experts][width, ff]
+  const uint16_t *shared_gate, *shared_up, *shared_down;
+  float *hidden;                  // f32 [top][ff] then [shared_ff]
+  float *stream;                  // f32 [width]
+  uint32_t activation;
+};
+hipError_t launch_moe_gemv_up(const MoeGemvArgs &args, hipStream_t stream);
+hipError_t launch_moe_gemv_down(const MoeGemvArgs &args, hipStream_t stream);
+
+}  // namespace llmopt

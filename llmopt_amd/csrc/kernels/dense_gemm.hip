@@ -1,0 +1,401 @@
+// Matrix product of many activation rows with bfloat16 weights on the matrix cores, and the small
+// row-wise kernels around it (norm, embedding).
+//
+//   out[r, c] = sum_k x[r, k] w[c, k]       x [m, k] bf16 or f32, w bf16 [n, k], sums in float32
+//
+// A workgroup of four waves owns a BM x BN tile and walks K in stages of 64, double-buffered through
+// LDS: the next stage travels global -> registers while this one is multiplied, one barrier a stage.
+// LDS rows carry 16 bytes of padding, so that the sixteen rows an operand read touches start in
+// different banks.  The weights are the A operand and the activations the B operand: a lane then ends
+// with four consecutive output columns of one row, and the epilogue stores 8 or 16 bytes at a time.
+//
+//  * gated: the 16-column groups of a tile alternate between the gate and the up matrix, so that both
+//    values of an output element meet in one lane.
+//  * routed: a tile belongs to one expert; its rows are gathered (or taken in place) from the order the
+//    route plan made, and tiles that the plan did not fill end at once.
+//  * workgroups are dealt to the XCDs in contiguous runs (blockIdx % 8 is the XCD), and inside a run
+//    eight row tiles share a column of weight tiles: both operands are re-read from that XCD's L2.
+#include <algorithm>
+
+#include "dense.h"
+#include "dense_common.h"
+#include "kernels_internal.h"
+
+namespace llmopt {
+namespace {
+
+constexpr int kStageK = 64;
+
+struct GemmParams {
+  DenseLinearArgs a;
+  uint32_t tiles_m, tiles_n, total, per_xcd;
+};
+
+template <typename T>
+constexpr int lds_stride() { return kStageK + 16 / (int)sizeof(T); }
+
+template <typename T, int BM, int BN>
+constexpr int gemm_lds_bytes() {
+  return 2 * (BM * lds_stride<T>() * (int)sizeof(T) + BN * lds_stride<__bf16>() * 2);
+}
+
+template <typename T>
+__device__ __forceinline__ void store4(T *out, f32x4 v, uint32_t count, bool vec) {
+  if (vec && count >= 4) {
+    typedef T x4 __attribute__((ext_vector_type(4)));
+    x4 packed;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) packed[i] = (T)v[i];
+    *reinterpret_cast<x4 *>(out) = packed;
+    return;
+  }
+#pragma unroll
+  for (int i = 0; i < 4; ++i)
+    if (i < (int)count) out[i] = (T)v[i];
+}
+
+// Four results of row r, columns c .. c + 3 (those below n).
+template <typename T>
+__device__ __forceinline__ void emit(const DenseLinearArgs &a, uint32_t r, uint32_t c, f32x4 v) {
+  const uint32_t count = a.n - c;
+  switch (a.epilogue) {
+    case DenseEpilogue::kStore:
+    case DenseEpilogue::kGated:
+      store4(static_cast<T *>(a.out) + (size_t)r * a.ld_out + c, v, count, (a.ld_out & 3) == 0);
+      return;
+    case DenseEpilogue::kStoreF32:
+      store4(a.out_f32 + (size_t)r * a.ld_f32 + c, v, count, (a.ld_f32 & 3) == 0);
+      return;
+    case DenseEpilogue::kAdd: {
+      float *p = a.out_f32 + (size_t)r * a.ld_f32 + c;
+      const float gate = a.row_gate ? sigmoid_f32(a.row_gate[(size_t)r * a.row_gate_stride]) : 1.0f;
+      if (count >= 4 && (a.ld_f32 & 3) == 0) {
+        f32x4 old = *reinterpret_cast<f32x4 *>(p);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) old[i] += gate * v[i];
+        *reinterpret_cast<f32x4 *>(p) = old;
+        return;
+      }
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+        if (i < (int)count) p[i] += gate * v[i];
+      return;
+    }
+    case DenseEpilogue::kQkv: {
+      if (a.mix.mode != 0) {
+        const uint32_t n_v = a.n - a.split;
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+          if (i < (int)count && c + i >= a.split) {
+            float *first = a.mix.v_first + (size_t)r * n_v + (c + i - a.split);
+            if (a.mix.mode == 1) *first = v[i];
+            else v[i] = (1.0f - a.mix.lambda) * v[i] + a.mix.lambda * *first;
+          }
+      }
+      store4(static_cast<T *>(a.out) + (size_t)r * a.ld_out + c, v, count, (a.ld_out & 3) == 0);
+      return;
+    }
+    case DenseEpilogue::kSplit:
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+        if (i < (int)count) {
+          if (c + i < a.split) static_cast<T *>(a.out)[(size_t)r * a.ld_out + c + i] = (T)v[i];
+          else a.out_f32[(size_t)r * a.ld_f32 + (c + i - a.split)] = v[i];
+        }
+      return;
+  }
+}
+
+// WM x WN waves; a wave owns (BM / WM) x (BN / WN).
+template <typename T, int BM, int BN, int WM, bool GATED, bool ROUTED, bool VEC>
+__global__ __launch_bounds__(256) void dense_gemm_kernel(GemmParams p) {
+  constexpr int WN = 4 / WM;
+  constexpr int MT = BM / WM / 16, NT = BN / WN / 16;
+  constexpr int A_PIECES = BM * 8 / 256, W_PIECES = BN * 8 / 256;
+  constexpr int SA = lds_stride<T>(), SW = lds_stride<__bf16>();
+  constexpr int COLUMNS = GATED ? BN / 2 : BN;
+  static_assert(!GATED || NT % 2 == 0, "gate and up of an element meet in one wave");
+  extern __shared__ __attribute__((aligned(16))) char lds[];
+  T *lds_a = reinterpret_cast<T *>(lds);
+  __bf16 *lds_w = reinterpret_cast<__bf16 *>(lds + 2 * BM * SA * sizeof(T));
+  const DenseLinearArgs &a = p.a;
+
+  uint32_t m_first, m_rows, n_first, expert = 0;
+  if (ROUTED) {
+    const uint32_t tile = blockIdx.y;
+    m_rows = a.tile_rows[tile];
+    if (m_rows == 0) return;
+    m_first = a.tile_first[tile];
+    expert = a.tile_expert[tile];
+    n_first = blockIdx.x * COLUMNS;
+  } else {
+    const uint32_t id = (blockIdx.x & 7) * p.per_xcd + (blockIdx.x >> 3);
+    if (id >= p.total) return;
+    // groups of eight row tiles walk the column tiles together
+    const uint32_t group_tiles = 8 * p.tiles_n, group = id / group_tiles, within = id % group_tiles;
+    const uint32_t rows_here = min(8u, p.tiles_m - group * 8);
+    const uint32_t tile_m = group * 8 + within % rows_here, tile_n = within / rows_here;
+    m_first = tile_m * BM;
+    m_rows = min((uint32_t)BM, a.m - m_first);
+    n_first = tile_n * COLUMNS;
+  }
+
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
+  const int wm = wave / WN, wn = wave % WN;
+  const int piece = tid & 7, row_in_pass = tid >> 3;  // 32 rows a pass
+
+  const T *src_a[A_PIECES];
+#pragma unroll
+  for (int i = 0; i < A_PIECES; ++i) {
+    uint32_t r = m_first + min((uint32_t)(row_in_pass + 32 * i), m_rows - 1);
+    if (ROUTED && a.row_source) r = a.row_source[r];
+    src_a[i] = static_cast<const T *>(a.x) + (size_t)r * a.ldx + piece * 8;
+  }
+  const __bf16 *src_w[W_PIECES];
+#pragma unroll
+  for (int i = 0; i < W_PIECES; ++i) {
+    const int r = row_in_pass + 32 * i;
+    const uint16_t *matrix = a.w;
+    uint32_t c = n_first + r;
+    if (GATED) {
+      if ((r >> 4) & 1) matrix = a.w_up;
+      c = n_first + (r >> 5) * 16 + (r & 15);
+    }
+    c = min(c, a.n - 1);
+    src_w[i] = reinterpret_cast<const __bf16 *>(matrix) + ((size_t)expert * a.n + c) * a.k + piece * 8;
+  }
+
+  Frag<T> reg_a[A_PIECES];
+  bf16x8 reg_w[W_PIECES];
+  auto fetch = [&](uint32_t k0) {
+    const int count = (int)a.k - (int)(k0 + piece * 8);
+#pragma unroll
+    for (int i = 0; i < W_PIECES; ++i) reg_w[i] = load_piece(src_w[i] + k0, count, VEC);
+#pragma unroll
+    for (int i = 0; i < A_PIECES; ++i) reg_a[i] = load_piece(src_a[i] + k0, count, VEC);
+  };
+  auto stash = [&](int buffer) {
+#pragma unroll
+    for (int i = 0; i < A_PIECES; ++i)
+      *reinterpret_cast<Frag<T> *>(lds_a + (buffer * BM + row_in_pass + 32 * i) * SA + piece * 8) = reg_a[i];
+#pragma unroll
+    for (int i = 0; i < W_PIECES; ++i)
+      *reinterpret_cast<bf16x8 *>(lds_w + (buffer * BN + row_in_pass + 32 * i) * SW + piece * 8) = reg_w[i];
+  };
+
+  f32x4 acc[MT][NT];
+#pragma unroll
+  for (int i = 0; i < MT; ++i)
+#pragma unroll
+    for (int j = 0; j < NT; ++j) acc[i][j] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+
+  fetch(0);
+  stash(0);
+  __syncthreads();
+  const int stages = (int)((a.k + kStageK - 1) / kStageK);
+  const int fr = lane & 15, fk = (lane >> 4) * 8;
+  for (int s = 0; s < stages; ++s) {
+    const int buffer = s & 1;
+    if (s + 1 < stages) fetch((s + 1) * kStageK);
+    const T *la = lds_a + (buffer * BM + wm * (BM / WM) + fr) * SA + fk;
+    const __bf16 *lw = lds_w + (buffer * BN + wn * (BN / WN) + fr) * SW + fk;
+#pragma unroll
+    for (int kk = 0; kk < kStageK; kk += 32) {
+      Frag<T> fa[MT];
+      Frag<T> fw[NT];
+#pragma unroll
+      for (int j = 0; j < NT; ++j)
+        fw[j] = convert_frag<T>(*reinterpret_cast<const bf16x8 *>(lw + j * 16 * SW + kk));
+#pragma unroll
+      for (int i = 0; i < MT; ++i) fa[i] = *reinterpret_cast<const Frag<T> *>(la + i * 16 * SA + kk);
+#pragma unroll
+      for (int i = 0; i < MT; ++i)
+#pragma unroll
+        for (int j = 0; j < NT; ++j) acc[i][j] = mma(fw[j], fa[i], acc[i][j]);
+    }
+    if (s + 1 < stages) stash(buffer ^ 1);
+    __syncthreads();
+  }
+
+  const int column = (lane >> 4) * 4;
+#pragma unroll
+  for (int i = 0; i < MT; ++i) {
+    const uint32_t r_in_tile = wm * (BM / WM) + i * 16 + fr;
+    if (r_in_tile >= m_rows) continue;
+    const uint32_t r = m_first + r_in_tile;
+    if (GATED) {
+#pragma unroll
+      for (int j = 0; j < NT; j += 2) {
+        const uint32_t c = n_first + (wn * NT / 2 + j / 2) * 16 + column;
+        if (c >= a.n) continue;
+        f32x4 v;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[e] = gate_activation(acc[i][j][e], a.activation) * acc[i][j + 1][e];
+        emit<T>(a, r, c, v);
+      }
+    } else {
+#pragma unroll
+      for (int j = 0; j < NT; ++j) {
+        const uint32_t c = n_first + wn * (BN / WN) + j * 16 + column;
+        if (c < a.n) emit<T>(a, r, c, acc[i][j]);
+      }
+    }
+  }
+}
+
+template <typename T, int BM, int BN, int WM, bool GATED, bool ROUTED, bool VEC>
+hipError_t run_gemm(const DenseLinearArgs &a, hipStream_t stream) {
+  constexpr int bytes = gemm_lds_bytes<T, BM, BN>();
+  static bool allowed[kMaxDevices] = {};
+  if (bytes > 64 * 1024)
+    if (hipError_t status = allow_dynamic_lds(
+            reinterpret_cast<const void *>(dense_gemm_kernel<T, BM, BN, WM, GATED, ROUTED, VEC>), bytes, allowed))
+      return status;
+  GemmParams p = {};
+  p.a = a;
+  constexpr uint32_t columns = GATED ? BN / 2 : BN;
+  p.tiles_n = (a.n + columns - 1) / columns;
+  dim3 grid;
+  if (ROUTED) {
+    grid = dim3(p.tiles_n, a.tiles);
+  } else {
+    p.tiles_m = (a.m + BM - 1) / BM;
+    p.total = p.tiles_m * p.tiles_n;
+    p.per_xcd = (p.total + 7) / 8;
+    grid = dim3(p.per_xcd * 8);
+  }
+  dense_gemm_kernel<T, BM, BN, WM, GATED, ROUTED, VEC><<<grid, 256, bytes, stream>>>(p);
+  return hipGetLastError();
+}
+
+template <bool GATED, bool ROUTED>
+hipError_t pick_gemm(const DenseLinearArgs &a, hipStream_t stream) {
+  const bool vec = a.k % 8 == 0 && a.ldx % 8 == 0;
+  constexpr int SMALL = ROUTED ? (int)kRoutedTileRows : 32;
+  const uint32_t columns = a.n * (GATED ? 2 : 1);
+  if (a.f32) {
+    if (!vec) return run_gemm<float, SMALL, 64, 2, GATED, ROUTED, false>(a, stream);
+    return run_gemm<float, SMALL, 64, 2, GATED, ROUTED, true>(a, stream);
+  }
+  if (!vec) return run_gemm<__bf16, SMALL, 64, 2, GATED, ROUTED, false>(a, stream);
+  if (ROUTED) return run_gemm<__bf16, (int)kRoutedTileRows, 128, 2, GATED, ROUTED, true>(a, stream);
+  const uint64_t big = (uint64_t)((a.m + 127) / 128) * ((columns + 127) / 128);
+  if (a.m > 64 && big >= 192) return run_gemm<__bf16, 128, 128, 2, GATED, false, true>(a, stream);
+  const uint64_t middle = (uint64_t)((a.m + 63) / 64) * ((columns + 127) / 128);
+  if (a.m > 32 && middle >= 192) return run_gemm<__bf16, 64, 128, 2, GATED, false, true>(a, stream);
+  return run_gemm<__bf16, SMALL, 64, 2, GATED, ROUTED, true>(a, stream);
+}
+
+// ---- row-wise kernels ------------------------------------------------------------------------------
+
+template <typename T>
+__global__ __launch_bounds__(256) void dense_norm_kernel(DenseNormArgs a) {
+  extern __shared__ float row[];
+  __shared__ float scratch[4];
+  const uint32_t r = blockIdx.x;
+  const uint32_t source = a.rows_index ? a.rows_index[r] : r;
+  const __bf16 *weight = reinterpret_cast<const __bf16 *>(a.weight);
+  const uint32_t part = a.width / a.groups;
+  for (uint32_t g = 0; g < a.groups; ++g) {
+    float sum = 0.0f;
+    for (uint32_t i = g * part + threadIdx.x; i < (g + 1) * part; i += 256) {
+      float v;
+      if (a.x_act) {
+        v = to_f32(static_cast<const T *>(a.x_act)[(size_t)source * a.width + i]);
+        if (a.gate) v *= silu_f32(to_f32(static_cast<const T *>(a.gate)[(size_t)source * a.ld_gate + i]));
+      } else {
+        v = a.x[(size_t)source * a.width + i];
+      }
+      row[i] = v;
+      sum += v * v;
+    }
+    sum = block_sum<4>(sum, scratch);
+    const float inverse = 1.0f / sqrtf(sum / (float)part + a.epsilon);
+    for (uint32_t i = g * part + threadIdx.x; i < (g + 1) * part; i += 256)
+      static_cast<T *>(a.out)[(size_t)r * a.width + i] = (T)(row[i] * inverse * (float)weight[i]);
+  }
+}
+
+// The same for widths a thread covers in pieces of eight (part % 8 == 0, at most 8 pieces a thread):
+// 16-byte accesses and the row in registers; four waves a row, one group at a time.
+template <typename T>
+__global__ __launch_bounds__(256) void dense_norm_vec_kernel(DenseNormArgs a) {
+  __shared__ float scratch[4];
+  const uint32_t r = blockIdx.x, group = blockIdx.y;
+  const uint32_t source = a.rows_index ? a.rows_index[r] : r;
+  const __bf16 *weight = reinterpret_cast<const __bf16 *>(a.weight);
+  const uint32_t part = a.width / a.groups, first = group * part;
+  f32x8 v[8];
+  float sum = 0.0f;
+#pragma unroll
+  for (int q = 0; q < 8; ++q) {
+    const uint32_t i = (q * 256 + threadIdx.x) * 8;
+    if (i >= part) break;
+    if (a.x_act) {
+      v[q] = convert_frag<float>(
+          *reinterpret_cast<const Frag<T> *>(static_cast<const T *>(a.x_act) + (size_t)source * a.width + first + i));
+      if (a.gate) {
+        const f32x8 g = convert_frag<float>(*reinterpret_cast<const Frag<T> *>(
+            static_cast<const T *>(a.gate) + (size_t)source * a.ld_gate + first + i));
+#pragma unroll
+        for (int e = 0; e < 8; ++e) v[q][e] *= silu_f32(g[e]);
+      }
+    } else {
+      v[q] = *reinterpret_cast<const f32x8 *>(a.x + (size_t)source * a.width + first + i);
+    }
+#pragma unroll
+    for (int e = 0; e < 8; ++e) sum += v[q][e] * v[q][e];
+  }
+  sum = block_sum<4>(sum, scratch);
+  const float inverse = 1.0f / sqrtf(sum / (float)part + a.epsilon);
+#pragma unroll
+  for (int q = 0; q < 8; ++q) {
+    const uint32_t i = (q * 256 + threadIdx.x) * 8;
+    if (i >= part) break;
+    const bf16x8 w = *reinterpret_cast<const bf16x8 *>(weight + first + i);
+    Frag<T> out;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) out[e] = (T)(v[q][e] * inverse * (float)w[e]);
+    *reinterpret_cast<Frag<T> *>(static_cast<T *>(a.out) + (size_t)r * a.width + first + i) = out;
+  }
+}
+
+__global__ __launch_bounds__(256) void dense_embedding_kernel(DenseEmbeddingArgs a) {
+  const uint32_t t = blockIdx.x;
+  const int64_t token = a.tokens[t];
+  const bool known = token >= 0 && token < (int64_t)a.vocabulary;
+  const __bf16 *source = reinterpret_cast<const __bf16 *>(a.embed) + (size_t)(known ? token : 0) * a.width;
+  for (uint32_t i = threadIdx.x; i < a.width; i += 256)
+    a.stream[(size_t)t * a.width + i] = known ? (float)source[i] * a.scale : 0.0f;
+}
+
+}  // namespace
+
+hipError_t launch_dense_gemm(const DenseLinearArgs &a, hipStream_t stream) {
+  const bool gated = a.epilogue == DenseEpilogue::kGated;
+  if (a.tile_expert) return gated ? pick_gemm<true, true>(a, stream) : pick_gemm<false, true>(a, stream);
+  return gated ? pick_gemm<true, false>(a, stream) : pick_gemm<false, false>(a, stream);
+}
+
+hipError_t launch_dense_norm(const DenseNormArgs &a, hipStream_t stream) {
+  const uint32_t part = a.width / a.groups;
+  const bool vec = part % 8 == 0 && part <= 8 * 256 * 8 && (!a.gate || a.ld_gate % 8 == 0);
+  if (vec) {
+    const dim3 grid(a.rows, a.groups);
+    if (a.f32) dense_norm_vec_kernel<float><<<grid, 256, 0, stream>>>(a);
+    else dense_norm_vec_kernel<__bf16><<<grid, 256, 0, stream>>>(a);
+    return hipGetLastError();
+  }
+  const size_t bytes = (size_t)a.width * 4;
+  if (bytes > 60 * 1024) return hipErrorInvalidValue;
+  if (a.f32) dense_norm_kernel<float><<<a.rows, 256, bytes, stream>>>(a);
+  else dense_norm_kernel<__bf16><<<a.rows, 256, bytes, stream>>>(a);
+  return hipGetLastError();
+}
+
+hipError_t launch_dense_embedding(const DenseEmbeddingArgs &a, hipStream_t stream) {
+  dense_embedding_kernel<<<a.m, 256, 0, stream>>>(a);
+  return hipGetLastError();
+}
+
+}  // namespace llmopt

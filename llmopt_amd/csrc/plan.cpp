@@ -47,6 +47,15 @@ struct llmopt_hip_prebaked : llmopt::RefCounted {
   uint32_t *device_past = nullptr;
   uint32_t past_count = 0;
   uint32_t past_capacity = 0xffffffffu;  // longest context the captured launches are sized for
+  // step words (position, state slot) in a buffer of the caller that the records read; null: none bound
+  llmopt_hip_buffer *step_buffer = nullptr;
+  uint32_t *past_words() const {
+    return step_buffer ? reinterpret_cast<uint32_t *>(step_buffer->device) : device_past;
+  }
+  uint32_t past_word_count() const { return step_buffer ? 1 : past_count; }
+  uint32_t *checkpoint_word() const {
+    return step_buffer ? reinterpret_cast<uint32_t *>(step_buffer->device) + 1 : device_checkpoint;
+  }
   // false: a record cannot be frozen (a masked attention: the mask's row length follows the
   // context) and every step launches the records from the host, as the reference does
   bool single_submission = true;
@@ -138,8 +147,8 @@ int enqueue_step(llmopt_hip_prebaked *plan, int64_t token, bool chain, int64_t p
   if (plan->single_submission) {
     if (plan->executable == nullptr || plan->workspace_generation != context->workspace_generation)
       if (int status = capture_plan(plan)) return status;
-    LLMOPT_HIP_TRY(launch_plan_state(token_slot, token, chain_from, plan->device_past, (uint32_t)past_tokens,
-                                     plan->past_count, plan->device_checkpoint, checkpoint, context->stream),
+    LLMOPT_HIP_TRY(launch_plan_state(token_slot, token, chain_from, plan->past_words(), (uint32_t)past_tokens,
+                                     plan->past_word_count(), plan->checkpoint_word(), checkpoint, context->stream),
                    "HIP could not write the decode step's state");
     LLMOPT_HIP_TRY(hipGraphLaunch(plan->executable, context->stream), "HIP graph launch failed");
   } else {
@@ -177,7 +186,9 @@ int enqueue_step(llmopt_hip_prebaked *plan, int64_t token, bool chain, int64_t p
 
 bool nan_check_applies(const std::string &name) {
   // integer buffers and packed cache bytes are not floating point (same exclusions as the reference)
-  return name.find("_i64") == std::string::npos && name.find("cache_pack") == std::string::npos;
+  // (and bfloat16 entries mix bfloat16 with float32 operands)
+  return name.find("_i64") == std::string::npos && name.find("cache_pack") == std::string::npos &&
+         name.find("_bf16") == std::string::npos;
 }
 
 int range_has_nan(llmopt_hip_prebaked *plan, const std::string &name, const BoundBuffer &buffer, bool *bad) {
@@ -210,9 +221,9 @@ int debug_step(llmopt_hip_prebaked *plan, int64_t token, int64_t past_tokens, bo
     token_slot = reinterpret_cast<int64_t *>(plan->token_buffer->device);
   }
   // frozen records read the context length from the plan's device words, the others from byte 12
-  LLMOPT_HIP_TRY(launch_plan_state(token_slot, token, nullptr, plan->single_submission ? plan->device_past : nullptr,
-                                   (uint32_t)past_tokens, plan->single_submission ? plan->past_count : 0,
-                                   plan->single_submission ? plan->device_checkpoint : nullptr, plan->checkpoint,
+  LLMOPT_HIP_TRY(launch_plan_state(token_slot, token, nullptr, plan->single_submission ? plan->past_words() : nullptr,
+                                   (uint32_t)past_tokens, plan->single_submission ? plan->past_word_count() : 0,
+                                   plan->single_submission ? plan->checkpoint_word() : nullptr, plan->checkpoint,
                                    context->stream),
                  "HIP could not write the decode step's state");
   hipEvent_t before = nullptr, after = nullptr;
@@ -421,6 +432,7 @@ void llmopt_hip_release_prebaked(llmopt_hip_prebaked *plan) {
   for (DispatchRecord &record : plan->records) drop_record(&record);
   if (plan->token_buffer) llmopt_hip_release_buffer(plan->token_buffer);
   if (plan->output_buffer) llmopt_hip_release_buffer(plan->output_buffer);
+  if (plan->step_buffer) llmopt_hip_release_buffer(plan->step_buffer);
   llmopt_hip_release_library(plan->library);
   delete plan;
 }
@@ -446,6 +458,21 @@ int llmopt_hip_prebaked_execute(llmopt_hip_prebaked *plan, int64_t token, int64_
   if (hipStreamSynchronize(plan->library->context->stream) != hipSuccess)
     return fail(LLMOPT_ERR_FAILURE, "Prebaked HIP batch failed");
   if (out_token) *out_token = (int64_t)next_token;
+  return LLMOPT_OK;
+}
+
+int llmopt_hip_prebaked_bind_step(llmopt_hip_prebaked *plan, llmopt_hip_buffer *step_words, int64_t max_past_tokens,
+                                  int64_t slots) {
+  if (plan == nullptr) return fail(LLMOPT_ERR_FAILURE, "HIP prebaked plan has been finalized");
+  if (step_words == nullptr) return fail(LLMOPT_ERR_FAILURE, "HIP buffer has been finalized");
+  if (step_words->length < 8 || max_past_tokens < 0 || max_past_tokens > 0xffffffffll || slots <= 0 || slots > 0x7fffffffll)
+    return fail(LLMOPT_ERR_INVALID, "prebaked HIP plan needs two step words and positive limits");
+  if (!plan->single_submission || plan->past_count != 0 || plan->device_checkpoint != nullptr || plan->step_buffer != nullptr)
+    return fail(LLMOPT_ERR_INVALID, "prebaked HIP plan already keeps its own step state");
+  plan->step_buffer = step_words;
+  retain(step_words);
+  plan->past_capacity = (uint32_t)max_past_tokens;
+  plan->checkpoint_limit = (uint32_t)slots - 1;
   return LLMOPT_OK;
 }
 

@@ -92,6 +92,9 @@ def lib() -> ctypes.CDLL:
         "llmopt_hip_f16_argmax": (ctypes.c_int, [vp, i64, ctypes.POINTER(i64)]),
         "llmopt_hip_sample_f16": (ctypes.c_int, [vp, i64, ctypes.c_double, i64, ctypes.c_double, ctypes.c_double,
                                                  i64, ctypes.POINTER(i64)]),
+        "llmopt_hip_f32_argmax": (ctypes.c_int, [vp, i64, ctypes.POINTER(i64)]),
+        "llmopt_hip_sample_f32": (ctypes.c_int, [vp, i64, ctypes.c_double, i64, ctypes.c_double, ctypes.c_double,
+                                                 i64, ctypes.POINTER(i64)]),
         "llmopt_hip_dispatch": (ctypes.c_int, [vp, item_p]),
         "llmopt_hip_begin_batch": (ctypes.c_int, [vp, pp]),
         "llmopt_hip_release_batch": (None, [vp]),
@@ -109,6 +112,7 @@ def lib() -> ctypes.CDLL:
         "llmopt_hip_prebaked_create": (ctypes.c_int, [vp, item_p, sz, vp, vp, pp]),
         "llmopt_hip_release_prebaked": (None, [vp]),
         "llmopt_hip_prebaked_execute": (ctypes.c_int, [vp, i64, i64, i64, ctypes.POINTER(i64)]),
+        "llmopt_hip_prebaked_bind_step": (ctypes.c_int, [vp, vp, i64, i64]),
         "llmopt_hip_prebaked_is_single_submission": (ctypes.c_int, [vp]),
         "llmopt_hip_ring_create": (ctypes.c_int, [pp]),
         "llmopt_hip_ring_submit": (ctypes.c_int, [vp, i64, i64, i64, i64]),
@@ -140,13 +144,13 @@ EXPORTED_SYMBOLS = (
     "llmopt_hip_buffer_contents", "llmopt_hip_buffer_length", "llmopt_hip_buffer_device_pointer",
     "llmopt_hip_buffer_copy", "llmopt_hip_buffer_write", "llmopt_hip_buffer_set_int64",
     "llmopt_hip_buffer_set_u32_array", "llmopt_hip_buffer_argmax_f16", "llmopt_hip_f16_argmax",
-    "llmopt_hip_sample_f16", "llmopt_hip_dispatch",
+    "llmopt_hip_sample_f16", "llmopt_hip_f32_argmax", "llmopt_hip_sample_f32", "llmopt_hip_dispatch",
     "llmopt_hip_begin_batch", "llmopt_hip_release_batch", "llmopt_hip_batch_dispatch",
     "llmopt_hip_batch_dispatch_all", "llmopt_hip_batch_copy", "llmopt_hip_batch_barrier",
     "llmopt_hip_commit_batch", "llmopt_hip_commit_batch_async",
     "llmopt_hip_commit_batch_profiled", "llmopt_hip_commit_batch_profiled_each", "llmopt_hip_abort_batch",
     "llmopt_hip_prebaked_create", "llmopt_hip_release_prebaked", "llmopt_hip_prebaked_execute",
-    "llmopt_hip_prebaked_is_single_submission",
+    "llmopt_hip_prebaked_bind_step", "llmopt_hip_prebaked_is_single_submission",
     "llmopt_hip_ring_create", "llmopt_hip_ring_submit", "llmopt_hip_ring_wait_completion",
     "llmopt_hip_ring_poll_completion", "llmopt_hip_ring_start_worker", "llmopt_hip_ring_start_worker_with",
     "llmopt_hip_ring_destroy",
@@ -380,6 +384,12 @@ class Batch:
         self.kernels.append(name)
         return name
 
+    def dispatch_all(self, dispatches: "DispatchList") -> None:
+        """Records a prepared list (Metal_native.Batch.dispatch_all)."""
+        _check(lib().llmopt_hip_batch_dispatch_all(self._handle, self.runtime.library, dispatches.items,
+                                                   dispatches.count))
+        self.kernels += dispatches.names
+
     def copy(self, source: Buffer, destination: Buffer) -> None:
         _check(lib().llmopt_hip_batch_copy(self._handle, source.handle, destination.handle))
 
@@ -444,6 +454,11 @@ class Prebaked:
                                                  ctypes.byref(out)))
         return int(out.value)
 
+    def bind_step(self, step_words: Buffer, max_past_tokens: int, slots: int) -> None:
+        """Every execute writes its past_tokens and checkpoint into the two u32 words of `step_words`,
+        which the plan's records read as position and state slot."""
+        _check(lib().llmopt_hip_prebaked_bind_step(self._handle, step_words.handle, max_past_tokens, slots))
+
     @property
     def single_submission(self) -> bool:
         """True when a step replays one HIP graph."""
@@ -461,6 +476,17 @@ def _make_items(dispatches):
         items[index] = item
         keep.append(alive)
     return items, len(dispatches), keep
+
+
+class DispatchList:
+    """Dispatches (name, buffers, parameters, grid, group) packed once for repeated recording; holds its
+    buffers."""
+
+    def __init__(self, dispatches: Iterable[tuple]):
+        dispatches = list(dispatches)
+        self.items, self.count, self._keep = _make_items(dispatches)
+        self._buffers = [buffers for _, buffers, _, _, _ in dispatches]
+        self.names = [dispatch[0] for dispatch in dispatches]
 
 
 class Ring:

@@ -15,6 +15,8 @@ import struct
 from dataclasses import dataclass
 from typing import Iterable, Sequence
 
+import numpy as np
+
 from . import native
 
 MAX_INT = (1 << 62) - 1  # OCaml's max_int on a 64-bit host
@@ -168,4 +170,23 @@ def sample(params: Params, vocabulary: int, data: bytes, suppress_token_ids: Ite
     native._check(native.lib().llmopt_hip_sample_f16(ctypes.cast(buffer, ctypes.c_void_p), vocabulary,
                                                      params.temperature, params.top_k, params.top_p, params.min_p,
                                                      params.seed, ctypes.byref(out)))
+    return int(out.value)
+
+
+def sample_f32(params: Params, row, suppress_token_ids: Sequence[int] = ()) -> int:
+    """`sample` over one row of float32 logits (models whose logits are not fp16)."""
+    row = np.array(row, dtype=np.float32).reshape(-1)
+    for token_id in suppress_token_ids:
+        if not 0 <= token_id < len(row):
+            raise SamplingError(f"suppressed token id {token_id} is outside vocabulary [0,{len(row)})")
+        row[token_id] = -np.inf
+    if len(set(suppress_token_ids)) >= len(row):
+        raise SamplingError("cannot suppress the complete sampling vocabulary")
+    out = ctypes.c_int64(0)
+    pointer = row.ctypes.data_as(ctypes.c_void_p)
+    if params.is_greedy():
+        native._check(native.lib().llmopt_hip_f32_argmax(pointer, len(row), ctypes.byref(out)))
+    else:
+        native._check(native.lib().llmopt_hip_sample_f32(pointer, len(row), params.temperature, params.top_k,
+                                                         params.top_p, params.min_p, params.seed, ctypes.byref(out)))
     return int(out.value)
