@@ -629,6 +629,167 @@ def bench_prefill(runtime, lengths=(512, 2048)):
     return results
 
 
+# Layered decoders (llmopt_amd.layered_model) at the sizes of real models' layers, two layers of each kind, and
+# the W4A16 transformer with the same hidden size, heads, feed-forward and layer count beside them.
+LAYERED_SIZES = {
+    "1024": dict(width=1024, heads=16, kv_heads=4, dim=64, chunk=2048, ssm_heads=32, state=128, ff=4096,
+                 experts=32, top=4, expert_ff=512, shared_ff=1024),
+    "2048": dict(width=2048, heads=32, kv_heads=8, dim=128, chunk=2048, ssm_heads=64, state=128, ff=8192,
+                 experts=64, top=8, expert_ff=1024, shared_ff=1024),
+    "4096": dict(width=4096, heads=32, kv_heads=8, dim=128, chunk=8192, ssm_heads=128, state=128, ff=14336,
+                 experts=16, top=4, expert_ff=2048, shared_ff=4096),
+}
+LAYERED_VOCABULARY = 32768
+
+
+def layered_config(size):
+    z = LAYERED_SIZES[size]
+    mamba = {"type": "mamba2", "mlp": {"kind": "dense", "ff": z["ff"]},
+             "mixer": {"heads": z["ssm_heads"], "vdim": 64, "state": z["state"], "groups": 1, "conv": 4,
+                       "norm_groups": 1}}
+    attention = {"type": "attention",
+                 "mlp": {"kind": "moe", "router": {"experts": z["experts"], "top": z["top"]},
+                         "expert": {"ff": z["expert_ff"]}, "shared": {"ff": z["shared_ff"]}},
+                 "mixer": {"heads": z["heads"], "kv_heads": z["kv_heads"], "dim": z["dim"], "vdim": z["dim"],
+                           "scale": z["dim"] ** -0.5, "softcap": 30.0, "v_mix": True, "mask": {"size": z["chunk"]}}}
+    return {"architecture": "Barovik", "vocab": LAYERED_VOCABULARY, "width": z["width"], "norm": {"eps": 1e-6},
+            "embedding": {"scale": 1.0}, "layers": [mamba, attention] * 2}
+
+
+class TiledWeights:
+    """Weights of any shape from one block of random values (making gigabytes of them would take minutes)."""
+
+    def __init__(self, shapes, rng):
+        from llmopt_amd.safetensors_file import to_bfloat16
+        self.shapes, self.block = shapes, rng.standard_normal((1 << 20) + 7).astype(np.float32)
+        self.convert = to_bfloat16
+
+    def __contains__(self, name):
+        return name in self.shapes
+
+    def __getitem__(self, name):
+        shape = self.shapes[name]
+        kind = name.rsplit(".", 1)[-1]
+        if "norm" in kind:
+            return self.convert(np.ones(shape))
+        gain = 0.5 if kind in ("A_log", "dt_bias", "D", "b", "sink", "conv", "embed") or not shape else shape[-1] ** -0.5
+        return np.resize(self.convert(self.block * np.float32(gain)), shape)
+
+
+def layered_work(model, m, context):
+    """Algorithmic flops of the products of a prefill of m tokens, and the bytes one decode step reads and
+    writes: weights it uses, keys and values of the chunk, recurrent state."""
+    from llmopt_amd.layered_model import AttentionMixer, DenseFfn
+    c, flops, weights, state = model.config, 0.0, 0, 0
+    for layer in c.layers:
+        x, f = layer.mixer, layer.ffn
+        if isinstance(x, AttentionMixer):
+            columns, inner = x.columns, x.heads * x.vdim
+            chunk = x.chunk or m
+            keys = sum(n * (n + 1) / 2 for n in [chunk] * (m // chunk) + [m % chunk])
+            flops += 2.0 * x.heads * (x.dim + x.vdim) * keys
+            state += 2 * x.kv_heads * (x.dim + x.vdim) * (context % chunk + 1)
+        else:
+            columns, inner = x.columns, x.inner
+            flops += m * (4.0 * x.inner * x.state + 2.0 * 64 * (x.inner + x.groups * x.state))
+            state += 8 * x.inner * x.state
+        flops += 2.0 * m * c.width * (columns + inner)
+        weights += 2 * c.width * (columns + inner)
+        used = f.ff if isinstance(f, DenseFfn) else f.top * f.ff + f.shared_ff
+        router = 0 if isinstance(f, DenseFfn) else f.experts + 1
+        flops += 2.0 * m * c.width * (3 * used + router)
+        weights += 2 * c.width * (3 * used + router)
+    return flops, weights + 2 * c.width * c.vocabulary + state
+
+
+def bench_layered(runtime, sizes, prompts=(512, 2048, 8192), context=2000):
+    """Prefill (one portion, logits of its last token) and decode (one token after `context`, a HIP graph) of
+    the layered decoders, and the same of the W4A16 transformer.  Medians of graph replays, in turn."""
+    from llmopt_amd.decode_step import DecodeConfig, DecodeStep, random_w4
+    from llmopt_amd.layered_model import LayeredConfig, LayeredModel
+    from llmopt_amd.native import DispatchList
+    from llmopt_amd.prefill_step import PrefillStep
+    rng = np.random.default_rng(SEED + 11)
+    median = lambda values: sorted(values)[len(values) // 2]
+    results = []
+    for size in sizes:
+        z = LAYERED_SIZES[size]
+        print("layered", size, file=sys.stderr, flush=True)
+        config = LayeredConfig.parse(layered_config(size))
+        model = LayeredModel(runtime, config, TiledWeights(config.tensor_shapes(), rng), slots=2, max_context=16384)
+        other = DecodeConfig(hidden=z["width"], q_heads=z["heads"], kv_heads=z["kv_heads"], head_dim=z["dim"],
+                             mlp=z["ff"], layers=len(config.layers), vocabulary=LAYERED_VOCABULARY, epsilon=1e-6)
+        h, kv = other.hidden, other.kv_heads * other.head_dim
+        layer = {"attn_norm": np.ones(h, np.float16), "ffn_norm": np.ones(h, np.float16),
+                 "q": random_w4(rng, other.q_heads * other.head_dim, h), "k": random_w4(rng, kv, h),
+                 "v": random_w4(rng, kv, h), "o": random_w4(rng, h, other.q_heads * other.head_dim),
+                 "gate": random_w4(rng, other.mlp, h), "up": random_w4(rng, other.mlp, h),
+                 "down": random_w4(rng, h, other.mlp)}
+        weights = {"embedding": (rng.standard_normal((1024, h)) * 0.5).astype(np.float16).repeat(32, axis=0),
+                   "layers": [layer] * other.layers, "final_norm": np.ones(h, np.float16),
+                   "lm_head": random_w4(rng, other.vocabulary, h)}
+        entry = {"width": z["width"], "layers": len(config.layers), "prefill": [], "decode": {}}
+        device_weights = None
+        for m in prompts:
+            tokens = rng.integers(0, LAYERED_VOCABULARY, m)
+            sequence = model.open()
+            logits = model.step(sequence, tokens, [m - 1])
+            model.close(sequence)
+            graph = runtime.begin_batch()
+            graph.dispatch_all(model._lists[m])
+            index = runtime.buffer_of_bytes(np.array([m - 1], np.uint32))
+            out = runtime.create_buffer(LAYERED_VOCABULARY * 4)
+            graph.dispatch_all(DispatchList([model._logits(1, m, model._work, index, out)]))
+            ms = median(graph.commit_profiled_each(repeats=5))
+            flops, _ = layered_work(model, m, context)
+            pool = runtime.create_buffer((m + 1) * other.token_stride)
+            step = PrefillStep(runtime, other, weights, m, pool, runtime.buffer_of_bytes(np.arange(m + 1, dtype=np.uint32)),
+                               device_weights=device_weights)
+            device_weights = step.device
+            step.run(tokens)
+            graph = runtime.begin_batch()
+            step.record(graph)
+            other_ms = median(graph.commit_profiled_each(repeats=5))
+            entry["prefill"].append({
+                "tokens": m, "ms": round(ms, 4), "tokens_per_s": round(m / ms * 1e3), "finite": bool(np.isfinite(logits).all()),
+                "TFLOPs": round(flops / ms / 1e9, 1), "mfma_frac": round(flops / ms / 1e9 / MFMA_F16_PEAK_TFLOPS, 4),
+                "w4a16": {"ms": round(other_ms, 4), "tokens_per_s": round(m / other_ms * 1e3),
+                          "TFLOPs": round(step.flops() / other_ms / 1e9, 1),
+                          "mfma_frac": round(step.flops() / other_ms / 1e9 / MFMA_F16_PEAK_TFLOPS, 4)}})
+            del step, pool
+        sequence = model.open()
+        model.step(sequence, rng.integers(0, LAYERED_VOCABULARY, context))
+        plan = model.decode_plan()
+        plan.execute(1, sequence)  # leaves the step words of a token behind the context
+        graph = runtime.begin_batch()
+        graph.dispatch_all(DispatchList(plan.dispatches))
+        ms = median(graph.commit_profiled_each(repeats=9))
+        started = time.perf_counter()
+        for _ in range(20):
+            plan.execute(1, sequence)
+        wall = (time.perf_counter() - started) / 20 * 1e3
+        model.close(sequence)
+        _, step_bytes = layered_work(model, 1, context)
+        slots = np.arange(context + 64, dtype=np.uint32)
+        step = DecodeStep(runtime, other, weights, 1, runtime.create_buffer(len(slots) * other.token_stride),
+                          runtime.buffer_of_bytes(slots), [0], [context], [context], [context], slots_host=slots)
+        step.run([1])
+        graph = runtime.begin_batch()
+        step.record(graph)
+        other_ms = median(graph.commit_profiled_each(repeats=9))
+        other_bytes = step.weight_bytes() + step.kv_bytes()
+        entry["decode"] = {
+            "context": context, "ms": round(ms, 4), "tokens_per_s": round(1e3 / ms, 1), "plan_wall_ms": round(wall, 4),
+            "bytes": int(step_bytes), "GBps": round(step_bytes / ms / 1e6, 1),
+            "hbm_frac": round(step_bytes / ms / 1e6 / HBM_PEAK_GBS, 4), "records": len(plan.dispatches),
+            "w4a16": {"ms": round(other_ms, 4), "tokens_per_s": round(1e3 / other_ms, 1), "bytes": int(other_bytes),
+                      "GBps": round(other_bytes / other_ms / 1e6, 1),
+                      "hbm_frac": round(other_bytes / other_ms / 1e6 / HBM_PEAK_GBS, 4), "records": len(step.dispatches)}}
+        results.append(entry)
+        del model, step, plan, graph, device_weights
+    return results
+
+
 PMC_LAUNCHES_PER_CASE = 8
 
 
@@ -781,6 +942,10 @@ def main():
     parser.add_argument("--serial-only", action="store_true",
                         help="leave out the concurrent-branch graphs and the warm (cached) per-case loops: every "
                              "launch of the run then is a serial, cold one (for kernel traces)")
+    parser.add_argument("--layered", nargs="?", const=",".join(LAYERED_SIZES), metavar="SIZES",
+                        help="only the layered decoders beside the W4A16 transformer, at these widths (default: "
+                             + ",".join(LAYERED_SIZES) + ")")
+    parser.add_argument("--layered-prompts", default="512,2048,8192", help="prompt lengths of --layered")
     parser.add_argument("--pmc-probe", action="store_true",
                         help="only the calibration copies and the cases of the GEMV sweep, for rocprofv3 --pmc")
     args = parser.parse_args()
@@ -791,6 +956,11 @@ def main():
     runtime = Runtime()
     if args.pmc_probe:
         print(json.dumps(pmc_probe(runtime)))
+        runtime.close()
+        return
+    if args.layered:
+        print(json.dumps({"layered": bench_layered(runtime, args.layered.split(","),
+                                                   tuple(int(m) for m in args.layered_prompts.split(",")))}))
         runtime.close()
         return
     gemv = bench_gemv(runtime, args.steps, args.warmup, serial_only=args.serial_only)

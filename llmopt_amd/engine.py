@@ -14,6 +14,15 @@ from typing import Optional, Sequence
 from . import sampling
 
 
+def _scatter(seed: int, index: int) -> int:
+    """The index-th output of the splitmix64 generator started at `seed`, as a positive 63-bit integer."""
+    mask = (1 << 64) - 1
+    z = (seed + (index + 1) * 0x9E3779B97F4A7C15) & mask
+    z = ((z ^ (z >> 30)) * 0xBF58476D1CE4E5B9) & mask
+    z = ((z ^ (z >> 27)) * 0x94D049BB133111EB) & mask
+    return ((z ^ (z >> 31)) >> 1) or 1
+
+
 @dataclass
 class Request:
     id: int
@@ -101,9 +110,10 @@ class Engine:
 
     @staticmethod
     def _step_params(request: Request) -> sampling.Params:
-        """A seed gives one sequence of draws: every token its own (0 stays 0, the clock)."""
+        """A seed gives one sequence of draws: every token a seed of its own, scattered (the sampler's
+        generator gives neighbouring seeds neighbouring first draws); 0 stays 0, the clock."""
         p = request.params
-        seed = p.seed + len(request.tokens) if p.seed else 0
+        seed = _scatter(p.seed, len(request.tokens)) if p.seed else 0
         return sampling.Params(p.temperature, p.top_k, p.top_p, p.min_p, seed)
 
     @staticmethod

@@ -7,7 +7,7 @@ import pytest
 
 from llmopt_amd.engine import Engine
 from oracle import hybrid_model
-from tests.layered_util import (TOLERANCE, attention, config, dense, expected_logits, make_model, make_weights, mamba2,
+from tests.layered_util import (assert_close, attention, config, dense, expected_logits, make_model, make_weights, mamba2,
                                 moe, relative, run_portions)
 
 pytestmark = pytest.mark.gpu
@@ -62,12 +62,12 @@ def check_streams(runtime, cfg, dtype, count=75, seed=0, change=None):
     logits = model.step(sequence, tokens, range(count), streams=got)
     model.close(sequence)
     for index, stream in enumerate(got):
-        assert relative(stream, streams[index]) < TOLERANCE[dtype], f"prompt, layer {index}"
-    assert relative(logits, expected) < TOLERANCE[dtype]
+        assert_close(stream, streams[index], dtype, f"prompt, layer {index}")
+    assert_close(logits, expected, dtype)
     sequence = model.open()
     decoded = np.concatenate([model.step(sequence, [t], [0]) for t in tokens])
     model.close(sequence)
-    assert relative(decoded, expected) < TOLERANCE[dtype], "token by token"
+    assert_close(decoded, expected, dtype, "token by token")
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
@@ -113,22 +113,32 @@ def test_value_mix_of_several_layers(runtime, dtype):
     check_streams(runtime, cfg, dtype, change=lambda name, values: lambdas.get(name))
 
 
-@pytest.fixture(scope="module")
-def mixed():
-    cfg = config(mamba2(mlp=dense()), attention(chunk=24, mlp=moe()), mamba2(vdim=10, mlp=moe(shared=0)),
+def mixed_model(top):
+    cfg = config(mamba2(mlp=dense()), attention(chunk=24, mlp=moe(top=top)), mamba2(vdim=10, mlp=moe(top=top, shared=0)),
                  attention(chunk=17, heads=3, mlp=dense()))
     patterns, weights = make_weights(cfg, 5)
     tokens = tokens_of(5, 210)
     return cfg, patterns, weights, tokens, expected_logits(cfg, weights, tokens)
 
 
+@pytest.fixture(scope="module")
+def mixed():
+    return mixed_model(top=2)
+
+
+@pytest.fixture(scope="module")
+def mixed_all():
+    """Every expert is chosen: no close call for bfloat16 to decide the other way."""
+    return mixed_model(top=6)
+
+
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("portions", [[210], [2], [3, 64], [1], [24], [17, 1, 2], [100, 1, 1, 9], [65, 63, 2]])
-def test_portions(runtime, mixed, portions, dtype):
-    cfg, patterns, _, tokens, expected = mixed
+def test_portions(runtime, mixed, mixed_all, portions, dtype):
+    cfg, patterns, _, tokens, expected = mixed if dtype == "float32" else mixed_all
     print(portions, dtype, flush=True)
     model = make_model(runtime, cfg, patterns, dtype)
-    assert relative(run_portions(model, tokens, portions), expected) < TOLERANCE[dtype]
+    assert_close(run_portions(model, tokens, portions), expected, dtype)
 
 
 def test_slots_are_reused_and_do_not_leak(runtime, mixed):
@@ -145,7 +155,7 @@ def test_slots_are_reused_and_do_not_leak(runtime, mixed):
         sequence, at = live[index]
         count = min(int(rng.integers(1, 30)), len(prompts[index]) - at)
         logits = model.step(sequence, prompts[index][at:at + count], range(count))
-        assert relative(logits, expected[index][at:at + count]) < TOLERANCE["float32"], (index, at, count)
+        assert_close(logits, expected[index][at:at + count], "float32", (index, at, count))
         live[index][1] += count
         if live[index][1] == len(prompts[index]):
             model.close(sequence)
@@ -196,14 +206,14 @@ def test_chunk_edges(runtime, chunk, dtype):
         print(chunk, place, dtype, flush=True)
         for portions in ([3 * chunk], [chunk - 1, 2], [chunk + 1, 1, 3], [1]):
             got = run_portions(model, tokens, portions)
-            assert relative(got, expected) < TOLERANCE[dtype], (place, portions)
+            assert_close(got, expected, dtype, (place, portions))
     # the comparison would notice a border that is one token off
     tokens = filler.copy()
     tokens[chunk - 1], tokens[chunk] = 1, 0
     for wrong in (chunk - 1, chunk + 1):
         shifted["layers"][0]["mixer"]["mask"]["size"] = wrong
         off = expected_logits(shifted, weights, tokens.tolist())
-        assert relative(off, expected_logits(cfg, weights, tokens.tolist())) > 10 * TOLERANCE["bfloat16"]
+        assert relative(off, expected_logits(cfg, weights, tokens.tolist())) > 0.3
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
@@ -218,10 +228,10 @@ def test_far_key_and_sink_over_many_splits(runtime, dtype):
         tokens[[6, 127, 128, 255, 256, 300, 383, 389]] = 0
         expected = expected_logits(cfg, weights, tokens.tolist())
         for portions in ([390], [383, 1], [120, 1, 1, 1, 1, 1, 1, 1, 1, 1, 1]):
-            assert relative(run_portions(model, tokens.tolist(), portions), expected) < TOLERANCE[dtype], (sink, portions)
+            assert_close(run_portions(model, tokens.tolist(), portions), expected, dtype, (sink, portions))
         without = {**weights, "l0.mix.sink": np.full(2, -30.0)}
         if sink > 0:
-            assert relative(expected_logits(cfg, without, tokens.tolist()), expected) > 10 * TOLERANCE["bfloat16"]
+            assert relative(expected_logits(cfg, without, tokens.tolist()), expected) > 0.3
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
@@ -244,15 +254,15 @@ def test_long_memory_of_the_recurrence(runtime, dtype):
     expected = expected_logits(cfg, weights, tokens)
     for portions in ([300], [70, 1, 1], [2], [1]):
         print(portions, dtype, flush=True)
-        assert relative(run_portions(model, tokens, portions), expected) < TOLERANCE[dtype], portions
+        assert_close(run_portions(model, tokens, portions), expected, dtype, portions)
 
 
 def test_first_tokens(runtime, mixed):
     cfg, patterns, _, tokens, expected = mixed
     model = make_model(runtime, cfg, patterns, "float32")
     for count in (1, 2, 3, 4, 5):
-        assert relative(run_portions(model, tokens[:count], [count]), expected[:count]) < TOLERANCE["float32"]
-        assert relative(run_portions(model, tokens[:count], [1]), expected[:count]) < TOLERANCE["float32"]
+        assert_close(run_portions(model, tokens[:count], [count]), expected[:count], "float32")
+        assert_close(run_portions(model, tokens[:count], [1]), expected[:count], "float32")
 
 
 def greedy(cfg, weights, prompt, count):
@@ -288,7 +298,7 @@ def test_generation_with_other_settings(runtime, mixed):
 def test_a_plan_replays_like_eager_steps(runtime, mixed):
     """The captured graph, many times, with other work on the stream in between."""
     cfg, patterns, _, tokens, expected = mixed
-    model = make_model(runtime, cfg, patterns, "bfloat16")
+    model = make_model(runtime, cfg, patterns, "float32")
     one, two = model.open(), model.open()
     at = {0: 0, 1: 0}
     for turn in range(60):
@@ -297,7 +307,7 @@ def test_a_plan_replays_like_eager_steps(runtime, mixed):
         count = 1 if turn % 5 else 3
         part = tokens[at[which]:at[which] + count]
         got = model.step(sequence, part, range(count))
-        assert relative(got, expected[at[which]:at[which] + count]) < TOLERANCE["bfloat16"], turn
+        assert_close(got, expected[at[which]:at[which] + count], "float32", turn)
         at[which] += count
     assert model.decode_plan().plan.single_submission
 
@@ -351,8 +361,8 @@ def test_command_line(runtime, mixed, tmp_path, capsys, monkeypatch):
                      "--max-tokens", "64"]) == 0
     assert capsys.readouterr().out.split("\n")[:3] == ["done 0", "done 1", "done 2"]
     read = lambda n, rows: np.fromfile(out / f"{n}.f32", dtype="<f4").reshape(rows, -1)
-    assert relative(read(0, 2), expected[[3, 19]]) < TOLERANCE["float32"]
-    assert relative(read(1, 1), expected[[20]]) < TOLERANCE["float32"]
+    assert_close(read(0, 2), expected[[3, 19]], "float32")
+    assert_close(read(1, 1), expected[[20]], "float32")
     assert not (out / "2.f32").exists()
 
 
@@ -371,5 +381,5 @@ def test_sizes_of_a_real_layer(runtime, dtype):
     # the recurrence alone is slow to restate at this size: the first layer over all tokens is enough for both
     expected, streams = hybrid_model.forward(cfg, weights, tokens)
     for index in range(2):
-        assert relative(got[index], streams[index]) < TOLERANCE[dtype], index
-    assert relative(logits, expected[[0, 1, 255, 256, 329]]) < TOLERANCE[dtype]
+        assert_close(got[index], streams[index], dtype, index)
+    assert_close(logits, expected[[0, 1, 255, 256, 329]], dtype)
