@@ -40,6 +40,7 @@ COMMON = ["-O3", "-std=c++17", "-fPIC", "--offload-arch=gfx950",
 PER_FILE = {
     "dense_attention.hip": ["-mllvm", "-amdgpu-mfma-vgpr-form=1"],
     "q8_attention.hip": ["-mllvm", "-amdgpu-mfma-vgpr-form=1"],
+    "chunk_attention.hip": ["-mllvm", "-amdgpu-mfma-vgpr-form=1"],
 }
 
 

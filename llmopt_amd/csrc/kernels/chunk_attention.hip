@@ -27,6 +27,7 @@ namespace {
 constexpr int kStageKeys = 64;
 constexpr uint32_t kSplitKeys = 128;
 constexpr float kFixedMaxCap = 40.0f;
+constexpr float kLog2e = 1.4426950408889634f;
 
 __device__ __forceinline__ uint32_t chunk_start(uint32_t position, uint32_t chunk) {
   return chunk ? position - position % chunk : 0;
@@ -37,18 +38,48 @@ __device__ __forceinline__ float capped(float s, float scale, float cap, float i
   return cap > 0.0f ? cap * tanh_f32(s * inverse_cap) : s;
 }
 
-template <typename T, int ND, int NE, int QT>
-__global__ __launch_bounds__(256) void chunk_prefill_kernel(ChunkAttentionArgs a) {
+// Values of four keys (rows of the stage) at the lane's column: what the V^T operand takes.  bf16: the
+// transposing LDS read - in a group of 16 lanes, lane 4 q + c receives element c of the 8-byte pieces named
+// by lanes q, 4 + q, 8 + q and 12 + q, so lane 4 e + q names (key e, columns 4 q ..).
+typedef short s16x4 __attribute__((ext_vector_type(4)));
+typedef __attribute__((address_space(3))) s16x4 *lds_piece_t;
+__device__ __forceinline__ bf16x4 four_keys(const __bf16 *stage, int stride, int lane) {
+  const __bf16 *piece = stage + ((lane & 15) >> 2) * stride + (lane & 3) * 4;
+  return __builtin_bit_cast(bf16x4, __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_piece_t)piece));
+}
+__device__ __forceinline__ f32x4 four_keys(const float *stage, int stride, int lane) {
+  f32x4 v;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) v[i] = stage[i * stride + (lane & 15)];
+  return v;
+}
+
+__device__ __forceinline__ float exp2_raw(float x) { return __builtin_amdgcn_exp2f(x); }
+
+template <typename T, int NE>
+constexpr int value_stride() { return NE * 16 + 32 / (int)sizeof(T); }
+
+template <typename T, int ND, int NE>
+constexpr int prefill_lds_bytes() {
+  return kStageKeys * (ND * 32 + 16 / (int)sizeof(T) + value_stride<T, NE>()) * (int)sizeof(T);
+}
+
+template <typename T, int ND, int NE, int QT, bool FIXED>
+__global__ __launch_bounds__(256, ND * 2 + NE <= 16 || sizeof(T) == 2 ? 2 : 1) void chunk_prefill_kernel(ChunkAttentionArgs a) {
   constexpr int DP = ND * 32, EP = NE * 16;
-  constexpr int PAD = 16 / (int)sizeof(T);
-  constexpr int SK = DP + PAD, SV = kStageKeys + PAD;
+  constexpr int SK = DP + 16 / (int)sizeof(T), SV = value_stride<T, NE>();
+  constexpr int K_LOADS = kStageKeys * DP / 8 / 256, V_PIECES = EP / 8;
+  constexpr int V_LOADS = (kStageKeys * V_PIECES + 255) / 256;
   extern __shared__ __attribute__((aligned(16))) char lds[];
   T *lds_k = reinterpret_cast<T *>(lds);
-  T *lds_v = lds_k + kStageKeys * SK;  // [EP][SV], transposed
+  T *lds_v = lds_k + kStageKeys * SK;
 
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, column = lane & 15, quad = lane >> 4;
-  const uint32_t head = blockIdx.y, group = head / (a.heads / a.kv_heads);
-  const uint32_t tile = gridDim.x - 1 - blockIdx.x;  // longest rows first
+  // heads of one key / value head follow each other kv_heads apart, so that they share an XCD's L2 when
+  // kv_heads is a multiple of the eight XCDs; the longest rows of all heads come first
+  const uint32_t per = a.heads / a.kv_heads, group = blockIdx.x % a.kv_heads;
+  const uint32_t head = group * per + blockIdx.x / a.kv_heads;
+  const uint32_t tile = gridDim.y - 1 - blockIdx.y;
   const uint32_t p0 = a.state[kStatePosition], slot = a.state[kStateSlot];
   const uint32_t row_first = tile * 64 * QT;
   const uint32_t row_end = min(row_first + 64 * QT, a.m);
@@ -75,18 +106,22 @@ __global__ __launch_bounds__(256) void chunk_prefill_kernel(ChunkAttentionArgs a
       fq[t][d] = load_piece(qkv + (size_t)r * ld + head * a.dim + k, (int)a.dim - k, vec);
     }
   }
+  const uint32_t wave_first = p0 + min(row_first + wave * QT * 16, a.m - 1);
   const uint32_t wave_last = p0 + min(row_first + (wave + 1) * QT * 16 - 1, a.m - 1);
-  const uint32_t wave_low = chunk_start(p0 + min(row_first + wave * QT * 16, a.m - 1), a.cache.chunk);
+  const uint32_t wave_low = chunk_start(wave_first, a.cache.chunk);
+  const uint32_t wave_low_last = chunk_start(wave_last, a.cache.chunk);
 
-  const bool has_sink = a.sink != nullptr;
-  const float sink = has_sink ? (float)reinterpret_cast<const __bf16 *>(a.sink)[head] : 0.0f;
-  const bool fixed = a.softcap > 0.0f && a.softcap <= kFixedMaxCap;
-  const float inverse_cap = a.softcap > 0.0f ? 1.0f / a.softcap : 0.0f;
+  // Exponents are taken to base two.  capped: score = cap tanh(scale s / cap), with
+  // tanh z = 1 - 2 / (1 + e^(2 z)); fixed: the cap bounds it, and the maximum is a constant.
+  const bool has_sink = a.sink != nullptr, capped = a.softcap > 0.0f;
+  const float sink = has_sink ? (float)reinterpret_cast<const __bf16 *>(a.sink)[head] * kLog2e : 0.0f;
+  const float cap = a.softcap * kLog2e;
+  const float inner = capped ? 2.0f * a.scale / a.softcap * kLog2e : a.scale * kLog2e;
   float top[QT], total[QT];
 #pragma unroll
   for (int t = 0; t < QT; ++t) {
-    top[t] = has_sink ? (fixed ? fmaxf(sink, 0.0f) : sink) : (fixed ? 0.0f : -1e30f);
-    total[t] = has_sink && quad == 0 ? __expf(sink - top[t]) : 0.0f;
+    top[t] = has_sink ? (FIXED ? fmaxf(sink, 0.0f) : sink) : (FIXED ? 0.0f : -1e30f);
+    total[t] = has_sink && quad == 0 ? exp2_raw(sink - top[t]) : 0.0f;
   }
   f32x4 out[NE][QT];
 #pragma unroll
@@ -96,34 +131,45 @@ __global__ __launch_bounds__(256) void chunk_prefill_kernel(ChunkAttentionArgs a
 
   const uint32_t last = p0 + row_end - 1;
   const uint32_t key_begin = chunk_start(p0 + row_first, a.cache.chunk);
-  for (uint32_t base = key_begin; base <= last; base += kStageKeys) {
-    __syncthreads();
+
+  // a stage travels global -> registers while the one before it is multiplied
+  Frag<T> reg_k[K_LOADS], reg_v[V_LOADS];
+  auto fetch = [&](uint32_t base) {
 #pragma unroll
-    for (int i = 0; i < ND; ++i) {
-      const int index = i * 256 + tid, row = index / (ND * 4), piece = (index % (ND * 4)) * 8;
+    for (int i = 0; i < K_LOADS; ++i) {
+      const int index = i * 256 + tid, row = index / (DP / 8), piece = (index % (DP / 8)) * 8;
       const uint32_t j = min(base + row, last);
       const T *source = j < p0 ? cache_k + (size_t)(j % a.cache.capacity) * a.dim : fresh_k + (size_t)(j - p0) * ld;
-      *reinterpret_cast<Frag<T> *>(lds_k + row * SK + piece) = load_piece(source + piece, (int)a.dim - piece, vec);
+      reg_k[i] = load_piece(source + piece, (int)a.dim - piece, vec);
     }
 #pragma unroll
-    for (int i = 0; i < (NE + 3) / 4; ++i) {
-      const int index = i * 256 + tid, pair = index & 31, piece = (index >> 5) * 8;
-      if (piece < EP) {
-        Frag<T> two[2];
-#pragma unroll
-        for (int h = 0; h < 2; ++h) {
-          const uint32_t j = min(base + pair * 2 + h, last);
-          const T *source =
-              j < p0 ? cache_v + (size_t)(j % a.cache.capacity) * a.vdim : fresh_v + (size_t)(j - p0) * ld;
-          two[h] = load_piece(source + piece, (int)a.vdim - piece, vec);
-        }
-        typedef T x2 __attribute__((ext_vector_type(2)));
-#pragma unroll
-        for (int e = 0; e < 8; ++e)
-          *reinterpret_cast<x2 *>(lds_v + (piece + e) * SV + pair * 2) = x2{two[0][e], two[1][e]};
-      }
+    for (int i = 0; i < V_LOADS; ++i) {
+      const int index = i * 256 + tid, row = min(index / V_PIECES, kStageKeys - 1), piece = (index % V_PIECES) * 8;
+      const uint32_t j = min(base + row, last);
+      const T *source = j < p0 ? cache_v + (size_t)(j % a.cache.capacity) * a.vdim : fresh_v + (size_t)(j - p0) * ld;
+      reg_v[i] = load_piece(source + piece, (int)a.vdim - piece, vec);
     }
+  };
+  auto stash = [&] {
+#pragma unroll
+    for (int i = 0; i < K_LOADS; ++i) {
+      const int index = i * 256 + tid;
+      *reinterpret_cast<Frag<T> *>(lds_k + index / (DP / 8) * SK + (index % (DP / 8)) * 8) = reg_k[i];
+    }
+#pragma unroll
+    for (int i = 0; i < V_LOADS; ++i) {
+      const int index = i * 256 + tid;
+      if (index < kStageKeys * V_PIECES)
+        *reinterpret_cast<Frag<T> *>(lds_v + index / V_PIECES * SV + (index % V_PIECES) * 8) = reg_v[i];
+    }
+  };
+
+  fetch(key_begin);
+  for (uint32_t base = key_begin; base <= last; base += kStageKeys) {
     __syncthreads();
+    stash();
+    __syncthreads();
+    if (base + kStageKeys <= last) fetch(base + kStageKeys);
     if (base > wave_last || base + kStageKeys <= wave_low) continue;
 
     f32x4 score[4][QT];
@@ -137,39 +183,67 @@ __global__ __launch_bounds__(256) void chunk_prefill_kernel(ChunkAttentionArgs a
 #pragma unroll
         for (int t = 0; t < QT; ++t) score[kt][t] = mma(fk, fq[t][d], score[kt][t]);
       }
+      __builtin_amdgcn_sched_barrier(0);  // operands of one key tile at a time: registers
     }
+    const bool whole = base >= wave_low_last && base + kStageKeys - 1 <= wave_first;  // no border in this stage
+    auto seen = [&](int t, int kt, int r) {
+      const uint32_t j = base + kt * 16 + quad * 4 + r;
+      return j >= low[t] && j <= query[t];
+    };
+    if (FIXED) {
 #pragma unroll
-    for (int t = 0; t < QT; ++t) {
-      float best = top[t];
+      for (int t = 0; t < QT; ++t) {
+        const float high = cap - top[t];
 #pragma unroll
-      for (int kt = 0; kt < 4; ++kt)
+        for (int kt = 0; kt < 4; ++kt)
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          const uint32_t j = base + kt * 16 + quad * 4 + r;
-          const bool seen = j >= low[t] && j <= query[t];
-          const float s = seen ? capped(score[kt][t][r], a.scale, a.softcap, inverse_cap) : -INFINITY;
-          score[kt][t][r] = s;
-          if (!fixed) best = fmaxf(best, s);
+          for (int r = 0; r < 4; ++r) {
+            const float tail = __builtin_amdgcn_rcpf(1.0f + exp2_raw(score[kt][t][r] * inner));
+            score[kt][t][r] = exp2_raw(fmaf(-2.0f * cap, tail, high));
+          }
+        if (!whole) {
+#pragma unroll
+          for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+            for (int r = 0; r < 4; ++r)
+              if (!seen(t, kt, r)) score[kt][t][r] = 0.0f;
         }
-      if (!fixed) {
+#pragma unroll
+        for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) total[t] += score[kt][t][r];
+      }
+    } else {
+#pragma unroll
+      for (int t = 0; t < QT; ++t) {
+        float best = top[t];
+#pragma unroll
+        for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) {
+            float s = score[kt][t][r] * inner;
+            if (capped) s = fmaf(-2.0f * cap, __builtin_amdgcn_rcpf(1.0f + exp2_raw(s)), cap);
+            if (!whole && !seen(t, kt, r)) s = -INFINITY;
+            score[kt][t][r] = s;
+            best = fmaxf(best, s);
+          }
         best = fmaxf(best, __shfl_xor(best, 16, 64));
         best = fmaxf(best, __shfl_xor(best, 32, 64));
-        const float alpha = __expf(top[t] - best);
+        const float alpha = exp2_raw(top[t] - best);
         top[t] = best;
         total[t] *= alpha;
 #pragma unroll
         for (int e = 0; e < NE; ++e)
 #pragma unroll
           for (int r = 0; r < 4; ++r) out[e][t][r] *= alpha;
+#pragma unroll
+        for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) {
+            score[kt][t][r] = exp2_raw(score[kt][t][r] - best);
+            total[t] += score[kt][t][r];
+          }
       }
-#pragma unroll
-      for (int kt = 0; kt < 4; ++kt)
-#pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          const float p = __expf(score[kt][t][r] - top[t]);
-          score[kt][t][r] = p;
-          total[t] += p;
-        }
     }
 #pragma unroll
     for (int ks = 0; ks < 2; ++ks) {
@@ -183,12 +257,12 @@ __global__ __launch_bounds__(256) void chunk_prefill_kernel(ChunkAttentionArgs a
         }
 #pragma unroll
       for (int e = 0; e < NE; ++e) {
-        typedef T x4 __attribute__((ext_vector_type(4)));
-        const T *row = lds_v + (e * 16 + column) * SV + ks * 32 + quad * 4;
-        const x4 first = *reinterpret_cast<const x4 *>(row), second = *reinterpret_cast<const x4 *>(row + 16);
+        const T *keys = lds_v + (ks * 32 + quad * 4) * SV + e * 16;
+        const auto first = four_keys(keys, SV, lane), second = four_keys(keys + 16 * SV, SV, lane);
         const Frag<T> fv = __builtin_shufflevector(first, second, 0, 1, 2, 3, 4, 5, 6, 7);
 #pragma unroll
         for (int t = 0; t < QT; ++t) out[e][t] = mma(fv, fp[t], out[e][t]);
+        if (e % 4 == 3) __builtin_amdgcn_sched_barrier(0);
       }
     }
   }
@@ -237,8 +311,13 @@ __global__ __launch_bounds__(256) void chunk_cache_write_kernel(ChunkAttentionAr
   }
 }
 
-// PIECES: 64-wide parts of a key row.  Partial results [heads][splits][vdim + 2] (sum, maximum, total).
-template <typename T, int PIECES>
+// KP, VP: 64-wide parts of a key and of a value row.  Eight lanes a row, 32 rows a pass, four passes: all of a
+// split's keys and values are requested before the first is used.  Partial results [heads][splits][vdim + 2]
+// (weighted sum, maximum, total).
+constexpr int kPasses = (int)kSplitKeys / 32;
+constexpr int kHeadBlock = 4;  // query heads that share one pass over the values
+
+template <typename T, int KP, int VP>
 __global__ __launch_bounds__(256) void chunk_decode_kernel(ChunkAttentionArgs a, uint32_t splits) {
   extern __shared__ __attribute__((aligned(16))) float shared[];
   const uint32_t position = a.state[kStatePosition], slot = a.state[kStateSlot];
@@ -248,27 +327,32 @@ __global__ __launch_bounds__(256) void chunk_decode_kernel(ChunkAttentionArgs a,
   if (begin > position) return;
   const uint32_t keys = min(kSplitKeys, position + 1 - begin);
   const uint32_t dim8 = (a.dim + 7) & ~7u;
-  float *q = shared;                    // [per][dim8]
-  float *scores = q + per * dim8;       // [per][kSplitKeys]
-  float *stats = scores + per * kSplitKeys;  // [per][2]
-  float *reduce = stats + 2 * per;      // [256][9]
-  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
+  float *q = shared;                         // [per][dim8]
+  float *scores = q + per * dim8;            // [per][kSplitKeys]
+  float *reduce = scores + per * kSplitKeys;  // [4][kHeadBlock][VP * 64]
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, sub = tid & 7;
   const bool vec = a.dim % 8 == 0 && a.vdim % 8 == 0;
   const size_t ring = ((size_t)slot * a.kv_heads + group) * a.cache.capacity;
   const T *cache_k = static_cast<const T *>(a.cache.keys) + ring * a.dim;
   const T *cache_v = static_cast<const T *>(a.cache.values) + ring * a.vdim;
 
-  // eight lanes a key, 32 keys a pass; all of a split's keys are requested at once
-  const int sub = tid & 7;
-  Frag<T> k[kSplitKeys / 32][PIECES];
+  Frag<T> k[kPasses][KP], v[kPasses][VP];
 #pragma unroll
-  for (int pass = 0; pass < (int)kSplitKeys / 32; ++pass) {
-    const uint32_t j = begin + min((uint32_t)(pass * 32 + (tid >> 3)), keys - 1);
-    const T *row = cache_k + (size_t)(j % a.cache.capacity) * a.dim;
+  for (int pass = 0; pass < kPasses; ++pass) {
+    const uint32_t j = (begin + min((uint32_t)(pass * 32 + (tid >> 3)), keys - 1)) % a.cache.capacity;
 #pragma unroll
-    for (int p = 0; p < PIECES; ++p) {
+    for (int p = 0; p < KP; ++p) {
       const int c = (p * 8 + sub) * 8;
-      k[pass][p] = load_piece(row + c, (int)a.dim - c, vec);
+      k[pass][p] = load_piece(cache_k + (size_t)j * a.dim + c, (int)a.dim - c, vec);
+    }
+  }
+#pragma unroll
+  for (int pass = 0; pass < kPasses; ++pass) {
+    const uint32_t j = (begin + min((uint32_t)(pass * 32 + (tid >> 3)), keys - 1)) % a.cache.capacity;
+#pragma unroll
+    for (int p = 0; p < VP; ++p) {
+      const int c = (p * 8 + sub) * 8;
+      v[pass][p] = load_piece(cache_v + (size_t)j * a.vdim + c, (int)a.vdim - c, vec);
     }
   }
   for (uint32_t i = tid; i < per * dim8; i += 256) {
@@ -278,17 +362,17 @@ __global__ __launch_bounds__(256) void chunk_decode_kernel(ChunkAttentionArgs a,
   __syncthreads();
   const float inverse_cap = a.softcap > 0.0f ? 1.0f / a.softcap : 0.0f;
   for (uint32_t h = 0; h < per; ++h) {
-    float dot[kSplitKeys / 32];
+    float dot[kPasses];
 #pragma unroll
-    for (int pass = 0; pass < (int)kSplitKeys / 32; ++pass) dot[pass] = 0.0f;
+    for (int pass = 0; pass < kPasses; ++pass) dot[pass] = 0.0f;
 #pragma unroll
-    for (int p = 0; p < PIECES; ++p) {
+    for (int p = 0; p < KP; ++p) {
       const uint32_t c = (p * 8 + sub) * 8;
       if (c >= dim8) continue;
       const f32x4 lo = *reinterpret_cast<const f32x4 *>(q + h * dim8 + c);
       const f32x4 hi = *reinterpret_cast<const f32x4 *>(q + h * dim8 + c + 4);
 #pragma unroll
-      for (int pass = 0; pass < (int)kSplitKeys / 32; ++pass)
+      for (int pass = 0; pass < kPasses; ++pass)
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
           dot[pass] = fmaf(to_f32(k[pass][p][e]), lo[e], dot[pass]);
@@ -296,7 +380,7 @@ __global__ __launch_bounds__(256) void chunk_decode_kernel(ChunkAttentionArgs a,
         }
     }
 #pragma unroll
-    for (int pass = 0; pass < (int)kSplitKeys / 32; ++pass) {
+    for (int pass = 0; pass < kPasses; ++pass) {
       float s = dot[pass];
       s += __shfl_xor(s, 1, 64);
       s += __shfl_xor(s, 2, 64);
@@ -307,89 +391,101 @@ __global__ __launch_bounds__(256) void chunk_decode_kernel(ChunkAttentionArgs a,
     }
   }
   __syncthreads();
-  for (uint32_t h = wave; h < per; h += 4) {
-    float *row = scores + h * kSplitKeys;
-    const float s0 = row[lane], s1 = row[64 + lane];
-    const float best = wave_max(fmaxf(s0, s1));
-    const float e0 = __expf(s0 - best), e1 = __expf(s1 - best);
-    row[lane] = e0;
-    row[64 + lane] = e1;
-    const float sum = wave_sum(e0 + e1);
-    if (lane == 0) {
-      stats[2 * h] = best;
-      stats[2 * h + 1] = sum;
-    }
-  }
-  __syncthreads();
-  const uint32_t pieces = (a.vdim + 7) / 8, subsets = 256 / pieces;
-  const uint32_t piece = tid % pieces, subset = tid / pieces;
-  constexpr int HEADS = 4;
-  for (uint32_t h0 = 0; h0 < per; h0 += HEADS) {
-    float acc[HEADS][8];
+  for (uint32_t h0 = 0; h0 < per; h0 += kHeadBlock) {
+    float best[kHeadBlock], total[kHeadBlock];
 #pragma unroll
-    for (int h = 0; h < HEADS; ++h)
+    for (int h = 0; h < kHeadBlock; ++h) {
+      const float *row = scores + min(h0 + h, per - 1) * kSplitKeys;
+      const float s0 = row[lane], s1 = row[64 + lane];
+      best[h] = wave_max(fmaxf(s0, s1));
+      total[h] = wave_sum(__expf(s0 - best[h]) + __expf(s1 - best[h]));
+      float p[kPasses];
 #pragma unroll
-      for (int e = 0; e < 8; ++e) acc[h][e] = 0.0f;
-    if (subset < subsets)
-#pragma unroll 4
-      for (uint32_t i = subset; i < keys; i += subsets) {
-        const T *row = cache_v + (size_t)((begin + i) % a.cache.capacity) * a.vdim;
-        const Frag<T> v = load_piece(row + piece * 8, (int)a.vdim - (int)piece * 8, vec);
+      for (int pass = 0; pass < kPasses; ++pass) p[pass] = __expf(row[pass * 32 + (tid >> 3)] - best[h]);
+      // the lane's columns over its four keys, then over the eight rows of the wave
 #pragma unroll
-        for (int h = 0; h < HEADS; ++h) {
-          const float p = scores[min(h0 + h, per - 1) * kSplitKeys + i];
+      for (int piece = 0; piece < VP; ++piece)
 #pragma unroll
-          for (int e = 0; e < 8; ++e) acc[h][e] = fmaf(p, to_f32(v[e]), acc[h][e]);
+        for (int e = 0; e < 8; ++e) {
+          float sum = 0.0f;
+#pragma unroll
+          for (int pass = 0; pass < kPasses; ++pass) sum = fmaf(p[pass], to_f32(v[pass][piece][e]), sum);
+          sum += __shfl_xor(sum, 8, 64);
+          sum += __shfl_xor(sum, 16, 64);
+          sum += __shfl_xor(sum, 32, 64);
+          if (lane < 8) reduce[(wave * kHeadBlock + h) * VP * 64 + (piece * 8 + sub) * 8 + e] = sum;
         }
-      }
+    }
+    __syncthreads();
+    for (uint32_t i = tid; i < kHeadBlock * VP * 64; i += 256) {
+      const uint32_t h = i / (VP * 64), c = i % (VP * 64);
+      if (h0 + h >= per || c >= a.vdim) continue;
+      float sum = 0.0f;
 #pragma unroll
-    for (int h = 0; h < HEADS; ++h) {
-      if (h0 + h >= per) break;
+      for (int w = 0; w < 4; ++w) sum += reduce[(w * kHeadBlock + h) * VP * 64 + c];
+      float b = best[0], t = total[0];
+#pragma unroll
+      for (int other = 1; other < kHeadBlock; ++other)
+        if ((int)h == other) {
+          b = best[other];
+          t = total[other];
+        }
       const uint32_t head = group * per + h0 + h;
-      __syncthreads();
-#pragma unroll
-      for (int e = 0; e < 8; ++e) reduce[tid * 9 + e] = acc[h][e];
-      __syncthreads();
-      for (uint32_t c = tid; c < a.vdim; c += 256) {
-        float sum = 0.0f;
-        for (uint32_t s = 0; s < subsets; ++s) sum += reduce[(s * pieces + c / 8) * 9 + c % 8];
-        const float best = stats[2 * (h0 + h)], total = stats[2 * (h0 + h) + 1];
-        if (splits == 1) {
-          const float sink = a.sink ? (float)reinterpret_cast<const __bf16 *>(a.sink)[head] : -INFINITY;
-          const float top = fmaxf(best, sink);
-          const float mine = __expf(best - top);
-          static_cast<T *>(a.out)[head * a.vdim + c] = (T)(sum * mine / (total * mine + __expf(sink - top)));
-        } else {
-          float *partial = static_cast<float *>(a.workspace) + ((size_t)head * splits + split) * (a.vdim + 2);
-          partial[c] = sum;
-          if (c == 0) {
-            partial[a.vdim] = best;
-            partial[a.vdim + 1] = total;
-          }
+      if (splits == 1) {
+        const float sink = a.sink ? (float)reinterpret_cast<const __bf16 *>(a.sink)[head] : -INFINITY;
+        const float top = fmaxf(b, sink);
+        const float mine = __expf(b - top);
+        static_cast<T *>(a.out)[head * a.vdim + c] = (T)(sum * mine / (t * mine + __expf(sink - top)));
+      } else {
+        float *partial = static_cast<float *>(a.workspace) + ((size_t)head * splits + split) * (a.vdim + 2);
+        partial[c] = sum;
+        if (c == 0) {
+          partial[a.vdim] = b;
+          partial[a.vdim + 1] = t;
         }
       }
     }
+    __syncthreads();
   }
 }
 
+// A workgroup a head; the splits' weights are formed once, in LDS.
 template <typename T>
 __global__ __launch_bounds__(256) void chunk_merge_kernel(ChunkAttentionArgs a, uint32_t splits) {
+  extern __shared__ __attribute__((aligned(16))) float shared[];
+  float *best = shared, *total = shared + splits;
   const uint32_t head = blockIdx.x, position = a.state[kStatePosition];
   const uint32_t live = min(splits, (position - chunk_start(position, a.cache.chunk)) / kSplitKeys + 1);
   const uint32_t stride = a.vdim + 2;
   const float *partial = static_cast<const float *>(a.workspace) + (size_t)head * splits * stride;
   const float sink = a.sink ? (float)reinterpret_cast<const __bf16 *>(a.sink)[head] : -INFINITY;
-  float top = sink;
-  for (uint32_t s = 0; s < live; ++s) top = fmaxf(top, partial[s * stride + a.vdim]);
-  float total = __expf(sink - top);
-  for (uint32_t s = 0; s < live; ++s)
-    total += partial[s * stride + a.vdim + 1] * __expf(partial[s * stride + a.vdim] - top);
-  for (uint32_t c = threadIdx.x; c < a.vdim; c += 256) {
-    float sum = 0.0f;
-    for (uint32_t s = 0; s < live; ++s)
-      sum = fmaf(partial[s * stride + c], __expf(partial[s * stride + a.vdim] - top), sum);
-    static_cast<T *>(a.out)[head * a.vdim + c] = (T)(sum / total);
+  constexpr uint32_t AHEAD = 8;
+  const uint32_t c = threadIdx.x;
+  float first[AHEAD];  // the first splits' values on their way while the weights are formed
+#pragma unroll
+  for (uint32_t s = 0; s < AHEAD; ++s) first[s] = s < live && c < a.vdim ? partial[s * stride + c] : 0.0f;
+  for (uint32_t s = threadIdx.x; s < live; s += 256) {
+    best[s] = partial[s * stride + a.vdim];
+    total[s] = partial[s * stride + a.vdim + 1];
   }
+  __syncthreads();
+  float top = sink;
+  for (uint32_t s = 0; s < live; ++s) top = fmaxf(top, best[s]);
+  float denominator = __expf(sink - top), sum = 0.0f;
+#pragma unroll
+  for (uint32_t s = 0; s < AHEAD; ++s)
+    if (s < live) {
+      const float weight = __expf(best[s] - top);
+      denominator = fmaf(total[s], weight, denominator);
+      sum = fmaf(first[s], weight, sum);
+    }
+#pragma unroll 8
+  for (uint32_t s = AHEAD; s < live; ++s) {
+    const float weight = __expf(best[s] - top);
+    denominator = fmaf(total[s], weight, denominator);
+    if (c < a.vdim) sum = fmaf(partial[s * stride + c], weight, sum);
+  }
+  if (c < a.vdim) static_cast<T *>(a.out)[head * a.vdim + c] = (T)(sum / denominator);
 }
 
 uint32_t decode_splits(const ChunkAttentionArgs &a) {
@@ -399,36 +495,48 @@ uint32_t decode_splits(const ChunkAttentionArgs &a) {
 
 uint32_t decode_lds_bytes(const ChunkAttentionArgs &a) {
   const uint32_t per = a.heads / a.kv_heads, dim8 = (a.dim + 7) & ~7u;
-  return (per * dim8 + per * kSplitKeys + 2 * per + 256 * 9) * 4;
+  return (per * dim8 + per * kSplitKeys + 4 * kHeadBlock * 256) * 4;
 }
 
-template <typename T, int PIECES>
+template <typename T, int KP, int VP>
 hipError_t run_decode(const ChunkAttentionArgs &a, hipStream_t stream) {
   static bool allowed[kMaxDevices] = {};
   const uint32_t splits = decode_splits(a), bytes = decode_lds_bytes(a);
   if (bytes > 64 * 1024)
-    if (hipError_t status = allow_dynamic_lds(reinterpret_cast<const void *>(chunk_decode_kernel<T, PIECES>),
+    if (hipError_t status = allow_dynamic_lds(reinterpret_cast<const void *>(chunk_decode_kernel<T, KP, VP>),
                                               160 * 1024, allowed))
       return status;
-  chunk_decode_kernel<T, PIECES><<<dim3(a.kv_heads, splits), 256, bytes, stream>>>(a, splits);
+  chunk_decode_kernel<T, KP, VP><<<dim3(a.kv_heads, splits), 256, bytes, stream>>>(a, splits);
   if (hipError_t status = hipGetLastError()) return status;
-  if (splits > 1) chunk_merge_kernel<T><<<a.heads, 256, 0, stream>>>(a, splits);
+  if (splits > 1) chunk_merge_kernel<T><<<a.heads, 256, splits * 8, stream>>>(a, splits);
+  return hipGetLastError();
+}
+
+template <typename T, int KP>
+hipError_t pick_decode(const ChunkAttentionArgs &a, hipStream_t stream) {
+  if (a.vdim <= 64) return run_decode<T, KP, 1>(a, stream);
+  if (a.vdim <= 128) return run_decode<T, KP, 2>(a, stream);
+  return run_decode<T, KP, 4>(a, stream);
+}
+
+template <typename T, int ND, int NE, bool FIXED>
+hipError_t run_prefill_kernel(const ChunkAttentionArgs &a, hipStream_t stream) {
+  constexpr int QT = sizeof(T) == 2 && ND <= 4 && NE <= 8 ? 2 : 1;
+  constexpr int bytes = prefill_lds_bytes<T, ND, NE>();
+  static bool allowed[kMaxDevices] = {};
+  if (bytes > 64 * 1024)
+    if (hipError_t status = allow_dynamic_lds(
+            reinterpret_cast<const void *>(chunk_prefill_kernel<T, ND, NE, QT, FIXED>), bytes, allowed))
+      return status;
+  const dim3 grid(a.heads, (a.m + 64 * QT - 1) / (64 * QT));
+  chunk_prefill_kernel<T, ND, NE, QT, FIXED><<<grid, 256, bytes, stream>>>(a);
   return hipGetLastError();
 }
 
 template <typename T, int ND, int NE>
 hipError_t run_prefill(const ChunkAttentionArgs &a, hipStream_t stream) {
-  constexpr int QT = sizeof(T) == 2 && ND <= 4 && NE <= 8 ? 2 : 1;
-  constexpr int PAD = 16 / (int)sizeof(T);
-  constexpr int bytes = (kStageKeys * (ND * 32 + PAD) + NE * 16 * (kStageKeys + PAD)) * (int)sizeof(T);
-  static bool allowed[kMaxDevices] = {};
-  if (bytes > 64 * 1024)
-    if (hipError_t status = allow_dynamic_lds(reinterpret_cast<const void *>(chunk_prefill_kernel<T, ND, NE, QT>),
-                                              bytes, allowed))
-      return status;
-  const dim3 grid((a.m + 64 * QT - 1) / (64 * QT), a.heads);
-  chunk_prefill_kernel<T, ND, NE, QT><<<grid, 256, bytes, stream>>>(a);
-  return hipGetLastError();
+  if (a.softcap > 0.0f && a.softcap <= kFixedMaxCap) return run_prefill_kernel<T, ND, NE, true>(a, stream);
+  return run_prefill_kernel<T, ND, NE, false>(a, stream);
 }
 
 template <typename T, int ND>
@@ -442,9 +550,9 @@ hipError_t pick_value_width(const ChunkAttentionArgs &a, hipStream_t stream) {
 template <typename T>
 hipError_t pick_attention(const ChunkAttentionArgs &a, hipStream_t stream) {
   if (a.m == 1) {
-    if (a.dim <= 64) return run_decode<T, 1>(a, stream);
-    if (a.dim <= 128) return run_decode<T, 2>(a, stream);
-    return run_decode<T, 4>(a, stream);
+    if (a.dim <= 64) return pick_decode<T, 1>(a, stream);
+    if (a.dim <= 128) return pick_decode<T, 2>(a, stream);
+    return pick_decode<T, 4>(a, stream);
   }
   if (a.dim <= 64) return pick_value_width<T, 2>(a, stream);
   if (a.dim <= 128) return pick_value_width<T, 4>(a, stream);
@@ -460,7 +568,7 @@ size_t chunk_attention_workspace_bytes(const ChunkAttentionArgs &a) {
 }
 
 bool chunk_attention_ok(const ChunkAttentionArgs &a) {
-  return a.dim <= 256 && a.vdim <= 256 && decode_lds_bytes(a) <= 160 * 1024;
+  return a.dim <= 256 && a.vdim <= 256 && decode_lds_bytes(a) <= 160 * 1024 && decode_splits(a) <= 8000;
 }
 
 hipError_t launch_chunk_attention(const ChunkAttentionArgs &a, hipStream_t stream) {

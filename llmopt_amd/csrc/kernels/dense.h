@@ -48,10 +48,8 @@ struct DenseLinearArgs {
   ValueMix mix;
   // routed rows (null: the plain product): see RoutePlan
   const uint32_t *tile_expert, *tile_first, *tile_rows, *row_source;
-  uint32_t tiles;
+  uint32_t tiles, tile;  // most tiles the plan can fill, rows of a tile
 };
-// Rows of a product tile of the routed form (what RoutePlan cuts experts into).
-constexpr uint32_t kRoutedTileRows = 64;
 hipError_t launch_dense_gemm(const DenseLinearArgs &args, hipStream_t stream);
 
 // out[r, :] = x[row, :] / rms * weight with row = rows ? rows[r] : r; `groups` equal parts normalised each
@@ -176,9 +174,10 @@ struct RoutePlan {
   uint32_t *position;   // [m, top]: row of the sorted order
   uint32_t *row_token;  // [m * top]
   uint32_t *tile_expert, *tile_first, *tile_rows;  // [max_tiles]
-  uint32_t max_tiles;
+  uint32_t max_tiles, tile;  // tile: rows of a product tile, 64 or 128
 };
-uint32_t route_max_tiles(uint32_t m, uint32_t experts, uint32_t top);
+uint32_t route_tile_rows(uint32_t m, uint32_t experts, uint32_t top, uint32_t width, uint32_t ff, bool f32);
+uint32_t route_max_tiles(uint32_t m, uint32_t experts, uint32_t top, uint32_t tile);
 // The `top` largest logits of every token (ties to the lower index), the softmax over them, the
 // (token, choice) pairs sorted by expert and cut into product tiles of one expert.
 hipError_t launch_route(const RoutePlan &plan, hipStream_t stream);

@@ -3,11 +3,10 @@
 //
 //   out[r, c] = sum_k x[r, k] w[c, k]       x [m, k] bf16 or f32, w bf16 [n, k], sums in float32
 //
-// A workgroup of four waves owns a BM x BN tile and walks K in stages of 64, double-buffered through
-// LDS: the next stage travels global -> registers while this one is multiplied, one barrier a stage.
-// LDS rows carry 16 bytes of padding, so that the sixteen rows an operand read touches start in
-// different banks.  The weights are the A operand and the activations the B operand: a lane then ends
-// with four consecutive output columns of one row, and the epilogue stores 8 or 16 bytes at a time.
+// A workgroup owns a BM x BN tile and walks K in stages of 64 staged in LDS (dense_gemm_direct_kernel for
+// bf16 rows of whole stages, dense_gemm_kernel through registers for the rest).  The weights are the A
+// operand and the activations the B operand: a lane then ends with four consecutive output columns of one
+// row, and the epilogue stores 8 or 16 bytes at a time.
 //
 //  * gated: the 16-column groups of a tile alternate between the gate and the up matrix, so that both
 //    values of an output element meet in one lane.
@@ -106,12 +105,74 @@ __device__ __forceinline__ void emit(const DenseLinearArgs &a, uint32_t r, uint3
   }
 }
 
-// WM x WN waves; a wave owns (BM / WM) x (BN / WN).
-template <typename T, int BM, int BN, int WM, bool GATED, bool ROUTED, bool VEC>
-__global__ __launch_bounds__(256) void dense_gemm_kernel(GemmParams p) {
-  constexpr int WN = 4 / WM;
+// Where a workgroup's tile lies; false: nothing to do.
+struct TilePlace {
+  uint32_t m_first, m_rows, n_first, expert;
+};
+
+template <int BM, int COLUMNS, bool ROUTED>
+__device__ __forceinline__ bool place_tile(const GemmParams &p, TilePlace &t) {
+  const DenseLinearArgs &a = p.a;
+  t.expert = 0;
+  if (ROUTED) {
+    const uint32_t tile = blockIdx.y;
+    t.m_rows = a.tile_rows[tile];
+    if (t.m_rows == 0) return false;
+    t.m_first = a.tile_first[tile];
+    t.expert = a.tile_expert[tile];
+    t.n_first = blockIdx.x * COLUMNS;
+    return true;
+  }
+  const uint32_t id = (blockIdx.x & 7) * p.per_xcd + (blockIdx.x >> 3);
+  if (id >= p.total) return false;
+  // groups of eight row tiles walk the column tiles together
+  const uint32_t group_tiles = 8 * p.tiles_n, group = id / group_tiles, within = id % group_tiles;
+  const uint32_t rows_here = min(8u, p.tiles_m - group * 8);
+  t.m_first = (group * 8 + within % rows_here) * BM;
+  t.m_rows = min((uint32_t)BM, a.m - t.m_first);
+  t.n_first = within / rows_here * COLUMNS;
+  return true;
+}
+
+// A wave's accumulators: MT x NT groups of 16 x 16 from row `row_offset` and tile column `column_offset` on.
+template <typename T, int MT, int NT, bool GATED>
+__device__ __forceinline__ void emit_tile(const DenseLinearArgs &a, const f32x4 (&acc)[MT][NT], uint32_t m_first,
+                                          uint32_t m_rows, uint32_t n_first, uint32_t row_offset,
+                                          uint32_t column_offset, int lane) {
+  const int column = (lane >> 4) * 4;
+#pragma unroll
+  for (int i = 0; i < MT; ++i) {
+    const uint32_t r_in_tile = row_offset + i * 16 + (lane & 15);
+    if (r_in_tile >= m_rows) continue;
+    const uint32_t r = m_first + r_in_tile;
+    if (GATED) {
+#pragma unroll
+      for (int j = 0; j < NT; j += 2) {
+        const uint32_t c = n_first + column_offset / 2 + (j / 2) * 16 + column;
+        if (c >= a.n) continue;
+        f32x4 v;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[e] = gate_activation(acc[i][j][e], a.activation) * acc[i][j + 1][e];
+        emit<T>(a, r, c, v);
+      }
+    } else {
+#pragma unroll
+      for (int j = 0; j < NT; ++j) {
+        const uint32_t c = n_first + column_offset + j * 16 + column;
+        if (c < a.n) emit<T>(a, r, c, acc[i][j]);
+      }
+    }
+  }
+}
+
+// WM x WN waves; a wave owns (BM / WM) x (BN / WN).  Two LDS stages: the next one travels global -> registers
+// while this one is multiplied, one barrier a stage; LDS rows carry 16 bytes of padding, so that the sixteen
+// rows an operand read touches start in different banks.
+template <typename T, int BM, int BN, int WM, bool GATED, bool ROUTED, bool VEC, int WAVES = 4>
+__global__ __launch_bounds__(WAVES * 64) void dense_gemm_kernel(GemmParams p) {
+  constexpr int WN = WAVES / WM, PASS = WAVES * 8;
   constexpr int MT = BM / WM / 16, NT = BN / WN / 16;
-  constexpr int A_PIECES = BM * 8 / 256, W_PIECES = BN * 8 / 256;
+  constexpr int A_PIECES = BM / PASS, W_PIECES = BN / PASS;
   constexpr int SA = lds_stride<T>(), SW = lds_stride<__bf16>();
   constexpr int COLUMNS = GATED ? BN / 2 : BN;
   static_assert(!GATED || NT % 2 == 0, "gate and up of an element meet in one wave");
@@ -120,41 +181,25 @@ __global__ __launch_bounds__(256) void dense_gemm_kernel(GemmParams p) {
   __bf16 *lds_w = reinterpret_cast<__bf16 *>(lds + 2 * BM * SA * sizeof(T));
   const DenseLinearArgs &a = p.a;
 
-  uint32_t m_first, m_rows, n_first, expert = 0;
-  if (ROUTED) {
-    const uint32_t tile = blockIdx.y;
-    m_rows = a.tile_rows[tile];
-    if (m_rows == 0) return;
-    m_first = a.tile_first[tile];
-    expert = a.tile_expert[tile];
-    n_first = blockIdx.x * COLUMNS;
-  } else {
-    const uint32_t id = (blockIdx.x & 7) * p.per_xcd + (blockIdx.x >> 3);
-    if (id >= p.total) return;
-    // groups of eight row tiles walk the column tiles together
-    const uint32_t group_tiles = 8 * p.tiles_n, group = id / group_tiles, within = id % group_tiles;
-    const uint32_t rows_here = min(8u, p.tiles_m - group * 8);
-    const uint32_t tile_m = group * 8 + within % rows_here, tile_n = within / rows_here;
-    m_first = tile_m * BM;
-    m_rows = min((uint32_t)BM, a.m - m_first);
-    n_first = tile_n * COLUMNS;
-  }
+  TilePlace place;
+  if (!place_tile<BM, COLUMNS, ROUTED>(p, place)) return;
+  const uint32_t m_first = place.m_first, m_rows = place.m_rows, n_first = place.n_first, expert = place.expert;
 
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
   const int wm = wave / WN, wn = wave % WN;
-  const int piece = tid & 7, row_in_pass = tid >> 3;  // 32 rows a pass
+  const int piece = tid & 7, row_in_pass = tid >> 3;  // PASS rows a pass
 
   const T *src_a[A_PIECES];
 #pragma unroll
   for (int i = 0; i < A_PIECES; ++i) {
-    uint32_t r = m_first + min((uint32_t)(row_in_pass + 32 * i), m_rows - 1);
+    uint32_t r = m_first + min((uint32_t)(row_in_pass + PASS * i), m_rows - 1);
     if (ROUTED && a.row_source) r = a.row_source[r];
     src_a[i] = static_cast<const T *>(a.x) + (size_t)r * a.ldx + piece * 8;
   }
   const __bf16 *src_w[W_PIECES];
 #pragma unroll
   for (int i = 0; i < W_PIECES; ++i) {
-    const int r = row_in_pass + 32 * i;
+    const int r = row_in_pass + PASS * i;
     const uint16_t *matrix = a.w;
     uint32_t c = n_first + r;
     if (GATED) {
@@ -177,10 +222,10 @@ __global__ __launch_bounds__(256) void dense_gemm_kernel(GemmParams p) {
   auto stash = [&](int buffer) {
 #pragma unroll
     for (int i = 0; i < A_PIECES; ++i)
-      *reinterpret_cast<Frag<T> *>(lds_a + (buffer * BM + row_in_pass + 32 * i) * SA + piece * 8) = reg_a[i];
+      *reinterpret_cast<Frag<T> *>(lds_a + (buffer * BM + row_in_pass + PASS * i) * SA + piece * 8) = reg_a[i];
 #pragma unroll
     for (int i = 0; i < W_PIECES; ++i)
-      *reinterpret_cast<bf16x8 *>(lds_w + (buffer * BN + row_in_pass + 32 * i) * SW + piece * 8) = reg_w[i];
+      *reinterpret_cast<bf16x8 *>(lds_w + (buffer * BN + row_in_pass + PASS * i) * SW + piece * 8) = reg_w[i];
   };
 
   f32x4 acc[MT][NT];
@@ -189,14 +234,9 @@ __global__ __launch_bounds__(256) void dense_gemm_kernel(GemmParams p) {
 #pragma unroll
     for (int j = 0; j < NT; ++j) acc[i][j] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
 
-  fetch(0);
-  stash(0);
-  __syncthreads();
   const int stages = (int)((a.k + kStageK - 1) / kStageK);
   const int fr = lane & 15, fk = (lane >> 4) * 8;
-  for (int s = 0; s < stages; ++s) {
-    const int buffer = s & 1;
-    if (s + 1 < stages) fetch((s + 1) * kStageK);
+  auto multiply = [&](int buffer) {
     const T *la = lds_a + (buffer * BM + wm * (BM / WM) + fr) * SA + fk;
     const __bf16 *lw = lds_w + (buffer * BN + wn * (BN / WN) + fr) * SW + fk;
 #pragma unroll
@@ -213,77 +253,192 @@ __global__ __launch_bounds__(256) void dense_gemm_kernel(GemmParams p) {
 #pragma unroll
         for (int j = 0; j < NT; ++j) acc[i][j] = mma(fw[j], fa[i], acc[i][j]);
     }
-    if (s + 1 < stages) stash(buffer ^ 1);
+  };
+  fetch(0);
+  stash(0);
+  __syncthreads();
+  for (int s = 0; s < stages; ++s) {
+    if (s + 1 < stages) fetch((s + 1) * kStageK);
+    multiply(s & 1);
+    if (s + 1 < stages) stash((s & 1) ^ 1);
     __syncthreads();
   }
 
-  const int column = (lane >> 4) * 4;
-#pragma unroll
-  for (int i = 0; i < MT; ++i) {
-    const uint32_t r_in_tile = wm * (BM / WM) + i * 16 + fr;
-    if (r_in_tile >= m_rows) continue;
-    const uint32_t r = m_first + r_in_tile;
-    if (GATED) {
-#pragma unroll
-      for (int j = 0; j < NT; j += 2) {
-        const uint32_t c = n_first + (wn * NT / 2 + j / 2) * 16 + column;
-        if (c >= a.n) continue;
-        f32x4 v;
-#pragma unroll
-        for (int e = 0; e < 4; ++e) v[e] = gate_activation(acc[i][j][e], a.activation) * acc[i][j + 1][e];
-        emit<T>(a, r, c, v);
-      }
-    } else {
-#pragma unroll
-      for (int j = 0; j < NT; ++j) {
-        const uint32_t c = n_first + wn * (BN / WN) + j * 16 + column;
-        if (c < a.n) emit<T>(a, r, c, acc[i][j]);
-      }
-    }
-  }
+  emit_tile<T, MT, NT, GATED>(a, acc, m_first, m_rows, n_first, wm * (BM / WM), wn * (BN / WN), lane);
 }
 
-template <typename T, int BM, int BN, int WM, bool GATED, bool ROUTED, bool VEC>
+template <int BM, int COLUMNS, bool ROUTED>
+GemmParams gemm_params(const DenseLinearArgs &a, dim3 *grid) {
+  GemmParams p = {};
+  p.a = a;
+  p.tiles_n = (a.n + COLUMNS - 1) / COLUMNS;
+  if (ROUTED) {
+    *grid = dim3(p.tiles_n, a.tiles);
+  } else {
+    p.tiles_m = (a.m + BM - 1) / BM;
+    p.total = p.tiles_m * p.tiles_n;
+    p.per_xcd = (p.total + 7) / 8;
+    *grid = dim3(p.per_xcd * 8);
+  }
+  return p;
+}
+
+template <typename T, int BM, int BN, int WM, bool GATED, bool ROUTED, bool VEC, int WAVES = 4>
 hipError_t run_gemm(const DenseLinearArgs &a, hipStream_t stream) {
   constexpr int bytes = gemm_lds_bytes<T, BM, BN>();
   static bool allowed[kMaxDevices] = {};
   if (bytes > 64 * 1024)
     if (hipError_t status = allow_dynamic_lds(
-            reinterpret_cast<const void *>(dense_gemm_kernel<T, BM, BN, WM, GATED, ROUTED, VEC>), bytes, allowed))
+            reinterpret_cast<const void *>(dense_gemm_kernel<T, BM, BN, WM, GATED, ROUTED, VEC, WAVES>), bytes, allowed))
       return status;
-  GemmParams p = {};
-  p.a = a;
-  constexpr uint32_t columns = GATED ? BN / 2 : BN;
-  p.tiles_n = (a.n + columns - 1) / columns;
   dim3 grid;
-  if (ROUTED) {
-    grid = dim3(p.tiles_n, a.tiles);
-  } else {
-    p.tiles_m = (a.m + BM - 1) / BM;
-    p.total = p.tiles_m * p.tiles_n;
-    p.per_xcd = (p.total + 7) / 8;
-    grid = dim3(p.per_xcd * 8);
-  }
-  dense_gemm_kernel<T, BM, BN, WM, GATED, ROUTED, VEC><<<grid, 256, bytes, stream>>>(p);
+  const GemmParams p = gemm_params<BM, GATED ? BN / 2 : BN, ROUTED>(a, &grid);
+  dense_gemm_kernel<T, BM, BN, WM, GATED, ROUTED, VEC, WAVES><<<grid, WAVES * 64, bytes, stream>>>(p);
   return hipGetLastError();
 }
 
-template <bool GATED, bool ROUTED>
-hipError_t pick_gemm(const DenseLinearArgs &a, hipStream_t stream) {
-  const bool vec = a.k % 8 == 0 && a.ldx % 8 == 0;
-  constexpr int SMALL = ROUTED ? (int)kRoutedTileRows : 32;
-  const uint32_t columns = a.n * (GATED ? 2 : 1);
-  if (a.f32) {
-    if (!vec) return run_gemm<float, SMALL, 64, 2, GATED, ROUTED, false>(a, stream);
-    return run_gemm<float, SMALL, 64, 2, GATED, ROUTED, true>(a, stream);
+// The same product for bf16 rows of a multiple of 64 values, staged by direct global -> LDS copies
+// (global_load_lds_dwordx4: 64 lanes x 16 bytes to consecutive LDS addresses) a ring of STAGES stages deep:
+// the copies of later stages run while a stage is multiplied, waited for by count, one barrier a stage.
+// LDS rows are 128 bytes with their 16-byte pieces XOR-ed by half the row, which spreads the sixteen rows
+// an operand read touches over all banks; the copies place pieces by permuting their source addresses.
+__device__ __forceinline__ void copy_to_lds(const __bf16 *source, uint32_t lds_address) {
+  asm volatile("s_mov_b32 m0, %1\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %0, off" : : "v"(source), "s"(lds_address) : "memory");
+}
+
+template <int BM, int BN, int WM, int WAVES, int STAGES, bool GATED, bool ROUTED>
+__global__ __launch_bounds__(WAVES * 64) void dense_gemm_direct_kernel(GemmParams p) {
+  constexpr int WN = WAVES / WM;
+  constexpr int MT = BM / WM / 16, NT = BN / WN / 16;
+  constexpr int ROWS = BM + BN;              // LDS rows of a stage: activations, then weights
+  constexpr int COPIES = ROWS / 8 / WAVES;   // 8-row copies of a wave per stage
+  constexpr int COLUMNS = GATED ? BN / 2 : BN;
+  static_assert(ROWS % (8 * WAVES) == 0 && (!GATED || NT % 2 == 0), "tile does not divide over the waves");
+  extern __shared__ __attribute__((aligned(16))) char lds[];
+  __bf16 *stage_rows = reinterpret_cast<__bf16 *>(lds);
+  const DenseLinearArgs &a = p.a;
+  TilePlace place;
+  if (!place_tile<BM, COLUMNS, ROUTED>(p, place)) return;
+
+  const int tid = threadIdx.x, lane = tid & 63;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int wm = wave / WN, wn = wave % WN;
+
+  const __bf16 *source[COPIES];
+#pragma unroll
+  for (int i = 0; i < COPIES; ++i) {
+    const int row = (i * WAVES + wave) * 8 + (lane >> 3);
+    const int piece = (lane & 7) ^ ((row >> 1) & 7);
+    if (row < BM) {
+      uint32_t r = place.m_first + min((uint32_t)row, place.m_rows - 1);
+      if (ROUTED && a.row_source) r = a.row_source[r];
+      source[i] = static_cast<const __bf16 *>(a.x) + (size_t)r * a.ldx + piece * 8;
+    } else {
+      const int w_row = row - BM;
+      const uint16_t *matrix = a.w;
+      uint32_t c = place.n_first + w_row;
+      if (GATED) {
+        if ((w_row >> 4) & 1) matrix = a.w_up;
+        c = place.n_first + (w_row >> 5) * 16 + (w_row & 15);
+      }
+      c = min(c, a.n - 1);
+      source[i] = reinterpret_cast<const __bf16 *>(matrix) + ((size_t)place.expert * a.n + c) * a.k + piece * 8;
+    }
   }
-  if (!vec) return run_gemm<__bf16, SMALL, 64, 2, GATED, ROUTED, false>(a, stream);
-  if (ROUTED) return run_gemm<__bf16, (int)kRoutedTileRows, 128, 2, GATED, ROUTED, true>(a, stream);
-  const uint64_t big = (uint64_t)((a.m + 127) / 128) * ((columns + 127) / 128);
-  if (a.m > 64 && big >= 192) return run_gemm<__bf16, 128, 128, 2, GATED, false, true>(a, stream);
-  const uint64_t middle = (uint64_t)((a.m + 63) / 64) * ((columns + 127) / 128);
-  if (a.m > 32 && middle >= 192) return run_gemm<__bf16, 64, 128, 2, GATED, false, true>(a, stream);
-  return run_gemm<__bf16, SMALL, 64, 2, GATED, ROUTED, true>(a, stream);
+  const uint32_t lds_base = (uint32_t)(size_t)(__attribute__((address_space(3))) char *)lds;
+  auto request = [&](int stage) {
+    const uint32_t slot = lds_base + (stage % STAGES) * ROWS * 128;
+#pragma unroll
+    for (int i = 0; i < COPIES; ++i) copy_to_lds(source[i] + stage * kStageK, slot + (i * WAVES + wave) * 1024);
+  };
+
+  f32x4 acc[MT][NT];
+#pragma unroll
+  for (int i = 0; i < MT; ++i)
+#pragma unroll
+    for (int j = 0; j < NT; ++j) acc[i][j] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+
+  const int stages = (int)(a.k / kStageK);
+  const int fr = lane & 15, quad = lane >> 4, twist = (fr >> 1) & 7;
+#pragma unroll
+  for (int s = 0; s < STAGES - 1; ++s)
+    if (s < stages) request(s);
+  for (int s = 0; s < stages; ++s) {
+    // this stage has landed once at most the copies of the STAGES - 2 later ones are under way (and this wave
+    // has all it read of the stage before)
+    if (s + STAGES - 2 < stages) asm volatile("s_waitcnt vmcnt(%0) lgkmcnt(0)" : : "n"((STAGES - 2) * COPIES) : "memory");
+    else asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)" ::: "memory");
+    __builtin_amdgcn_s_barrier();
+    asm volatile("" ::: "memory");
+    // every wave is done with the stage before: its slot is free
+    if (s + STAGES - 1 < stages) request(s + STAGES - 1);
+    const __bf16 *rows = stage_rows + (s % STAGES) * ROWS * 64;
+    const __bf16 *la = rows + (wm * (BM / WM) + fr) * 64, *lw = rows + (BM + wn * (BN / WN) + fr) * 64;
+#pragma unroll
+    for (int kk = 0; kk < 2; ++kk) {
+      const int at = ((kk * 4 + quad) ^ twist) * 8;
+      bf16x8 fa[MT], fw[NT];
+#pragma unroll
+      for (int j = 0; j < NT; ++j) fw[j] = *reinterpret_cast<const bf16x8 *>(lw + j * 16 * 64 + at);
+#pragma unroll
+      for (int i = 0; i < MT; ++i) fa[i] = *reinterpret_cast<const bf16x8 *>(la + i * 16 * 64 + at);
+#pragma unroll
+      for (int i = 0; i < MT; ++i)
+#pragma unroll
+        for (int j = 0; j < NT; ++j) acc[i][j] = mma(fw[j], fa[i], acc[i][j]);
+    }
+  }
+  emit_tile<__bf16, MT, NT, GATED>(a, acc, place.m_first, place.m_rows, place.n_first, wm * (BM / WM),
+                                   wn * (BN / WN), lane);
+}
+
+template <int BM, int BN, int WM, int WAVES, int STAGES, bool GATED, bool ROUTED>
+hipError_t run_direct(const DenseLinearArgs &a, hipStream_t stream) {
+  constexpr int bytes = STAGES * (BM + BN) * 128;
+  static bool allowed[kMaxDevices] = {};
+  const auto kernel = dense_gemm_direct_kernel<BM, BN, WM, WAVES, STAGES, GATED, ROUTED>;
+  if (bytes > 64 * 1024)
+    if (hipError_t status = allow_dynamic_lds(reinterpret_cast<const void *>(kernel), bytes, allowed)) return status;
+  dim3 grid;
+  const GemmParams p = gemm_params<BM, GATED ? BN / 2 : BN, ROUTED>(a, &grid);
+  kernel<<<grid, WAVES * 64, bytes, stream>>>(p);
+  return hipGetLastError();
+}
+
+// Rows whose length is no multiple of the stage, and float32 rows: through registers.
+template <typename T, int BM, bool GATED, bool ROUTED>
+hipError_t run_registers(const DenseLinearArgs &a, hipStream_t stream) {
+  if (a.k % 8 == 0 && a.ldx % 8 == 0) return run_gemm<T, BM, 64, 2, GATED, ROUTED, true>(a, stream);
+  return run_gemm<T, BM, 64, 2, GATED, ROUTED, false>(a, stream);
+}
+
+template <bool GATED>
+hipError_t pick_routed(const DenseLinearArgs &a, hipStream_t stream) {
+  const bool direct = !a.f32 && a.k % kStageK == 0 && a.ldx % 8 == 0;
+  if (a.tile == 128) return direct ? run_direct<128, 128, 2, 4, 2, GATED, true>(a, stream) : hipErrorInvalidValue;
+  if (direct) return run_direct<64, 128, 2, 4, 3, GATED, true>(a, stream);
+  return a.f32 ? run_registers<float, 64, GATED, true>(a, stream) : run_registers<__bf16, 64, GATED, true>(a, stream);
+}
+
+// The largest tile that still gives the 256 CUs whole rounds of work.  Measured, TFLOP/s (m x n x k):
+// 8192 x 4096 x 4096 937 / 827 with 256 x 256 / 128 x 128 tiles; 2048 x 8512 x 2048 500 / 680 / 643 with
+// 256 x 256 / 128 x 128 / 64 x 128; 2048 x 2048 x 8192 723 / 842 / 681 with 128 x 128 / 64 x 128 / 64 x 64;
+// 512 x 2048 x 4096 261 / 359 with 64 x 128 / 64 x 64; 64 x 4096 x 2048 80 / 89 with 64 x 64 / 32 x 64.
+template <bool GATED>
+hipError_t pick_gemm(const DenseLinearArgs &a, hipStream_t stream) {
+  if (a.f32) return run_registers<float, 32, GATED, false>(a, stream);
+  const uint32_t columns = a.n * (GATED ? 2 : 1);
+  auto tiles = [&](uint32_t rows, uint32_t width) {
+    return (uint64_t)((a.m + rows - 1) / rows) * ((columns + width - 1) / width);
+  };
+  if (a.k % kStageK != 0 || a.ldx % 8 != 0) return run_registers<__bf16, 32, GATED, false>(a, stream);
+  const uint64_t largest = tiles(256, 256), over = largest % 256;
+  if (largest >= 1024 || (largest >= 256 && (over == 0 || over >= 192)))
+    return run_direct<256, 256, 2, 8, 2, GATED, false>(a, stream);
+  if (tiles(128, 128) > 320) return run_direct<128, 128, 2, 4, 2, GATED, false>(a, stream);
+  if (tiles(64, 128) >= 320) return run_direct<64, 128, 2, 4, 3, GATED, false>(a, stream);
+  if (tiles(64, 64) >= 160) return run_direct<64, 64, 2, 4, 4, GATED, false>(a, stream);
+  return run_direct<32, 64, 2, 4, 6, GATED, false>(a, stream);
 }
 
 // ---- row-wise kernels ------------------------------------------------------------------------------
@@ -373,8 +528,8 @@ __global__ __launch_bounds__(256) void dense_embedding_kernel(DenseEmbeddingArgs
 
 hipError_t launch_dense_gemm(const DenseLinearArgs &a, hipStream_t stream) {
   const bool gated = a.epilogue == DenseEpilogue::kGated;
-  if (a.tile_expert) return gated ? pick_gemm<true, true>(a, stream) : pick_gemm<false, true>(a, stream);
-  return gated ? pick_gemm<true, false>(a, stream) : pick_gemm<false, false>(a, stream);
+  if (a.tile_expert) return gated ? pick_routed<true>(a, stream) : pick_routed<false>(a, stream);
+  return gated ? pick_gemm<true>(a, stream) : pick_gemm<false>(a, stream);
 }
 
 hipError_t launch_dense_norm(const DenseNormArgs &a, hipStream_t stream) {

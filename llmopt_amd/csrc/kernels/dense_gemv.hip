@@ -24,14 +24,38 @@ __device__ __forceinline__ uint32_t staged_index(uint32_t k, uint32_t plane) {
   return ((k >> 2) & 1) * plane + ((k >> 3) << 2) + (k & 3);
 }
 
-// Stages the f32 row x, normalised in `groups` parts by norm_weight when that is not null.
-template <typename T>
-__device__ __forceinline__ void stage_activation(const DenseGemvArgs &a, float *xs, uint32_t plane, float *scratch) {
+// Stages the f32 row x, normalised in `groups` parts by norm_weight when that is not null.  `ahead` is
+// called once the row has been requested (loads return in order: what it requests does not delay the row).
+template <typename T, typename Ahead>
+__device__ __forceinline__ void stage_activation(const DenseGemvArgs &a, float *xs, uint32_t plane, float *scratch,
+                                                 Ahead ahead) {
   const uint32_t k = a.k;
   const __bf16 *weight = reinterpret_cast<const __bf16 *>(a.norm_weight);
   // whole pieces behind the row's end read as zeros
   for (uint32_t i = k + threadIdx.x; i < ((k + 7) & ~7u); i += kWaves * 64) xs[staged_index(i, plane)] = 0.0f;
   if (weight == nullptr) {
+    if ((k & 7) == 0 && k <= 8 * 8 * kWaves * 64) {
+      f32x8 v[8];
+#pragma unroll
+      for (int q = 0; q < 8; ++q) {
+        const uint32_t i = (q * kWaves * 64 + threadIdx.x) * 8;
+        if (i < k)
+          v[q] = a.x_is_f32 ? *reinterpret_cast<const f32x8 *>(static_cast<const float *>(a.x) + i)
+                            : convert_frag<float>(*reinterpret_cast<const Frag<T> *>(static_cast<const T *>(a.x) + i));
+      }
+      ahead();
+#pragma unroll
+      for (int q = 0; q < 8; ++q) {
+        const uint32_t i = (q * kWaves * 64 + threadIdx.x) * 8;
+        if (i < k) {
+          *reinterpret_cast<f32x4 *>(xs + (i >> 1)) = f32x4{v[q][0], v[q][1], v[q][2], v[q][3]};
+          *reinterpret_cast<f32x4 *>(xs + plane + (i >> 1)) = f32x4{v[q][4], v[q][5], v[q][6], v[q][7]};
+        }
+      }
+      __syncthreads();
+      return;
+    }
+    ahead();
     for (uint32_t i = threadIdx.x; i < k; i += kWaves * 64)
       xs[staged_index(i, plane)] =
           a.x_is_f32 ? static_cast<const float *>(a.x)[i] : to_f32(static_cast<const T *>(a.x)[i]);
@@ -40,27 +64,29 @@ __device__ __forceinline__ void stage_activation(const DenseGemvArgs &a, float *
   }
   const float *x = static_cast<const float *>(a.x);
   const uint32_t part = k / a.norm_groups;
-  if (a.norm_groups == 1 && (k & 3) == 0 && k <= 4 * 4 * kWaves * 64) {
+  constexpr int PIECES = 8;
+  if (a.norm_groups == 1 && (k & 3) == 0 && k <= PIECES * 4 * kWaves * 64) {
     // the row in registers: one trip to memory
-    f32x4 v[4];
-    bf16x4 w[4];
+    f32x4 v[PIECES];
+    bf16x4 w[PIECES];
     float sum = 0.0f;
 #pragma unroll
-    for (int q = 0; q < 4; ++q) {
+    for (int q = 0; q < PIECES; ++q) {
       const uint32_t i = (q * kWaves * 64 + threadIdx.x) * 4;
+      v[q] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
       if (i < k) {
         v[q] = *reinterpret_cast<const f32x4 *>(x + i);
         w[q] = *reinterpret_cast<const bf16x4 *>(weight + i);
-      } else {
-        v[q] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
       }
     }
+    ahead();
 #pragma unroll
-    for (int q = 0; q < 4; ++q) sum += v[q][0] * v[q][0] + v[q][1] * v[q][1] + v[q][2] * v[q][2] + v[q][3] * v[q][3];
+    for (int q = 0; q < PIECES; ++q)
+      sum += v[q][0] * v[q][0] + v[q][1] * v[q][1] + v[q][2] * v[q][2] + v[q][3] * v[q][3];
     sum = block_sum<kWaves>(sum, scratch);
     const float inverse = 1.0f / sqrtf(sum / (float)k + a.epsilon);
 #pragma unroll
-    for (int q = 0; q < 4; ++q) {
+    for (int q = 0; q < PIECES; ++q) {
       const uint32_t i = (q * kWaves * 64 + threadIdx.x) * 4;
       if (i < k) {
         f32x4 out;
@@ -72,6 +98,7 @@ __device__ __forceinline__ void stage_activation(const DenseGemvArgs &a, float *
     __syncthreads();
     return;
   }
+  ahead();
   for (uint32_t g = 0; g < a.norm_groups; ++g) {
     float sum = 0.0f;
     for (uint32_t i = g * part + threadIdx.x; i < (g + 1) * part; i += kWaves * 64) sum += x[i] * x[i];
@@ -83,40 +110,51 @@ __device__ __forceinline__ void stage_activation(const DenseGemvArgs &a, float *
   __syncthreads();
 }
 
-// sums[r] = w[row_r] . x for ROWS rows (pointers to their starts); every lane ends with every sum.
+// ROWS weight rows streamed against the staged activation in blocks of 2048 columns; the first block is
+// requested by `request`, ahead of the staging.
 template <int ROWS, bool VEC>
-__device__ __forceinline__ void dot_rows(const __bf16 *const (&rows)[ROWS], const float *xs, uint32_t plane,
-                                         uint32_t k, int lane, float (&sums)[ROWS]) {
-  constexpr int STEPS = ROWS >= 4 ? 2 : 4;
-#pragma unroll
-  for (int r = 0; r < ROWS; ++r) sums[r] = 0.0f;
-  for (uint32_t k0 = 0; k0 < k; k0 += 512 * STEPS) {
-    bf16x8 w[STEPS][ROWS];
+struct RowStream {
+  static constexpr int STEPS = 4;
+  const __bf16 *rows[ROWS];
+  bf16x8 w[STEPS][ROWS];
+  float sums[ROWS];
+
+  __device__ __forceinline__ void fetch(uint32_t k0, uint32_t k, int lane) {
 #pragma unroll
     for (int s = 0; s < STEPS; ++s) {
       const uint32_t kk = k0 + s * 512 + lane * 8;
 #pragma unroll
       for (int r = 0; r < ROWS; ++r) w[s][r] = load_piece(rows[r] + kk, (int)k - (int)kk, VEC);
     }
+  }
+  __device__ __forceinline__ void request(uint32_t k, int lane) { fetch(0, k, lane); }
+
+  // every lane ends with every sum
+  __device__ __forceinline__ void run(const float *xs, uint32_t plane, uint32_t k, int lane) {
 #pragma unroll
-    for (int s = 0; s < STEPS; ++s) {
-      const uint32_t kk = k0 + s * 512 + lane * 8;
-      if (kk >= k) continue;
-      const f32x4 lo = *reinterpret_cast<const f32x4 *>(xs + (kk >> 1));
-      const f32x4 hi = *reinterpret_cast<const f32x4 *>(xs + plane + (kk >> 1));
+    for (int r = 0; r < ROWS; ++r) sums[r] = 0.0f;
+    for (uint32_t k0 = 0; k0 < k; k0 += 512 * STEPS) {
+      if (k0 > 0) fetch(k0, k, lane);
 #pragma unroll
-      for (int r = 0; r < ROWS; ++r) {
+      for (int s = 0; s < STEPS; ++s) {
+        const uint32_t kk = k0 + s * 512 + lane * 8;
+        if (kk >= k) continue;
+        const f32x4 lo = *reinterpret_cast<const f32x4 *>(xs + (kk >> 1));
+        const f32x4 hi = *reinterpret_cast<const f32x4 *>(xs + plane + (kk >> 1));
 #pragma unroll
-        for (int e = 0; e < 4; ++e) {
-          sums[r] = fmaf((float)w[s][r][e], lo[e], sums[r]);
-          sums[r] = fmaf((float)w[s][r][4 + e], hi[e], sums[r]);
+        for (int r = 0; r < ROWS; ++r) {
+#pragma unroll
+          for (int e = 0; e < 4; ++e) {
+            sums[r] = fmaf((float)w[s][r][e], lo[e], sums[r]);
+            sums[r] = fmaf((float)w[s][r][4 + e], hi[e], sums[r]);
+          }
         }
       }
     }
-  }
 #pragma unroll
-  for (int r = 0; r < ROWS; ++r) sums[r] = wave_sum(sums[r]);
-}
+    for (int r = 0; r < ROWS; ++r) sums[r] = wave_sum(sums[r]);
+  }
+};
 
 template <typename T>
 __device__ __forceinline__ void cache_store(const DenseGemvArgs &a, uint32_t n, float v) {
@@ -179,17 +217,17 @@ __global__ __launch_bounds__(256) void dense_gemv_kernel(DenseGemvArgs a) {
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   constexpr int OUTPUTS = GATED ? ROWS / 2 : ROWS;
   const uint32_t first = (blockIdx.x * kWaves + wave) * OUTPUTS;
-  stage_activation<T>(a, xs, plane, scratch);
-  if (first >= a.n) return;
-  const __bf16 *rows[ROWS];
+  RowStream<ROWS, VEC> stream;
 #pragma unroll
   for (int r = 0; r < ROWS; ++r) {
     const uint16_t *matrix = GATED && (r & 1) ? a.w_up : a.w;
     const uint32_t n = min(first + (GATED ? r / 2 : r), a.n - 1);
-    rows[r] = reinterpret_cast<const __bf16 *>(matrix) + (size_t)n * a.k;
+    stream.rows[r] = reinterpret_cast<const __bf16 *>(matrix) + (size_t)n * a.k;
   }
-  float sums[ROWS];
-  dot_rows<ROWS, VEC>(rows, xs, plane, a.k, lane, sums);
+  stage_activation<T>(a, xs, plane, scratch, [&] { stream.request(a.k, lane); });
+  if (first >= a.n) return;
+  stream.run(xs, plane, a.k, lane);
+  const float(&sums)[ROWS] = stream.sums;
   float mine = 0.0f, up = 0.0f;
 #pragma unroll
   for (int o = 0; o < OUTPUTS; ++o)
@@ -274,7 +312,7 @@ __global__ __launch_bounds__(256) void moe_gemv_up_kernel(MoeGemvArgs a) {
   in.norm_groups = 1;
   in.epsilon = a.epsilon;
   in.k = a.width;
-  stage_activation<T>(in, xs, plane, scratch);
+  stage_activation<T>(in, xs, plane, scratch, [] {});
   uint32_t expert = 0;
   if (!shared) {
     select_experts<256>(a.logits, a.experts, a.top, z, ids, weights);
@@ -285,12 +323,13 @@ __global__ __launch_bounds__(256) void moe_gemv_up_kernel(MoeGemvArgs a) {
   if (first >= n_total) return;
   const uint16_t *gate = shared ? a.shared_gate : a.gate + (size_t)expert * a.ff * a.width;
   const uint16_t *up = shared ? a.shared_up : a.up + (size_t)expert * a.ff * a.width;
-  const __bf16 *rows[4];
+  RowStream<4, VEC> stream;
 #pragma unroll
   for (int r = 0; r < 4; ++r)
-    rows[r] = reinterpret_cast<const __bf16 *>((r & 1) ? up : gate) + (size_t)min(first + r / 2, n_total - 1) * a.width;
-  float sums[4];
-  dot_rows<4, VEC>(rows, xs, plane, a.width, lane, sums);
+    stream.rows[r] = reinterpret_cast<const __bf16 *>((r & 1) ? up : gate) + (size_t)min(first + r / 2, n_total - 1) * a.width;
+  stream.request(a.width, lane);
+  stream.run(xs, plane, a.width, lane);
+  const float(&sums)[4] = stream.sums;
   const float g = lane == 0 ? sums[0] : sums[2], u = lane == 0 ? sums[1] : sums[3];
   if (lane < 2 && first + lane < n_total)
     a.hidden[(size_t)blockIdx.y * a.ff + first + lane] = gate_activation(g, a.activation) * u;

@@ -40,6 +40,7 @@ struct SsmWorkspace {
   void *b, *c;    // T [chunks * Q][groups * np]
   float *dt;      // [chunks][heads][Q]
   float *sum;     // [chunks][heads][2][Q] (high parts, low parts)
+  float *tail;    // [chunks][heads][Q]: dt times the decay to the chunk's end
   float *scores;  // [chunks][groups][Q][Q]
   uint32_t chunks, inner, np;
   size_t bytes;
@@ -66,6 +67,7 @@ SsmWorkspace layout(const SsmArgs &a) {
   w.c = take(tokens * a.groups * w.np * element);
   w.dt = static_cast<float *>(take(tokens * a.heads * 4));
   w.sum = static_cast<float *>(take(tokens * a.heads * 8));
+  w.tail = static_cast<float *>(take(tokens * a.heads * 4));
   w.scores = static_cast<float *>(take((size_t)w.chunks * a.groups * Q * Q * 4));
   w.bytes = at;
   return w;
@@ -116,7 +118,8 @@ __global__ __launch_bounds__(256) void ssm_step_kernel(SsmArgs a) {
 
 // ---- many tokens ----------------------------------------------------------------------------------------
 
-template <typename T>
+// TAPS: the convolution's length (0: any length, its inputs read once per tap).
+template <typename T, int TAPS>
 __global__ __launch_bounds__(256) void ssm_conv_kernel(SsmArgs a, SsmWorkspace w) {
   const uint32_t n = a.state_size, channels = w.inner + 2 * a.groups * n;
   const uint32_t padded = w.inner + 2 * a.groups * w.np;
@@ -144,17 +147,26 @@ __global__ __launch_bounds__(256) void ssm_conv_kernel(SsmArgs a, SsmWorkspace w
     float sum[kConvTokens];
 #pragma unroll
     for (int i = 0; i < kConvTokens; ++i) sum[i] = bias;
-    for (uint32_t back = 0; back < a.taps; ++back) {
-      const float weight = bf16_at(a.conv, (size_t)channel * a.taps + a.taps - 1 - back);
+    // the input of token t (negative: before the step)
+    auto at = [&](int t) {
+      if (t >= 0) return t < (int)a.m ? to_f32(input[(size_t)t * ld]) : 0.0f;
+      return (int64_t)position + t >= 0 ? ring[(size_t)((position + t) % a.taps) * channels] : 0.0f;
+    };
+    if (TAPS > 0) {
+      float window[kConvTokens + TAPS - 1];
 #pragma unroll
-      for (int i = 0; i < kConvTokens; ++i) {
-        const uint32_t t = t0 + i;
-        float v = 0.0f;
-        if (t < a.m) {
-          if (t >= back) v = to_f32(input[(size_t)(t - back) * ld]);
-          else if (position + t >= back) v = ring[(size_t)((position + t - back) % a.taps) * channels];
-        }
-        sum[i] = fmaf(weight, v, sum[i]);
+      for (int i = 0; i < kConvTokens + TAPS - 1; ++i) window[i] = at((int)t0 + i - (TAPS - 1));
+#pragma unroll
+      for (int tap = 0; tap < TAPS; ++tap) {
+        const float weight = bf16_at(a.conv, (size_t)channel * TAPS + tap);
+#pragma unroll
+        for (int i = 0; i < kConvTokens; ++i) sum[i] = fmaf(weight, window[i + tap], sum[i]);
+      }
+    } else {
+      for (uint32_t tap = 0; tap < a.taps; ++tap) {
+        const float weight = bf16_at(a.conv, (size_t)channel * a.taps + tap);
+#pragma unroll
+        for (int i = 0; i < kConvTokens; ++i) sum[i] = fmaf(weight, at((int)t0 + i - (int)(a.taps - 1 - tap)), sum[i]);
       }
     }
 #pragma unroll
@@ -183,31 +195,35 @@ __global__ __launch_bounds__(256) void ssm_conv_kernel(SsmArgs a, SsmWorkspace w
   }
 }
 
-// Blocks [0, chunks): softplus and running sums, a thread a head.  The blocks behind: the step's last
-// `taps` convolution inputs into the ring.
+// Blocks [0, chunks * ceil(heads / 4)): softplus and running sums, a wave a head and a lane a token.  The
+// blocks behind: the step's last `taps` convolution inputs into the ring.
 template <typename T>
 __global__ __launch_bounds__(256) void ssm_prepare_kernel(SsmArgs a, SsmWorkspace w) {
-  if (blockIdx.x < w.chunks) {
-    for (uint32_t head = threadIdx.x; head < a.heads; head += 256) {
-      const double rate = -(double)expf(bf16_at(a.a_log, head));
-      const float bias = bf16_at(a.dt_bias, head);
-      float *dt = w.dt + ((size_t)blockIdx.x * a.heads + head) * Q;
-      float *sum = w.sum + ((size_t)blockIdx.x * a.heads + head) * 2 * Q;
-      double running = 0.0;
-      for (int j = 0; j < Q; ++j) {
-        const uint32_t t = blockIdx.x * Q + j;
-        const float step = t < a.m ? softplus_f32(a.dt[(size_t)t * a.heads + head] + bias) : 0.0f;
-        running += rate * (double)step;
-        dt[j] = step;
-        const float high = (float)running;
-        sum[j] = high;
-        sum[Q + j] = (float)(running - (double)high);
-      }
+  const uint32_t head_blocks = (a.heads + 3) / 4;
+  if (blockIdx.x < w.chunks * head_blocks) {
+    const uint32_t chunk = blockIdx.x / head_blocks, head = blockIdx.x % head_blocks * 4 + (threadIdx.x >> 6);
+    if (head >= a.heads) return;
+    const int j = threadIdx.x & 63;
+    const uint32_t t = chunk * Q + j;
+    const float bias = bf16_at(a.dt_bias, head);
+    const float step = t < a.m ? softplus_f32(a.dt[(size_t)t * a.heads + head] + bias) : 0.0f;
+    double running = -(double)expf(bf16_at(a.a_log, head)) * (double)step;
+#pragma unroll
+    for (int d = 1; d < 64; d <<= 1) {
+      const double before = __shfl_up(running, d, 64);
+      if (j >= d) running += before;
     }
+    const double end = __shfl(running, 63, 64);
+    const size_t at = (size_t)chunk * a.heads + head;
+    const float high = (float)running;
+    w.dt[at * Q + j] = step;
+    w.tail[at * Q + j] = step * __expf((float)(end - running));
+    w.sum[at * 2 * Q + j] = high;
+    w.sum[at * 2 * Q + Q + j] = (float)(running - (double)high);
     return;
   }
   const uint32_t channels = w.inner + 2 * a.groups * a.state_size;
-  const uint32_t t = a.m - 1 - (blockIdx.x - w.chunks), position = a.step[kStatePosition] + t;
+  const uint32_t t = a.m - 1 - (blockIdx.x - w.chunks * head_blocks), position = a.step[kStatePosition] + t;
   float *ring = a.conv_state + ((size_t)a.step[kStateSlot] * a.taps + position % a.taps) * channels;
   const T *input = static_cast<const T *>(a.projected) + (size_t)t * (w.inner + channels) + w.inner;
   for (uint32_t c = threadIdx.x; c < channels; c += 256) ring[c] = to_f32(input[c]);
@@ -244,13 +260,14 @@ struct ChunkOperands {
   Frag<T> c[2 * NT];     // c rows of the wave's 16 tokens, np / 32 steps (np <= 64 NT)
   Frag<T> x[2];          // x^T of the 16 state rows, 32 tokens each
   Frag<T> b[NT][2];      // b^T of the wave's state columns
-  f32x8 score[2], dt[2], high[2], low[2];
-  float own_high, own_low, end_high, end_low;
+  f32x8 score[2], dt[2], tail[2], high[2];
+  f32x8 low[sizeof(T) == 4 ? 2 : 1];  // bf16 does without the running sums' low parts
+  float own_high, own_low, end;
 };
 
 // NT: 16-column tiles of the state a wave owns (state_size <= 64 NT).
 template <typename T, int NT>
-__global__ __launch_bounds__(256) void ssm_scan_kernel(SsmArgs a, SsmWorkspace w) {
+__global__ __launch_bounds__(256, 1) void ssm_scan_kernel(SsmArgs a, SsmWorkspace w) {
   constexpr int STRIDE = 64 * NT + 4;
   __shared__ __attribute__((aligned(16))) float states[2][16 * STRIDE];
   const uint32_t head = blockIdx.x, v0 = blockIdx.y * 16, group = head / (a.heads / a.groups);
@@ -281,14 +298,16 @@ __global__ __launch_bounds__(256) void ssm_scan_kernel(SsmArgs a, SsmWorkspace w
     const T *x = static_cast<const T *>(w.xt) + ((size_t)chunk * w.inner + head * a.vdim + v_row) * Q + quad * 8;
     const float *score = w.scores + (((size_t)chunk * a.groups + group) * Q + token) * Q + quad * 8;
     const float *dt = w.dt + ((size_t)chunk * a.heads + head) * Q;
+    const float *tail = w.tail + ((size_t)chunk * a.heads + head) * Q;
     const float *sum = w.sum + ((size_t)chunk * a.heads + head) * 2 * Q;
 #pragma unroll
     for (int s = 0; s < 2; ++s) {
       o.x[s] = *reinterpret_cast<const Frag<T> *>(x + s * 32);
       o.score[s] = *reinterpret_cast<const f32x8 *>(score + s * 32);
       o.dt[s] = *reinterpret_cast<const f32x8 *>(dt + s * 32 + quad * 8);
+      o.tail[s] = *reinterpret_cast<const f32x8 *>(tail + s * 32 + quad * 8);
       o.high[s] = *reinterpret_cast<const f32x8 *>(sum + s * 32 + quad * 8);
-      o.low[s] = *reinterpret_cast<const f32x8 *>(sum + Q + s * 32 + quad * 8);
+      if (sizeof(T) == 4) o.low[s] = *reinterpret_cast<const f32x8 *>(sum + Q + s * 32 + quad * 8);
 #pragma unroll
       for (int t = 0; t < NT; ++t) {
         const uint32_t k = (wave + 4 * t) * 16 + column;
@@ -299,8 +318,7 @@ __global__ __launch_bounds__(256) void ssm_scan_kernel(SsmArgs a, SsmWorkspace w
     }
     o.own_high = sum[token];
     o.own_low = sum[Q + token];
-    o.end_high = sum[Q - 1];
-    o.end_low = sum[2 * Q - 1];
+    o.end = sum[Q - 1];
   };
 
   auto step = [&](const ChunkOperands<T, NT> &o, uint32_t chunk) {
@@ -325,7 +343,7 @@ __global__ __launch_bounds__(256) void ssm_scan_kernel(SsmArgs a, SsmWorkspace w
         }
         y = mma_wide(fs, o.c[s], y);
       }
-    const float scale = __expf(o.own_high + o.own_low);
+    const float scale = __expf(o.own_high);
 #pragma unroll
     for (int r = 0; r < 4; ++r) y[r] *= scale;
 #pragma unroll
@@ -335,13 +353,15 @@ __global__ __launch_bounds__(256) void ssm_scan_kernel(SsmArgs a, SsmWorkspace w
 #pragma unroll
       for (int e = 0; e < 8; ++e) {
         const int j = s * 32 + quad * 8 + e;
-        const float weight = __expf((o.own_high - o.high[s][e]) + (o.own_low - o.low[s][e])) * o.dt[s][e];
-        fp.set(e, j <= token ? o.score[s][e] * weight : 0.0f);
+        const float weight = __expf(sizeof(T) == 4 ? (o.own_high - o.high[s][e]) + (o.own_low - o.low[s][e])
+                                              : o.own_high - o.high[s][e]) * o.dt[s][e];
+        // the skip connection is one more weight on the token's own input
+        fp.set(e, j > token ? 0.0f : fmaf(o.score[s][e], weight, j == token ? skip : 0.0f));
       }
       y = mma_wide_b(o.x[s], fp, y);
     }
     // the new state
-    const float carry = __expf(o.end_high + o.end_low);
+    const float carry = __expf(o.end);
 #pragma unroll
     for (int t = 0; t < NT; ++t)
 #pragma unroll
@@ -351,19 +371,18 @@ __global__ __launch_bounds__(256) void ssm_scan_kernel(SsmArgs a, SsmWorkspace w
       WideFrag<T> fx;
 #pragma unroll
       for (int e = 0; e < 8; ++e)
-        fx.set(e, to_f32(o.x[s][e]) * o.dt[s][e] * __expf((o.end_high - o.high[s][e]) + (o.end_low - o.low[s][e])));
+        fx.set(e, to_f32(o.x[s][e]) * o.tail[s][e]);
 #pragma unroll
       for (int t = 0; t < NT; ++t)
         if ((wave + 4 * t) * 16 < (int)w.np) state[t] = mma_wide(fx, o.b[t][s], state[t]);
     }
     const uint32_t row = chunk * Q + token;
     if (row < a.m) {
-      const T *x = static_cast<const T *>(w.xt) + ((size_t)chunk * w.inner + head * a.vdim) * Q + token;
       T *out = static_cast<T *>(a.y) + (size_t)row * w.inner + head * a.vdim;
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const uint32_t v = v0 + quad * 4 + r;
-        if (v < a.vdim) out[v] = (T)(y[r] + skip * to_f32(x[(size_t)v * Q]));
+        if (v < a.vdim) out[v] = (T)y[r];
       }
     }
   };
@@ -372,9 +391,11 @@ __global__ __launch_bounds__(256) void ssm_scan_kernel(SsmArgs a, SsmWorkspace w
   load(even, 0);
   for (uint32_t chunk = 0; chunk < w.chunks; chunk += 2) {
     if (chunk + 1 < w.chunks) load(odd, chunk + 1);
+    __builtin_amdgcn_sched_barrier(0);  // the requests stay ahead of the arithmetic
     step(even, chunk);
     if (chunk + 1 < w.chunks) {
       if (chunk + 2 < w.chunks) load(even, chunk + 2);
+      __builtin_amdgcn_sched_barrier(0);
       step(odd, chunk + 1);
     }
   }
@@ -391,9 +412,12 @@ template <typename T>
 hipError_t run_prefill(const SsmArgs &a, hipStream_t stream) {
   const SsmWorkspace w = layout(a);
   const uint32_t padded = w.inner + 2 * a.groups * w.np;
-  ssm_conv_kernel<T><<<dim3((padded + 255) / 256, w.chunks * Q / kConvTokens), 256, 0, stream>>>(a, w);
+  const dim3 conv_grid((padded + 255) / 256, w.chunks * Q / kConvTokens);
+  if (a.taps == 4) ssm_conv_kernel<T, 4><<<conv_grid, 256, 0, stream>>>(a, w);
+  else if (a.taps == 3) ssm_conv_kernel<T, 3><<<conv_grid, 256, 0, stream>>>(a, w);
+  else ssm_conv_kernel<T, 0><<<conv_grid, 256, 0, stream>>>(a, w);
   if (hipError_t status = hipGetLastError()) return status;
-  ssm_prepare_kernel<T><<<w.chunks + std::min(a.m, a.taps), 256, 0, stream>>>(a, w);
+  ssm_prepare_kernel<T><<<w.chunks * ((a.heads + 3) / 4) + std::min(a.m, a.taps), 256, 0, stream>>>(a, w);
   if (hipError_t status = hipGetLastError()) return status;
   ssm_scores_kernel<T><<<dim3(w.chunks, a.groups), 256, 0, stream>>>(a, w);
   if (hipError_t status = hipGetLastError()) return status;

@@ -646,7 +646,8 @@ int rms_routed_ffn_add(llmopt_hip_context *context, const DispatchRecord &record
   plan.experts = experts;
   plan.top = top;
   plan.ld_logits = columns;
-  plan.max_tiles = route_max_tiles(m, experts, top);
+  plan.tile = route_tile_rows(m, experts, top, width, ff, F32);
+  plan.max_tiles = route_max_tiles(m, experts, top, plan.tile);
   const size_t normed = scratch.want((size_t)m * width * kElement<F32>);
   const size_t hidden = scratch.want(std::max(pairs * ff, (size_t)m * shared_ff) * kElement<F32>);
   const size_t rows = scratch.want(pairs * width * kElement<F32>);
@@ -683,6 +684,7 @@ int rms_routed_ffn_add(llmopt_hip_context *context, const DispatchRecord &record
   up.tile_first = plan.tile_first;
   up.tile_rows = plan.tile_rows;
   up.tiles = plan.max_tiles;
+  up.tile = plan.tile;
   up.row_source = plan.row_token;
   if (int status = launched(launch_dense_gemm(up, context->stream), name)) return status;
   DenseLinearArgs down = linear(F32, scratch.at<void>(hidden), as_bf16(record.buffers[5]), (uint32_t)pairs, width, ff);
@@ -693,6 +695,7 @@ int rms_routed_ffn_add(llmopt_hip_context *context, const DispatchRecord &record
   down.tile_first = plan.tile_first;
   down.tile_rows = plan.tile_rows;
   down.tiles = plan.max_tiles;
+  down.tile = plan.tile;
   if (int status = launched(launch_dense_gemm(down, context->stream), name)) return status;
   RouteCombineArgs combine = {F32, &plan, scratch.at<void>(rows), stream, width};
   if (int status = launched(launch_route_combine(combine, context->stream), name)) return status;
