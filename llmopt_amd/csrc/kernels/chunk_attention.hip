@@ -14,7 +14,8 @@
 //    follows: probabilities never leave their lane.  Caps of at most kFixedMaxCap bound the exponent, so
 //    the running maximum (and the rescaling) is dropped for a constant one.
 //  * chunk_decode_kernel: one token.  A workgroup takes kSplitKeys keys of one key / value head for all
-//    query heads on it; chunk_merge_kernel joins the splits when the ring is longer than one.
+//    query heads on it, which are the operand columns; chunk_merge_kernel joins the splits when the ring is
+//    longer than one.
 #include <algorithm>
 
 #include "dense.h"
@@ -31,11 +32,6 @@ constexpr float kLog2e = 1.4426950408889634f;
 
 __device__ __forceinline__ uint32_t chunk_start(uint32_t position, uint32_t chunk) {
   return chunk ? position - position % chunk : 0;
-}
-
-__device__ __forceinline__ float capped(float s, float scale, float cap, float inverse_cap) {
-  s *= scale;
-  return cap > 0.0f ? cap * tanh_f32(s * inverse_cap) : s;
 }
 
 // Values of four keys (rows of the stage) at the lane's column: what the V^T operand takes.  bf16: the
@@ -311,137 +307,138 @@ __global__ __launch_bounds__(256) void chunk_cache_write_kernel(ChunkAttentionAr
   }
 }
 
-// KP, VP: 64-wide parts of a key and of a value row.  Eight lanes a row, 32 rows a pass, four passes: all of a
-// split's keys and values are requested before the first is used.  Partial results [heads][splits][vdim + 2]
-// (weighted sum, maximum, total).
-constexpr int kPasses = (int)kSplitKeys / 32;
-constexpr int kHeadBlock = 4;  // query heads that share one pass over the values
+// One token: the query heads of one key / value head are the operand columns (16 at a time), a wave takes 32
+// keys of the workgroup's 128; all keys and values of a split are requested before the first is used.  The
+// values pass through a wave's own LDS rows on the way to their transposed operand.  Partial results
+// [heads][splits][vdim + 2] (weighted sum, maximum, total), or the output when there is one split.
+template <typename T, int NE>
+constexpr int decode_lds_floats() {
+  return 4 * 32 * value_stride<T, NE>() * (int)sizeof(T) / 4 + 2 * 4 * 16;
+}
 
-template <typename T, int KP, int VP>
+template <typename T, int ND, int NE>
 __global__ __launch_bounds__(256) void chunk_decode_kernel(ChunkAttentionArgs a, uint32_t splits) {
-  extern __shared__ __attribute__((aligned(16))) float shared[];
+  constexpr int EP = NE * 16, SV = value_stride<T, NE>(), V_PIECES = EP / 8;
+  extern __shared__ __attribute__((aligned(16))) char lds[];
   const uint32_t position = a.state[kStatePosition], slot = a.state[kStateSlot];
   const uint32_t group = blockIdx.x, split = blockIdx.y, per = a.heads / a.kv_heads;
-  const uint32_t low = chunk_start(position, a.cache.chunk);
-  const uint32_t begin = low + split * kSplitKeys;
+  const uint32_t begin = chunk_start(position, a.cache.chunk) + split * kSplitKeys;
   if (begin > position) return;
-  const uint32_t keys = min(kSplitKeys, position + 1 - begin);
-  const uint32_t dim8 = (a.dim + 7) & ~7u;
-  float *q = shared;                         // [per][dim8]
-  float *scores = q + per * dim8;            // [per][kSplitKeys]
-  float *reduce = scores + per * kSplitKeys;  // [4][kHeadBlock][VP * 64]
-  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, sub = tid & 7;
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, column = lane & 15, quad = lane >> 4;
+  // a wave's own rows: the values [32][SV], then its sums [16][EP] in their place
+  constexpr int OWN = 32 * SV * (int)sizeof(T);
+  static_assert(16 * EP * 4 <= OWN, "the sums fit the values' place");
+  T *lds_v = reinterpret_cast<T *>(lds + wave * OWN);
+  float *lds_top = reinterpret_cast<float *>(lds + 4 * OWN), *lds_total = lds_top + 4 * 16;  // [4][16] each
   const bool vec = a.dim % 8 == 0 && a.vdim % 8 == 0;
   const size_t ring = ((size_t)slot * a.kv_heads + group) * a.cache.capacity;
   const T *cache_k = static_cast<const T *>(a.cache.keys) + ring * a.dim;
   const T *cache_v = static_cast<const T *>(a.cache.values) + ring * a.vdim;
+  const uint32_t wave_begin = begin + wave * 32;
 
-  Frag<T> k[kPasses][KP], v[kPasses][VP];
+  Frag<T> fk[2][ND], reg_v[NE];
 #pragma unroll
-  for (int pass = 0; pass < kPasses; ++pass) {
-    const uint32_t j = (begin + min((uint32_t)(pass * 32 + (tid >> 3)), keys - 1)) % a.cache.capacity;
+  for (int kt = 0; kt < 2; ++kt) {
+    const T *row = cache_k + (size_t)(min(wave_begin + kt * 16 + column, position) % a.cache.capacity) * a.dim;
 #pragma unroll
-    for (int p = 0; p < KP; ++p) {
-      const int c = (p * 8 + sub) * 8;
-      k[pass][p] = load_piece(cache_k + (size_t)j * a.dim + c, (int)a.dim - c, vec);
-    }
+    for (int d = 0; d < ND; ++d) fk[kt][d] = load_piece(row + d * 32 + quad * 8, (int)a.dim - (d * 32 + quad * 8), vec);
   }
 #pragma unroll
-  for (int pass = 0; pass < kPasses; ++pass) {
-    const uint32_t j = (begin + min((uint32_t)(pass * 32 + (tid >> 3)), keys - 1)) % a.cache.capacity;
-#pragma unroll
-    for (int p = 0; p < VP; ++p) {
-      const int c = (p * 8 + sub) * 8;
-      v[pass][p] = load_piece(cache_v + (size_t)j * a.vdim + c, (int)a.vdim - c, vec);
-    }
+  for (int i = 0; i < NE; ++i) {
+    const int index = i * 64 + lane, row = index / V_PIECES, piece = (index % V_PIECES) * 8;
+    const uint32_t j = min(wave_begin + row, position) % a.cache.capacity;
+    reg_v[i] = load_piece(cache_v + (size_t)j * a.vdim + piece, (int)a.vdim - piece, vec);
   }
-  for (uint32_t i = tid; i < per * dim8; i += 256) {
-    const uint32_t h = i / dim8, c = i % dim8;
-    q[i] = c < a.dim ? to_f32(static_cast<const T *>(a.qkv)[(group * per + h) * a.dim + c]) : 0.0f;
-  }
-  __syncthreads();
-  const float inverse_cap = a.softcap > 0.0f ? 1.0f / a.softcap : 0.0f;
-  for (uint32_t h = 0; h < per; ++h) {
-    float dot[kPasses];
+  const bool capped = a.softcap > 0.0f;
+  const float cap = a.softcap * kLog2e;
+  const float inner = capped ? 2.0f * a.scale / a.softcap * kLog2e : a.scale * kLog2e;
+
+  for (uint32_t h0 = 0; h0 < per; h0 += 16) {
+    const uint32_t head = group * per + min(h0 + column, per - 1);
+    Frag<T> fq[ND];
 #pragma unroll
-    for (int pass = 0; pass < kPasses; ++pass) dot[pass] = 0.0f;
+    for (int d = 0; d < ND; ++d)
+      fq[d] = load_piece(static_cast<const T *>(a.qkv) + (size_t)head * a.dim + d * 32 + quad * 8,
+                         (int)a.dim - (d * 32 + quad * 8), vec);
+    f32x4 score[2];
+    float best = -1e30f;
 #pragma unroll
-    for (int p = 0; p < KP; ++p) {
-      const uint32_t c = (p * 8 + sub) * 8;
-      if (c >= dim8) continue;
-      const f32x4 lo = *reinterpret_cast<const f32x4 *>(q + h * dim8 + c);
-      const f32x4 hi = *reinterpret_cast<const f32x4 *>(q + h * dim8 + c + 4);
+    for (int kt = 0; kt < 2; ++kt) {
+      score[kt] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
 #pragma unroll
-      for (int pass = 0; pass < kPasses; ++pass)
+      for (int d = 0; d < ND; ++d) score[kt] = mma(fk[kt][d], fq[d], score[kt]);
 #pragma unroll
-        for (int e = 0; e < 4; ++e) {
-          dot[pass] = fmaf(to_f32(k[pass][p][e]), lo[e], dot[pass]);
-          dot[pass] = fmaf(to_f32(k[pass][p][4 + e]), hi[e], dot[pass]);
-        }
+      for (int r = 0; r < 4; ++r) {
+        float s = score[kt][r] * inner;
+        if (capped) s = fmaf(-2.0f * cap, __builtin_amdgcn_rcpf(1.0f + exp2_raw(s)), cap);
+        if (wave_begin + kt * 16 + quad * 4 + r > position) s = -INFINITY;
+        score[kt][r] = s;
+        best = fmaxf(best, s);
+      }
     }
+    best = fmaxf(best, __shfl_xor(best, 16, 64));
+    best = fmaxf(best, __shfl_xor(best, 32, 64));
+    if (quad == 0) lds_top[wave * 16 + column] = best;
 #pragma unroll
-    for (int pass = 0; pass < kPasses; ++pass) {
-      float s = dot[pass];
-      s += __shfl_xor(s, 1, 64);
-      s += __shfl_xor(s, 2, 64);
-      s += __shfl_xor(s, 4, 64);
-      const uint32_t index = pass * 32 + (tid >> 3);
-      if (sub == 0)
-        scores[h * kSplitKeys + index] = index < keys ? capped(s, a.scale, a.softcap, inverse_cap) : -INFINITY;
-    }
-  }
-  __syncthreads();
-  for (uint32_t h0 = 0; h0 < per; h0 += kHeadBlock) {
-    float best[kHeadBlock], total[kHeadBlock];
-#pragma unroll
-    for (int h = 0; h < kHeadBlock; ++h) {
-      const float *row = scores + min(h0 + h, per - 1) * kSplitKeys;
-      const float s0 = row[lane], s1 = row[64 + lane];
-      best[h] = wave_max(fmaxf(s0, s1));
-      total[h] = wave_sum(__expf(s0 - best[h]) + __expf(s1 - best[h]));
-      float p[kPasses];
-#pragma unroll
-      for (int pass = 0; pass < kPasses; ++pass) p[pass] = __expf(row[pass * 32 + (tid >> 3)] - best[h]);
-      // the lane's columns over its four keys, then over the eight rows of the wave
-#pragma unroll
-      for (int piece = 0; piece < VP; ++piece)
-#pragma unroll
-        for (int e = 0; e < 8; ++e) {
-          float sum = 0.0f;
-#pragma unroll
-          for (int pass = 0; pass < kPasses; ++pass) sum = fmaf(p[pass], to_f32(v[pass][piece][e]), sum);
-          sum += __shfl_xor(sum, 8, 64);
-          sum += __shfl_xor(sum, 16, 64);
-          sum += __shfl_xor(sum, 32, 64);
-          if (lane < 8) reduce[(wave * kHeadBlock + h) * VP * 64 + (piece * 8 + sub) * 8 + e] = sum;
-        }
+    for (int i = 0; i < NE; ++i) {
+      const int index = i * 64 + lane;
+      *reinterpret_cast<Frag<T> *>(lds_v + index / V_PIECES * SV + (index % V_PIECES) * 8) = reg_v[i];
     }
     __syncthreads();
-    for (uint32_t i = tid; i < kHeadBlock * VP * 64; i += 256) {
-      const uint32_t h = i / (VP * 64), c = i % (VP * 64);
-      if (h0 + h >= per || c >= a.vdim) continue;
-      float sum = 0.0f;
 #pragma unroll
-      for (int w = 0; w < 4; ++w) sum += reduce[(w * kHeadBlock + h) * VP * 64 + c];
-      float b = best[0], t = total[0];
+    for (int w = 0; w < 4; ++w) best = fmaxf(best, lds_top[w * 16 + column]);
+    Frag<T> fp;
+    float total = 0.0f;
 #pragma unroll
-      for (int other = 1; other < kHeadBlock; ++other)
-        if ((int)h == other) {
-          b = best[other];
-          t = total[other];
-        }
-      const uint32_t head = group * per + h0 + h;
+    for (int kt = 0; kt < 2; ++kt)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const float p = exp2_raw(score[kt][r] - best);
+        total += p;
+        fp[kt * 4 + r] = (T)p;
+      }
+    total += __shfl_xor(total, 16, 64);
+    total += __shfl_xor(total, 32, 64);
+    if (quad == 0) lds_total[wave * 16 + column] = total;
+    f32x4 out[NE];
+#pragma unroll
+    for (int e = 0; e < NE; ++e) {
+      const T *keys = lds_v + quad * 4 * SV + e * 16;
+      const auto first = four_keys(keys, SV, lane), second = four_keys(keys + 16 * SV, SV, lane);
+      const Frag<T> fv = __builtin_shufflevector(first, second, 0, 1, 2, 3, 4, 5, 6, 7);
+      out[e] = mma(fv, fp, f32x4{0.0f, 0.0f, 0.0f, 0.0f});
+    }
+    __syncthreads();  // every read of the values is done
+#pragma unroll
+    for (int e = 0; e < NE; ++e)
+      *reinterpret_cast<f32x4 *>(lds + wave * OWN + (column * EP + e * 16 + quad * 4) * 4) = out[e];
+    __syncthreads();
+    const uint32_t live = min(16u, per - h0);
+    for (uint32_t i = tid; i < live * EP; i += 256) {
+      const uint32_t h = i / EP, c = i % EP;
+      if (c >= a.vdim) continue;
+      float sum = 0.0f, all = 0.0f, top = -1e30f;
+#pragma unroll
+      for (int w = 0; w < 4; ++w) {
+        sum += *reinterpret_cast<const float *>(lds + w * OWN + (h * EP + c) * 4);
+        all += lds_total[w * 16 + h];
+        top = fmaxf(top, lds_top[w * 16 + h]);
+      }
+      const uint32_t target = group * per + h0 + h;
       if (splits == 1) {
-        const float sink = a.sink ? (float)reinterpret_cast<const __bf16 *>(a.sink)[head] : -INFINITY;
-        const float top = fmaxf(b, sink);
-        const float mine = __expf(b - top);
-        static_cast<T *>(a.out)[head * a.vdim + c] = (T)(sum * mine / (t * mine + __expf(sink - top)));
+        if (a.sink) {
+          const float sink = (float)reinterpret_cast<const __bf16 *>(a.sink)[target] * kLog2e, most = fmaxf(top, sink);
+          const float mine = exp2_raw(top - most);
+          sum *= mine;
+          all = all * mine + exp2_raw(sink - most);
+        }
+        static_cast<T *>(a.out)[target * a.vdim + c] = (T)(sum / all);
       } else {
-        float *partial = static_cast<float *>(a.workspace) + ((size_t)head * splits + split) * (a.vdim + 2);
+        float *partial = static_cast<float *>(a.workspace) + ((size_t)target * splits + split) * (a.vdim + 2);
         partial[c] = sum;
         if (c == 0) {
-          partial[a.vdim] = b;
-          partial[a.vdim + 1] = t;
+          partial[a.vdim] = top;
+          partial[a.vdim + 1] = all;
         }
       }
     }
@@ -449,7 +446,7 @@ __global__ __launch_bounds__(256) void chunk_decode_kernel(ChunkAttentionArgs a,
   }
 }
 
-// A workgroup a head; the splits' weights are formed once, in LDS.
+// A workgroup a head; the splits' weights are formed once, in LDS (maxima are exponents of two).
 template <typename T>
 __global__ __launch_bounds__(256) void chunk_merge_kernel(ChunkAttentionArgs a, uint32_t splits) {
   extern __shared__ __attribute__((aligned(16))) float shared[];
@@ -458,7 +455,7 @@ __global__ __launch_bounds__(256) void chunk_merge_kernel(ChunkAttentionArgs a, 
   const uint32_t live = min(splits, (position - chunk_start(position, a.cache.chunk)) / kSplitKeys + 1);
   const uint32_t stride = a.vdim + 2;
   const float *partial = static_cast<const float *>(a.workspace) + (size_t)head * splits * stride;
-  const float sink = a.sink ? (float)reinterpret_cast<const __bf16 *>(a.sink)[head] : -INFINITY;
+  const float sink = a.sink ? (float)reinterpret_cast<const __bf16 *>(a.sink)[head] * kLog2e : -INFINITY;
   constexpr uint32_t AHEAD = 8;
   const uint32_t c = threadIdx.x;
   float first[AHEAD];  // the first splits' values on their way while the weights are formed
@@ -471,17 +468,17 @@ __global__ __launch_bounds__(256) void chunk_merge_kernel(ChunkAttentionArgs a, 
   __syncthreads();
   float top = sink;
   for (uint32_t s = 0; s < live; ++s) top = fmaxf(top, best[s]);
-  float denominator = __expf(sink - top), sum = 0.0f;
+  float denominator = exp2_raw(sink - top), sum = 0.0f;
 #pragma unroll
   for (uint32_t s = 0; s < AHEAD; ++s)
     if (s < live) {
-      const float weight = __expf(best[s] - top);
+      const float weight = exp2_raw(best[s] - top);
       denominator = fmaf(total[s], weight, denominator);
       sum = fmaf(first[s], weight, sum);
     }
 #pragma unroll 8
   for (uint32_t s = AHEAD; s < live; ++s) {
-    const float weight = __expf(best[s] - top);
+    const float weight = exp2_raw(best[s] - top);
     denominator = fmaf(total[s], weight, denominator);
     if (c < a.vdim) sum = fmaf(partial[s * stride + c], weight, sum);
   }
@@ -493,30 +490,18 @@ uint32_t decode_splits(const ChunkAttentionArgs &a) {
   return (longest + kSplitKeys - 1) / kSplitKeys;
 }
 
-uint32_t decode_lds_bytes(const ChunkAttentionArgs &a) {
-  const uint32_t per = a.heads / a.kv_heads, dim8 = (a.dim + 7) & ~7u;
-  return (per * dim8 + per * kSplitKeys + 4 * kHeadBlock * 256) * 4;
-}
-
-template <typename T, int KP, int VP>
+template <typename T, int ND, int NE>
 hipError_t run_decode(const ChunkAttentionArgs &a, hipStream_t stream) {
   static bool allowed[kMaxDevices] = {};
-  const uint32_t splits = decode_splits(a), bytes = decode_lds_bytes(a);
+  constexpr int bytes = decode_lds_floats<T, NE>() * 4;
+  const uint32_t splits = decode_splits(a);
   if (bytes > 64 * 1024)
-    if (hipError_t status = allow_dynamic_lds(reinterpret_cast<const void *>(chunk_decode_kernel<T, KP, VP>),
-                                              160 * 1024, allowed))
+    if (hipError_t status = allow_dynamic_lds(reinterpret_cast<const void *>(chunk_decode_kernel<T, ND, NE>), bytes, allowed))
       return status;
-  chunk_decode_kernel<T, KP, VP><<<dim3(a.kv_heads, splits), 256, bytes, stream>>>(a, splits);
+  chunk_decode_kernel<T, ND, NE><<<dim3(a.kv_heads, splits), 256, bytes, stream>>>(a, splits);
   if (hipError_t status = hipGetLastError()) return status;
   if (splits > 1) chunk_merge_kernel<T><<<a.heads, 256, splits * 8, stream>>>(a, splits);
   return hipGetLastError();
-}
-
-template <typename T, int KP>
-hipError_t pick_decode(const ChunkAttentionArgs &a, hipStream_t stream) {
-  if (a.vdim <= 64) return run_decode<T, KP, 1>(a, stream);
-  if (a.vdim <= 128) return run_decode<T, KP, 2>(a, stream);
-  return run_decode<T, KP, 4>(a, stream);
 }
 
 template <typename T, int ND, int NE, bool FIXED>
@@ -539,21 +524,21 @@ hipError_t run_prefill(const ChunkAttentionArgs &a, hipStream_t stream) {
   return run_prefill_kernel<T, ND, NE, false>(a, stream);
 }
 
+template <typename T, int ND, int NE>
+hipError_t run_attention(const ChunkAttentionArgs &a, hipStream_t stream) {
+  return a.m == 1 ? run_decode<T, ND, NE>(a, stream) : run_prefill<T, ND, NE>(a, stream);
+}
+
 template <typename T, int ND>
 hipError_t pick_value_width(const ChunkAttentionArgs &a, hipStream_t stream) {
-  if (a.vdim <= 32) return run_prefill<T, ND, 2>(a, stream);
-  if (a.vdim <= 64) return run_prefill<T, ND, 4>(a, stream);
-  if (a.vdim <= 128) return run_prefill<T, ND, 8>(a, stream);
-  return run_prefill<T, ND, 16>(a, stream);
+  if (a.vdim <= 32) return run_attention<T, ND, 2>(a, stream);
+  if (a.vdim <= 64) return run_attention<T, ND, 4>(a, stream);
+  if (a.vdim <= 128) return run_attention<T, ND, 8>(a, stream);
+  return run_attention<T, ND, 16>(a, stream);
 }
 
 template <typename T>
 hipError_t pick_attention(const ChunkAttentionArgs &a, hipStream_t stream) {
-  if (a.m == 1) {
-    if (a.dim <= 64) return pick_decode<T, 1>(a, stream);
-    if (a.dim <= 128) return pick_decode<T, 2>(a, stream);
-    return pick_decode<T, 4>(a, stream);
-  }
   if (a.dim <= 64) return pick_value_width<T, 2>(a, stream);
   if (a.dim <= 128) return pick_value_width<T, 4>(a, stream);
   return pick_value_width<T, 8>(a, stream);
@@ -568,7 +553,7 @@ size_t chunk_attention_workspace_bytes(const ChunkAttentionArgs &a) {
 }
 
 bool chunk_attention_ok(const ChunkAttentionArgs &a) {
-  return a.dim <= 256 && a.vdim <= 256 && decode_lds_bytes(a) <= 160 * 1024 && decode_splits(a) <= 8000;
+  return a.dim <= 256 && a.vdim <= 256 && decode_splits(a) <= 8000;  // (the merge keeps two words a split in LDS)
 }
 
 hipError_t launch_chunk_attention(const ChunkAttentionArgs &a, hipStream_t stream) {

@@ -24,6 +24,44 @@ __device__ __forceinline__ uint32_t staged_index(uint32_t k, uint32_t plane) {
   return ((k >> 2) & 1) * plane + ((k >> 3) << 2) + (k & 3);
 }
 
+// A row of at most PIECES * 1024 values through registers: one trip to memory.
+template <int PIECES, typename Ahead>
+__device__ __forceinline__ void stage_normed_row(const DenseGemvArgs &a, float *xs, uint32_t plane, float *scratch,
+                                                 Ahead ahead) {
+  const uint32_t k = a.k;
+  const float *x = static_cast<const float *>(a.x);
+  const __bf16 *weight = reinterpret_cast<const __bf16 *>(a.norm_weight);
+  f32x4 v[PIECES];
+  bf16x4 w[PIECES];
+  float sum = 0.0f;
+#pragma unroll
+  for (int q = 0; q < PIECES; ++q) {
+    const uint32_t i = (q * kWaves * 64 + threadIdx.x) * 4;
+    v[q] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+    if (i < k) {
+      v[q] = *reinterpret_cast<const f32x4 *>(x + i);
+      w[q] = *reinterpret_cast<const bf16x4 *>(weight + i);
+    }
+  }
+  ahead();
+#pragma unroll
+  for (int q = 0; q < PIECES; ++q)
+    sum += v[q][0] * v[q][0] + v[q][1] * v[q][1] + v[q][2] * v[q][2] + v[q][3] * v[q][3];
+  sum = block_sum<kWaves>(sum, scratch);
+  const float inverse = 1.0f / sqrtf(sum / (float)k + a.epsilon);
+#pragma unroll
+  for (int q = 0; q < PIECES; ++q) {
+    const uint32_t i = (q * kWaves * 64 + threadIdx.x) * 4;
+    if (i < k) {
+      f32x4 out;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) out[e] = v[q][e] * inverse * (float)w[q][e];
+      *reinterpret_cast<f32x4 *>(xs + staged_index(i, plane)) = out;
+    }
+  }
+  __syncthreads();
+}
+
 // Stages the f32 row x, normalised in `groups` parts by norm_weight when that is not null.  `ahead` is
 // called once the row has been requested (loads return in order: what it requests does not delay the row).
 template <typename T, typename Ahead>
@@ -64,38 +102,12 @@ __device__ __forceinline__ void stage_activation(const DenseGemvArgs &a, float *
   }
   const float *x = static_cast<const float *>(a.x);
   const uint32_t part = k / a.norm_groups;
-  constexpr int PIECES = 8;
-  if (a.norm_groups == 1 && (k & 3) == 0 && k <= PIECES * 4 * kWaves * 64) {
-    // the row in registers: one trip to memory
-    f32x4 v[PIECES];
-    bf16x4 w[PIECES];
-    float sum = 0.0f;
-#pragma unroll
-    for (int q = 0; q < PIECES; ++q) {
-      const uint32_t i = (q * kWaves * 64 + threadIdx.x) * 4;
-      v[q] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
-      if (i < k) {
-        v[q] = *reinterpret_cast<const f32x4 *>(x + i);
-        w[q] = *reinterpret_cast<const bf16x4 *>(weight + i);
-      }
-    }
-    ahead();
-#pragma unroll
-    for (int q = 0; q < PIECES; ++q)
-      sum += v[q][0] * v[q][0] + v[q][1] * v[q][1] + v[q][2] * v[q][2] + v[q][3] * v[q][3];
-    sum = block_sum<kWaves>(sum, scratch);
-    const float inverse = 1.0f / sqrtf(sum / (float)k + a.epsilon);
-#pragma unroll
-    for (int q = 0; q < PIECES; ++q) {
-      const uint32_t i = (q * kWaves * 64 + threadIdx.x) * 4;
-      if (i < k) {
-        f32x4 out;
-#pragma unroll
-        for (int e = 0; e < 4; ++e) out[e] = v[q][e] * inverse * (float)w[q][e];
-        *reinterpret_cast<f32x4 *>(xs + staged_index(i, plane)) = out;
-      }
-    }
-    __syncthreads();
+  if (a.norm_groups == 1 && (k & 3) == 0 && k <= 4 * 4 * kWaves * 64) {
+    stage_normed_row<4>(a, xs, plane, scratch, ahead);
+    return;
+  }
+  if (a.norm_groups == 1 && (k & 3) == 0 && k <= 8 * 4 * kWaves * 64) {
+    stage_normed_row<8>(a, xs, plane, scratch, ahead);
     return;
   }
   ahead();
@@ -110,11 +122,11 @@ __device__ __forceinline__ void stage_activation(const DenseGemvArgs &a, float *
   __syncthreads();
 }
 
-// ROWS weight rows streamed against the staged activation in blocks of 2048 columns; the first block is
-// requested by `request`, ahead of the staging.
+// ROWS weight rows streamed against the staged activation in blocks of STEPS * 512 columns; the first block
+// is requested by `request`, ahead of the staging where the rows are known by then.
 template <int ROWS, bool VEC>
 struct RowStream {
-  static constexpr int STEPS = 4;
+  static constexpr int STEPS = ROWS > 4 ? 2 : 4;
   const __bf16 *rows[ROWS];
   bf16x8 w[STEPS][ROWS];
   float sums[ROWS];
@@ -295,7 +307,9 @@ __device__ __forceinline__ void select_experts(const float *logits, uint32_t exp
   __syncthreads();
 }
 
-// blockIdx.y: choice 0 .. top - 1, or `top`: the shared expert.
+// blockIdx.y: choice 0 .. top - 1, or `top`: the shared expert.  A wave owns kUpOutputs hidden values.
+constexpr int kUpOutputs = 4;
+
 template <typename T, bool VEC>
 __global__ __launch_bounds__(256) void moe_gemv_up_kernel(MoeGemvArgs a) {
   extern __shared__ __attribute__((aligned(16))) float lds[];
@@ -305,7 +319,7 @@ __global__ __launch_bounds__(256) void moe_gemv_up_kernel(MoeGemvArgs a) {
   uint32_t *ids = reinterpret_cast<uint32_t *>(weights + a.top);
   const bool shared = blockIdx.y == a.top;
   const uint32_t n_total = shared ? a.shared_ff : a.ff;
-  if (blockIdx.x * kWaves * 2 >= n_total) return;
+  if (blockIdx.x * kWaves * kUpOutputs >= n_total) return;
   DenseGemvArgs in = {};
   in.x = a.x;
   in.norm_weight = a.norm_weight;
@@ -319,58 +333,70 @@ __global__ __launch_bounds__(256) void moe_gemv_up_kernel(MoeGemvArgs a) {
     expert = ids[blockIdx.y];
   }
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
-  const uint32_t first = (blockIdx.x * kWaves + wave) * 2;
+  const uint32_t first = (blockIdx.x * kWaves + wave) * kUpOutputs;
   if (first >= n_total) return;
   const uint16_t *gate = shared ? a.shared_gate : a.gate + (size_t)expert * a.ff * a.width;
   const uint16_t *up = shared ? a.shared_up : a.up + (size_t)expert * a.ff * a.width;
-  RowStream<4, VEC> stream;
+  RowStream<2 * kUpOutputs, VEC> stream;
 #pragma unroll
-  for (int r = 0; r < 4; ++r)
+  for (int r = 0; r < 2 * kUpOutputs; ++r)
     stream.rows[r] = reinterpret_cast<const __bf16 *>((r & 1) ? up : gate) + (size_t)min(first + r / 2, n_total - 1) * a.width;
   stream.request(a.width, lane);
   stream.run(xs, plane, a.width, lane);
-  const float(&sums)[4] = stream.sums;
-  const float g = lane == 0 ? sums[0] : sums[2], u = lane == 0 ? sums[1] : sums[3];
-  if (lane < 2 && first + lane < n_total)
+  float g = 0.0f, u = 0.0f;
+#pragma unroll
+  for (int o = 0; o < kUpOutputs; ++o)
+    if (lane == o) {
+      g = stream.sums[2 * o];
+      u = stream.sums[2 * o + 1];
+    }
+  if (lane < kUpOutputs && first + lane < n_total)
     a.hidden[(size_t)blockIdx.y * a.ff + first + lane] = gate_activation(g, a.activation) * u;
 }
 
 // stream[n] += sum_s weight_s down[expert_s][n] . hidden_s (+ sigmoid(gate) shared_down[n] . hidden_shared).
-// A workgroup owns ROWS columns of the stream; its waves take the choices in turn.
-template <typename T, int ROWS, bool VEC>
-__global__ __launch_bounds__(256) void moe_gemv_down_kernel(MoeGemvArgs a) {
+// A workgroup owns ROWS columns of the stream; its waves take the choices in pieces of 1024 in turn.
+constexpr int kDownWaves = 8;
+
+template <int ROWS, bool VEC>
+__global__ __launch_bounds__(kDownWaves * 64) void moe_gemv_down_kernel(MoeGemvArgs a) {
   extern __shared__ __attribute__((aligned(16))) float lds[];
-  __shared__ float partial[kWaves][ROWS];
+  __shared__ float partial[kDownWaves][ROWS];
   float *z = lds, *weights = z + a.experts;
   uint32_t *ids = reinterpret_cast<uint32_t *>(weights + a.top);
-  select_experts<256>(a.logits, a.experts, a.top, z, ids, weights);
+  select_experts<kDownWaves * 64>(a.logits, a.experts, a.top, z, ids, weights);
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const uint32_t first = blockIdx.x * ROWS;
   float acc[ROWS];
 #pragma unroll
   for (int r = 0; r < ROWS; ++r) acc[r] = 0.0f;
-  const uint32_t choices = a.top + (a.shared_ff ? 1 : 0);
-  for (uint32_t s = wave; s < choices; s += kWaves) {
+  const uint32_t per = (a.ff + 1023) / 1024, units = a.top * per + (a.shared_ff + 1023) / 1024;
+  for (uint32_t unit = wave; unit < units; unit += kDownWaves) {
+    const uint32_t s = min(unit / per, a.top);
     const bool shared = s == a.top;
-    const uint32_t k = shared ? a.shared_ff : a.ff;
+    const uint32_t k = shared ? a.shared_ff : a.ff, k0 = (unit - s * per) * 1024;
     const __bf16 *down = reinterpret_cast<const __bf16 *>(shared ? a.shared_down : a.down + (size_t)ids[s] * a.width * a.ff);
     const float weight = shared ? sigmoid_f32(a.logits[a.experts]) : weights[s];
     const float *hidden = a.hidden + (size_t)s * a.ff;
-    for (uint32_t k0 = 0; k0 < k; k0 += 512) {
-      const uint32_t kk = k0 + lane * 8;
+    f32x8 h[2];
+    bf16x8 w[2][ROWS];
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+      const uint32_t kk = k0 + i * 512 + lane * 8;
       const int count = (int)k - (int)kk;
-      const f32x8 h = load_piece(hidden + kk, count, VEC);
-      bf16x8 w[ROWS];
+      h[i] = load_piece(hidden + kk, count, VEC);
 #pragma unroll
       for (int r = 0; r < ROWS; ++r)
-        w[r] = load_piece(down + (size_t)min(first + r, a.width - 1) * k + kk, count, VEC);
+        w[i][r] = load_piece(down + (size_t)min(first + r, a.width - 1) * k + kk, count, VEC);
+    }
 #pragma unroll
-      for (int r = 0; r < ROWS; ++r) {
-        float sum = 0.0f;
+    for (int r = 0; r < ROWS; ++r) {
+      float sum = 0.0f;
 #pragma unroll
-        for (int e = 0; e < 8; ++e) sum = fmaf((float)w[r][e], h[e], sum);
-        acc[r] = fmaf(weight, sum, acc[r]);
-      }
+      for (int i = 0; i < 2; ++i)
+#pragma unroll
+        for (int e = 0; e < 8; ++e) sum = fmaf((float)w[i][r][e], h[i][e], sum);
+      acc[r] = fmaf(weight, sum, acc[r]);
     }
   }
 #pragma unroll
@@ -382,7 +408,7 @@ __global__ __launch_bounds__(256) void moe_gemv_down_kernel(MoeGemvArgs a) {
   if (threadIdx.x < ROWS && first + threadIdx.x < a.width) {
     float total = 0.0f;
 #pragma unroll
-    for (int w = 0; w < kWaves; ++w) total += partial[w][threadIdx.x];
+    for (int w = 0; w < kDownWaves; ++w) total += partial[w][threadIdx.x];
     a.stream[first + threadIdx.x] += total;
   }
 }
@@ -399,7 +425,7 @@ hipError_t launch_moe_gemv_up(const MoeGemvArgs &a, hipStream_t stream) {
   const uint32_t bytes = ((a.width + 7) / 8) * 32 + (a.experts + 2 * a.top) * 4;
   if (bytes > 60 * 1024) return hipErrorInvalidValue;
   const uint32_t widest = std::max(a.ff, a.shared_ff);
-  const dim3 grid((widest + 2 * kWaves - 1) / (2 * kWaves), a.top + (a.shared_ff ? 1 : 0));
+  const dim3 grid((widest + kUpOutputs * kWaves - 1) / (kUpOutputs * kWaves), a.top + (a.shared_ff ? 1 : 0));
   if (a.width % 8 == 0) moe_gemv_up_kernel<float, true><<<grid, 256, bytes, stream>>>(a);
   else moe_gemv_up_kernel<float, false><<<grid, 256, bytes, stream>>>(a);
   return hipGetLastError();
@@ -410,8 +436,8 @@ hipError_t launch_moe_gemv_down(const MoeGemvArgs &a, hipStream_t stream) {
   const bool vec = a.ff % 8 == 0 && a.shared_ff % 8 == 0;
   constexpr int ROWS = 8;
   const uint32_t grid = (a.width + ROWS - 1) / ROWS;
-  if (vec) moe_gemv_down_kernel<float, ROWS, true><<<grid, 256, bytes, stream>>>(a);
-  else moe_gemv_down_kernel<float, ROWS, false><<<grid, 256, bytes, stream>>>(a);
+  if (vec) moe_gemv_down_kernel<ROWS, true><<<grid, kDownWaves * 64, bytes, stream>>>(a);
+  else moe_gemv_down_kernel<ROWS, false><<<grid, kDownWaves * 64, bytes, stream>>>(a);
   return hipGetLastError();
 }
 

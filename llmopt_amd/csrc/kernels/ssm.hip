@@ -14,9 +14,10 @@
 //  * ssm_prepare_kernel: softplus, the running sums (in double, kept as two floats: their differences
 //    enter an exponential) and the convolution's last inputs into the ring;
 //  * ssm_scores_kernel: c_i . b_j of every chunk and group, shared by the heads of the group;
-//  * ssm_scan_kernel: a workgroup owns 16 state rows of one head and walks the chunks, its slice of the
-//    state in registers.  Operands that must keep float32 accuracy (the state, the decay-weighted
-//    inputs) enter the bfloat16 matrix cores as a high and a low part.
+//  * ssm_state_kernel: the serial part, and nothing else: the state from chunk to chunk, in registers;
+//  * ssm_output_kernel: the outputs of all chunks at once, from the states the serial part left.
+// Operands that must keep float32 accuracy (the state, decay-weighted inputs and scores) enter the bfloat16
+// matrix cores as a high and a low part.
 // The position-0 token starts from a zero state and zero history, whatever a slot held before.
 #include <algorithm>
 
@@ -42,6 +43,7 @@ struct SsmWorkspace {
   float *sum;     // [chunks][heads][2][Q] (high parts, low parts)
   float *tail;    // [chunks][heads][Q]: dt times the decay to the chunk's end
   float *scores;  // [chunks][groups][Q][Q]
+  void *states;   // T [chunks][heads][planes][vdim to 16][np]: every chunk's incoming state, in operand order
   uint32_t chunks, inner, np;
   size_t bytes;
 };
@@ -69,6 +71,7 @@ SsmWorkspace layout(const SsmArgs &a) {
   w.sum = static_cast<float *>(take(tokens * a.heads * 8));
   w.tail = static_cast<float *>(take(tokens * a.heads * 4));
   w.scores = static_cast<float *>(take((size_t)w.chunks * a.groups * Q * Q * 4));
+  w.states = take((size_t)w.chunks * a.heads * ((a.vdim + 15) / 16 * 16) * w.np * 4);  // two bf16 planes or one f32
   w.bytes = at;
   return w;
 }
@@ -254,113 +257,81 @@ __global__ __launch_bounds__(256) void ssm_scores_kernel(SsmArgs a, SsmWorkspace
     *reinterpret_cast<f32x4 *>(scores + (wave * 16 + column) * Q + t * 16 + quad * 4) = acc[t];
 }
 
-// What a wave reads of one chunk, requested a chunk ahead.
+// A chunk's incoming state as the matrix cores take it: float as it is, bf16 as a high and a low plane, in
+// operand order: [16 state rows][32 columns] blocks, lane (column / 8) * 16 + row holding eight columns, so
+// that an operand is one contiguous load and the serial part stores whole lines.
+template <typename T>
+constexpr int kStatePlanes = sizeof(T) == 4 ? 1 : 2;
+template <typename T>
+__device__ __forceinline__ T *state_block(const SsmArgs &a, const SsmWorkspace &w, uint32_t chunk, uint32_t head,
+                                          int plane, uint32_t v0) {
+  const size_t rows = (a.vdim + 15) & ~15u;
+  return static_cast<T *>(w.states) +
+         ((((size_t)chunk * a.heads + head) * kStatePlanes<T> + plane) * rows + v0) * w.np;
+}
+
 template <typename T, int NT>
-struct ChunkOperands {
-  Frag<T> c[2 * NT];     // c rows of the wave's 16 tokens, np / 32 steps (np <= 64 NT)
-  Frag<T> x[2];          // x^T of the 16 state rows, 32 tokens each
-  Frag<T> b[NT][2];      // b^T of the wave's state columns
-  f32x8 score[2], dt[2], tail[2], high[2];
-  f32x8 low[sizeof(T) == 4 ? 2 : 1];  // bf16 does without the running sums' low parts
-  float own_high, own_low, end;
+struct StateOperands {
+  Frag<T> x[2];      // x^T of the 16 state rows, 32 tokens each
+  Frag<T> b[NT][2];  // b^T of the wave's state columns
+  f32x8 tail[2];
+  float end;
 };
 
-// NT: 16-column tiles of the state a wave owns (state_size <= 64 NT).
+// The serial part: a workgroup owns 16 state rows of one head, its waves the 16-column tiles wave + 4 t
+// (state_size <= 64 NT); the chunks' incoming states go to the workspace.  No exchange between waves.
 template <typename T, int NT>
-__global__ __launch_bounds__(256, 1) void ssm_scan_kernel(SsmArgs a, SsmWorkspace w) {
-  constexpr int STRIDE = 64 * NT + 4;
-  __shared__ __attribute__((aligned(16))) float states[2][16 * STRIDE];
+__global__ __launch_bounds__(256, 1) void ssm_state_kernel(SsmArgs a, SsmWorkspace w) {
   const uint32_t head = blockIdx.x, v0 = blockIdx.y * 16, group = head / (a.heads / a.groups);
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, column = lane & 15, quad = lane >> 4;
   const uint32_t n = a.state_size, slot = a.step[kStateSlot];
   const bool fresh = a.step[kStatePosition] == 0;
   const size_t ld = (size_t)a.groups * w.np;
-  const int token = wave * 16 + column;  // the token of the lane's output column
-  // state rows beyond the head's end repeat its last one and are not stored
-  const uint32_t v_row = min(v0 + column, a.vdim - 1);
-  float *saved = a.ssm_state + ((size_t)slot * a.heads + head) * a.vdim * n;
-  const float skip = bf16_at(a.d_skip, head);
+  // lane: state row v, columns k .. k + 3 of every tile; rows beyond the head's end repeat its last one
+  const uint32_t v = v0 + column, v_row = min(v, a.vdim - 1);
+  float *saved = a.ssm_state + (((size_t)slot * a.heads + head) * a.vdim + v_row) * n;
 
   f32x4 state[NT];
 #pragma unroll
   for (int t = 0; t < NT; ++t)
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
-      const uint32_t v = v0 + quad * 4 + r, k = (wave + 4 * t) * 16 + column;
-      state[t][r] = !fresh && v < a.vdim && k < n ? saved[(size_t)v * n + k] : 0.0f;
+      const uint32_t k = (wave + 4 * t) * 16 + quad * 4 + r;
+      state[t][r] = !fresh && k < n ? saved[k] : 0.0f;
     }
 
-  auto load = [&](ChunkOperands<T, NT> &o, uint32_t chunk) {
-    const T *c = static_cast<const T *>(w.c) + ((size_t)chunk * Q + token) * ld + group * w.np + quad * 8;
-#pragma unroll
-    for (int s = 0; s < 2 * NT; ++s)
-      if (s * 32 < (int)w.np) o.c[s] = *reinterpret_cast<const Frag<T> *>(c + s * 32);
+  auto load = [&](StateOperands<T, NT> &o, uint32_t chunk) {
     const T *x = static_cast<const T *>(w.xt) + ((size_t)chunk * w.inner + head * a.vdim + v_row) * Q + quad * 8;
-    const float *score = w.scores + (((size_t)chunk * a.groups + group) * Q + token) * Q + quad * 8;
-    const float *dt = w.dt + ((size_t)chunk * a.heads + head) * Q;
-    const float *tail = w.tail + ((size_t)chunk * a.heads + head) * Q;
-    const float *sum = w.sum + ((size_t)chunk * a.heads + head) * 2 * Q;
+    const float *tail = w.tail + ((size_t)chunk * a.heads + head) * Q + quad * 8;
+    o.end = w.sum[((size_t)chunk * a.heads + head) * 2 * Q + Q - 1];
 #pragma unroll
     for (int s = 0; s < 2; ++s) {
       o.x[s] = *reinterpret_cast<const Frag<T> *>(x + s * 32);
-      o.score[s] = *reinterpret_cast<const f32x8 *>(score + s * 32);
-      o.dt[s] = *reinterpret_cast<const f32x8 *>(dt + s * 32 + quad * 8);
-      o.tail[s] = *reinterpret_cast<const f32x8 *>(tail + s * 32 + quad * 8);
-      o.high[s] = *reinterpret_cast<const f32x8 *>(sum + s * 32 + quad * 8);
-      if (sizeof(T) == 4) o.low[s] = *reinterpret_cast<const f32x8 *>(sum + Q + s * 32 + quad * 8);
+      o.tail[s] = *reinterpret_cast<const f32x8 *>(tail + s * 32);
 #pragma unroll
-      for (int t = 0; t < NT; ++t) {
-        const uint32_t k = (wave + 4 * t) * 16 + column;
+      for (int t = 0; t < NT; ++t)
         if ((wave + 4 * t) * 16 < (int)w.np)
           o.b[t][s] = *reinterpret_cast<const Frag<T> *>(
-              static_cast<const T *>(w.bt) + ((size_t)chunk * ld + group * w.np + k) * Q + s * 32 + quad * 8);
-      }
+              static_cast<const T *>(w.bt) +
+              ((size_t)chunk * ld + group * w.np + (wave + 4 * t) * 16 + column) * Q + s * 32 + quad * 8);
     }
-    o.own_high = sum[token];
-    o.own_low = sum[Q + token];
-    o.end = sum[Q - 1];
   };
-
-  auto step = [&](const ChunkOperands<T, NT> &o, uint32_t chunk) {
-    float *lds = states[chunk & 1];
+  auto step = [&](const StateOperands<T, NT> &o, uint32_t chunk) {
 #pragma unroll
-    for (int t = 0; t < NT; ++t)
+    for (int t = 0; t < NT; ++t) {
+      const uint32_t k = (wave + 4 * t) * 16;
+      if (k >= w.np) continue;
+      typedef T x4 __attribute__((ext_vector_type(4)));
+      x4 high, low;
 #pragma unroll
-      for (int r = 0; r < 4; ++r) lds[(quad * 4 + r) * STRIDE + (wave + 4 * t) * 16 + column] = state[t][r];
-    __syncthreads();
-    // y^T: rows = state rows, column = the lane's token
-    f32x4 y = {0.0f, 0.0f, 0.0f, 0.0f};
-#pragma unroll
-    for (int s = 0; s < 2 * NT; ++s)
-      if (s * 32 < (int)w.np) {
-        WideFrag<T> fs;
-        const float *row = lds + column * STRIDE + s * 32 + quad * 8;
-        const f32x4 lo = *reinterpret_cast<const f32x4 *>(row), hi = *reinterpret_cast<const f32x4 *>(row + 4);
-#pragma unroll
-        for (int e = 0; e < 4; ++e) {
-          fs.set(e, lo[e]);
-          fs.set(4 + e, hi[e]);
-        }
-        y = mma_wide(fs, o.c[s], y);
+      for (int r = 0; r < 4; ++r) {
+        high[r] = (T)state[t][r];
+        low[r] = (T)(state[t][r] - (float)high[r]);
       }
-    const float scale = __expf(o.own_high);
-#pragma unroll
-    for (int r = 0; r < 4; ++r) y[r] *= scale;
-#pragma unroll
-    for (int s = 0; s < 2; ++s) {
-      if (s * 32 > wave * 16 + 15) continue;  // all of these tokens come later
-      WideFrag<T> fp;
-#pragma unroll
-      for (int e = 0; e < 8; ++e) {
-        const int j = s * 32 + quad * 8 + e;
-        const float weight = __expf(sizeof(T) == 4 ? (o.own_high - o.high[s][e]) + (o.own_low - o.low[s][e])
-                                              : o.own_high - o.high[s][e]) * o.dt[s][e];
-        // the skip connection is one more weight on the token's own input
-        fp.set(e, j > token ? 0.0f : fmaf(o.score[s][e], weight, j == token ? skip : 0.0f));
-      }
-      y = mma_wide_b(o.x[s], fp, y);
+      const uint32_t at = k / 32 * 512 + ((k / 16 % 2 * 2 + quad / 2) * 16 + column) * 8 + quad % 2 * 4;
+      *reinterpret_cast<x4 *>(state_block<T>(a, w, chunk, head, 0, v0) + at) = high;
+      if (kStatePlanes<T> == 2) *reinterpret_cast<x4 *>(state_block<T>(a, w, chunk, head, 1, v0) + at) = low;
     }
-    // the new state
     const float carry = __expf(o.end);
 #pragma unroll
     for (int t = 0; t < NT; ++t)
@@ -370,42 +341,109 @@ __global__ __launch_bounds__(256, 1) void ssm_scan_kernel(SsmArgs a, SsmWorkspac
     for (int s = 0; s < 2; ++s) {
       WideFrag<T> fx;
 #pragma unroll
-      for (int e = 0; e < 8; ++e)
-        fx.set(e, to_f32(o.x[s][e]) * o.tail[s][e]);
+      for (int e = 0; e < 8; ++e) fx.set(e, to_f32(o.x[s][e]) * o.tail[s][e]);
 #pragma unroll
       for (int t = 0; t < NT; ++t)
-        if ((wave + 4 * t) * 16 < (int)w.np) state[t] = mma_wide(fx, o.b[t][s], state[t]);
-    }
-    const uint32_t row = chunk * Q + token;
-    if (row < a.m) {
-      T *out = static_cast<T *>(a.y) + (size_t)row * w.inner + head * a.vdim;
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const uint32_t v = v0 + quad * 4 + r;
-        if (v < a.vdim) out[v] = (T)y[r];
-      }
+        if ((wave + 4 * t) * 16 < (int)w.np) state[t] = mma_wide_b(o.b[t][s], fx, state[t]);
     }
   };
 
-  ChunkOperands<T, NT> even, odd;
-  load(even, 0);
-  for (uint32_t chunk = 0; chunk < w.chunks; chunk += 2) {
-    if (chunk + 1 < w.chunks) load(odd, chunk + 1);
-    __builtin_amdgcn_sched_barrier(0);  // the requests stay ahead of the arithmetic
-    step(even, chunk);
-    if (chunk + 1 < w.chunks) {
-      if (chunk + 2 < w.chunks) load(even, chunk + 2);
-      __builtin_amdgcn_sched_barrier(0);
-      step(odd, chunk + 1);
+  // operands two chunks ahead
+  StateOperands<T, NT> ring[3];
+  load(ring[0], 0);
+  load(ring[1], min(1u, w.chunks - 1));
+  for (uint32_t chunk = 0; chunk < w.chunks; chunk += 3) {
+#pragma unroll
+    for (int i = 0; i < 3; ++i) {
+      if (chunk + i >= w.chunks) break;
+      load(ring[(i + 2) % 3], min(chunk + i + 2, w.chunks - 1));
+      __builtin_amdgcn_sched_barrier(0);  // the requests stay ahead of the arithmetic
+      step(ring[i], chunk + i);
     }
   }
+  if (v < a.vdim)
 #pragma unroll
-  for (int t = 0; t < NT; ++t)
+    for (int t = 0; t < NT; ++t)
 #pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const uint32_t v = v0 + quad * 4 + r, k = (wave + 4 * t) * 16 + column;
-      if (v < a.vdim && k < n) saved[(size_t)v * n + k] = state[t][r];
+      for (int r = 0; r < 4; ++r) {
+        const uint32_t k = (wave + 4 * t) * 16 + quad * 4 + r;
+        if (k < n) saved[k] = state[t][r];
+      }
+}
+
+// The parallel part: a workgroup per chunk and head, 16 tokens a wave.  y^T of 16 state rows: the incoming
+// state against c, scaled by the decay since the chunk's start, and x^T against the weighted scores of the
+// chunk's earlier tokens (the skip connection is one more weight on the token's own input).
+template <typename T, int STEPS>
+__global__ __launch_bounds__(256) void ssm_output_kernel(SsmArgs a, SsmWorkspace w) {
+  const uint32_t chunk = blockIdx.x, head = blockIdx.y, group = head / (a.heads / a.groups);
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, column = lane & 15, quad = lane >> 4;
+  const size_t ld = (size_t)a.groups * w.np;
+  const int token = wave * 16 + column;  // of the lane's output column
+  const uint32_t row = chunk * Q + token;
+  const size_t at = (size_t)chunk * a.heads + head;
+  const float *dt = w.dt + at * Q, *sum = w.sum + at * 2 * Q;
+  const float *score = w.scores + (((size_t)chunk * a.groups + group) * Q + token) * Q;
+  const T *c = static_cast<const T *>(w.c) + (size_t)row * ld + group * w.np + quad * 8;
+  const float skip = bf16_at(a.d_skip, head);
+  Frag<T> fc[STEPS];
+#pragma unroll
+  for (int s = 0; s < STEPS; ++s)
+    if (s * 32 < (int)w.np) fc[s] = *reinterpret_cast<const Frag<T> *>(c + s * 32);
+  const float own_high = sum[token], own_low = sum[Q + token];
+  WideFrag<T> weight[2];
+#pragma unroll
+  for (int s = 0; s < 2; ++s) {
+    const int j0 = s * 32 + quad * 8;
+    const f32x8 sc = *reinterpret_cast<const f32x8 *>(score + j0), d = *reinterpret_cast<const f32x8 *>(dt + j0);
+    const f32x8 high = *reinterpret_cast<const f32x8 *>(sum + j0), low = *reinterpret_cast<const f32x8 *>(sum + Q + j0);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      const float decayed = __expf((own_high - high[e]) + (own_low - low[e])) * d[e];
+      const int j = j0 + e;
+      weight[s].set(e, j > token ? 0.0f : fmaf(sc[e], decayed, j == token ? skip : 0.0f));
     }
+  }
+  const float scale = __expf(own_high);
+  for (uint32_t v0 = blockIdx.z * 16; v0 < a.vdim; v0 += gridDim.z * 16) {
+    const uint32_t v_row = min(v0 + column, a.vdim - 1);
+    f32x4 high = {0.0f, 0.0f, 0.0f, 0.0f}, low = high, within = high;
+#pragma unroll
+    for (int s = 0; s < STEPS; ++s)
+      if (s * 32 < (int)w.np) {
+        high = mma(reinterpret_cast<const Frag<T> *>(state_block<T>(a, w, chunk, head, 0, v0))[s * 64 + lane], fc[s], high);
+        if (kStatePlanes<T> == 2)
+          low = mma(reinterpret_cast<const Frag<T> *>(state_block<T>(a, w, chunk, head, 1, v0))[s * 64 + lane], fc[s], low);
+      }
+    const T *x = static_cast<const T *>(w.xt) + ((size_t)chunk * w.inner + head * a.vdim + v_row) * Q + quad * 8;
+#pragma unroll
+    for (int s = 0; s < 2; ++s)
+      if (s * 32 <= wave * 16 + 15)  // the others come later than all of the wave's tokens
+        within = mma_wide_b(*reinterpret_cast<const Frag<T> *>(x + s * 32), weight[s], within);
+    if (row >= a.m) continue;
+    T *out = static_cast<T *>(a.y) + (size_t)row * w.inner + head * a.vdim + v0 + quad * 4;
+    typedef T x4 __attribute__((ext_vector_type(4)));
+    x4 y;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) y[r] = (T)fmaf(scale, high[r] + low[r], within[r]);
+    if (a.vdim % 4 == 0) {
+      if (v0 + quad * 4 < a.vdim) *reinterpret_cast<x4 *>(out) = y;
+    } else {
+#pragma unroll
+      for (int r = 0; r < 4; ++r)
+        if (v0 + quad * 4 + r < a.vdim) out[r] = y[r];
+    }
+  }
+}
+
+template <typename T, int NT>
+hipError_t run_scan(const SsmArgs &a, const SsmWorkspace &w, hipStream_t stream) {
+  ssm_state_kernel<T, NT><<<dim3(a.heads, (a.vdim + 15) / 16), 256, 0, stream>>>(a, w);
+  if (hipError_t status = hipGetLastError()) return status;
+  const uint32_t blocks = (a.vdim + 15) / 16;
+  const uint32_t parts = std::min<uint32_t>(blocks, std::max<uint32_t>(1, 1024 / std::max<uint32_t>(1, w.chunks * a.heads)));
+  ssm_output_kernel<T, 2 * NT><<<dim3(w.chunks, a.heads, parts), 256, 0, stream>>>(a, w);
+  return hipGetLastError();
 }
 
 template <typename T>
@@ -421,12 +459,10 @@ hipError_t run_prefill(const SsmArgs &a, hipStream_t stream) {
   if (hipError_t status = hipGetLastError()) return status;
   ssm_scores_kernel<T><<<dim3(w.chunks, a.groups), 256, 0, stream>>>(a, w);
   if (hipError_t status = hipGetLastError()) return status;
-  const dim3 grid(a.heads, (a.vdim + 15) / 16);
-  if (w.np <= 64) ssm_scan_kernel<T, 1><<<grid, 256, 0, stream>>>(a, w);
-  else if (w.np <= 128) ssm_scan_kernel<T, 2><<<grid, 256, 0, stream>>>(a, w);
-  else if (w.np <= 256) ssm_scan_kernel<T, 4><<<grid, 256, 0, stream>>>(a, w);
-  else return hipErrorInvalidValue;
-  return hipGetLastError();
+  if (w.np <= 64) return run_scan<T, 1>(a, w, stream);
+  if (w.np <= 128) return run_scan<T, 2>(a, w, stream);
+  if (w.np <= 256) return run_scan<T, 4>(a, w, stream);
+  return hipErrorInvalidValue;
 }
 
 }  // namespace
