@@ -124,9 +124,8 @@ __device__ __forceinline__ void stage_activation(const DenseGemvArgs &a, float *
 
 // ROWS weight rows streamed against the staged activation in blocks of STEPS * 512 columns; the first block
 // is requested by `request`, ahead of the staging where the rows are known by then.
-template <int ROWS, bool VEC>
+template <int ROWS, bool VEC, int STEPS = 4>
 struct RowStream {
-  static constexpr int STEPS = ROWS > 4 ? 2 : 4;
   const __bf16 *rows[ROWS];
   bf16x8 w[STEPS][ROWS];
   float sums[ROWS];
@@ -308,7 +307,7 @@ __device__ __forceinline__ void select_experts(const float *logits, uint32_t exp
 }
 
 // blockIdx.y: choice 0 .. top - 1, or `top`: the shared expert.  A wave owns kUpOutputs hidden values.
-constexpr int kUpOutputs = 4;
+constexpr int kUpOutputs = 4, kUpSteps = 2;
 
 template <typename T, bool VEC>
 __global__ __launch_bounds__(256) void moe_gemv_up_kernel(MoeGemvArgs a) {
@@ -326,22 +325,25 @@ __global__ __launch_bounds__(256) void moe_gemv_up_kernel(MoeGemvArgs a) {
   in.norm_groups = 1;
   in.epsilon = a.epsilon;
   in.k = a.width;
-  stage_activation<T>(in, xs, plane, scratch, [] {});
-  uint32_t expert = 0;
-  if (!shared) {
-    select_experts<256>(a.logits, a.experts, a.top, z, ids, weights);
-    expert = ids[blockIdx.y];
-  }
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const uint32_t first = (blockIdx.x * kWaves + wave) * kUpOutputs;
-  if (first >= n_total) return;
-  const uint16_t *gate = shared ? a.shared_gate : a.gate + (size_t)expert * a.ff * a.width;
-  const uint16_t *up = shared ? a.shared_up : a.up + (size_t)expert * a.ff * a.width;
-  RowStream<2 * kUpOutputs, VEC> stream;
+  RowStream<2 * kUpOutputs, VEC, kUpSteps> stream;
+  // the choice is made, and its weights are requested, while the activation is on its way to LDS
+  stage_activation<T>(in, xs, plane, scratch, [&] {
+    uint32_t expert = 0;
+    if (!shared) {
+      select_experts<256>(a.logits, a.experts, a.top, z, ids, weights);
+      expert = ids[blockIdx.y];
+    }
+    const uint16_t *gate = shared ? a.shared_gate : a.gate + (size_t)expert * a.ff * a.width;
+    const uint16_t *up = shared ? a.shared_up : a.up + (size_t)expert * a.ff * a.width;
 #pragma unroll
-  for (int r = 0; r < 2 * kUpOutputs; ++r)
-    stream.rows[r] = reinterpret_cast<const __bf16 *>((r & 1) ? up : gate) + (size_t)min(first + r / 2, n_total - 1) * a.width;
-  stream.request(a.width, lane);
+    for (int r = 0; r < 2 * kUpOutputs; ++r)
+      stream.rows[r] =
+          reinterpret_cast<const __bf16 *>((r & 1) ? up : gate) + (size_t)min(first + r / 2, n_total - 1) * a.width;
+    stream.request(a.width, lane);
+  });
+  if (first >= n_total) return;
   stream.run(xs, plane, a.width, lane);
   float g = 0.0f, u = 0.0f;
 #pragma unroll
