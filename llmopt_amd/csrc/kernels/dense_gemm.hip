@@ -53,6 +53,19 @@ __device__ __forceinline__ void store4(T *out, f32x4 v, uint32_t count, bool vec
     if (i < (int)count) out[i] = (T)v[i];
 }
 
+// kQkv: value columns of row r mixed with (or kept for) other layers.
+__device__ __forceinline__ void mix_values(const DenseLinearArgs &a, uint32_t r, uint32_t c, f32x4 &v) {
+  if (a.mix.mode == 0 || c + 3 < a.split) return;
+  const uint32_t n_v = a.n - a.split;
+#pragma unroll
+  for (int i = 0; i < 4; ++i)
+    if (c + i < a.n && c + i >= a.split) {
+      float *first = a.mix.v_first + (size_t)r * n_v + (c + i - a.split);
+      if (a.mix.mode == 1) *first = v[i];
+      else v[i] = (1.0f - a.mix.lambda) * v[i] + a.mix.lambda * *first;
+    }
+}
+
 // Four results of row r, columns c .. c + 3 (those below n).
 template <typename T>
 __device__ __forceinline__ void emit(const DenseLinearArgs &a, uint32_t r, uint32_t c, f32x4 v) {
@@ -81,16 +94,7 @@ __device__ __forceinline__ void emit(const DenseLinearArgs &a, uint32_t r, uint3
       return;
     }
     case DenseEpilogue::kQkv: {
-      if (a.mix.mode != 0) {
-        const uint32_t n_v = a.n - a.split;
-#pragma unroll
-        for (int i = 0; i < 4; ++i)
-          if (i < (int)count && c + i >= a.split) {
-            float *first = a.mix.v_first + (size_t)r * n_v + (c + i - a.split);
-            if (a.mix.mode == 1) *first = v[i];
-            else v[i] = (1.0f - a.mix.lambda) * v[i] + a.mix.lambda * *first;
-          }
-      }
+      mix_values(a, r, c, v);
       store4(static_cast<T *>(a.out) + (size_t)r * a.ld_out + c, v, count, (a.ld_out & 3) == 0);
       return;
     }
@@ -297,6 +301,61 @@ hipError_t run_gemm(const DenseLinearArgs &a, hipStream_t stream) {
   return hipGetLastError();
 }
 
+// The bf16 outputs of a wave, 16 rows at a time through its own LDS rows, so that a store covers whole lines.
+template <int MT, int NT, bool GATED>
+__device__ __forceinline__ void emit_rows(const DenseLinearArgs &a, const f32x4 (&acc)[MT][NT], uint32_t m_first,
+                                          uint32_t m_rows, uint32_t n_first, uint32_t row_offset,
+                                          uint32_t column_offset, int lane, __bf16 *rows) {
+  constexpr int WIDTH = (GATED ? NT / 2 : NT) * 16, STRIDE = WIDTH + 8, PIECES = WIDTH / 8;
+  const uint32_t c_first = n_first + (GATED ? column_offset / 2 : column_offset);
+  const uint32_t limit = a.epilogue == DenseEpilogue::kSplit ? a.split : a.n;  // columns of `out`
+  const int quad = lane >> 4;
+#pragma unroll
+  for (int i = 0; i < MT; ++i) {
+    const uint32_t r_in_tile = row_offset + i * 16 + (lane & 15), r = m_first + r_in_tile;
+#pragma unroll
+    for (int j = 0; j < (GATED ? NT / 2 : NT); ++j) {
+      const uint32_t c = c_first + j * 16 + quad * 4;
+      f32x4 v;
+      if (GATED) {
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[e] = gate_activation(acc[i][2 * j][e], a.activation) * acc[i][2 * j + 1][e];
+      } else {
+        v = acc[i][j];
+        if (a.epilogue == DenseEpilogue::kQkv && r_in_tile < m_rows) mix_values(a, r, c, v);
+        if (a.epilogue == DenseEpilogue::kSplit && r_in_tile < m_rows && c + 3 >= a.split) {
+#pragma unroll
+          for (int e = 0; e < 4; ++e)
+            if (c + e >= a.split && c + e < a.n) a.out_f32[(size_t)r * a.ld_f32 + (c + e - a.split)] = v[e];
+        }
+      }
+      bf16x4 packed;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) packed[e] = (__bf16)v[e];
+      *reinterpret_cast<bf16x4 *>(rows + (lane & 15) * STRIDE + j * 16 + quad * 4) = packed;
+    }
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");  // the wave's rows are whole
+    __builtin_amdgcn_wave_barrier();
+#pragma unroll
+    for (int q = 0; q < (16 * PIECES + 63) / 64; ++q) {
+      const int index = q * 64 + lane, row = index / PIECES, piece = index % PIECES;
+      const uint32_t at = row_offset + i * 16 + row, c = c_first + piece * 8;
+      if (row >= 16 || at >= m_rows || c >= limit) continue;
+      const bf16x8 v = *reinterpret_cast<const bf16x8 *>(rows + row * STRIDE + piece * 8);
+      __bf16 *out = static_cast<__bf16 *>(a.out) + (size_t)(m_first + at) * a.ld_out + c;
+      if (c + 8 <= limit && a.ld_out % 8 == 0) {
+        *reinterpret_cast<bf16x8 *>(out) = v;
+      } else {
+#pragma unroll
+        for (int e = 0; e < 8; ++e)
+          if (c + e < limit) out[e] = v[e];
+      }
+    }
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");  // read before the next sixteen rows are written
+    __builtin_amdgcn_wave_barrier();
+  }
+}
+
 // The same product for bf16 rows of a multiple of 64 values, staged by direct global -> LDS copies
 // (global_load_lds_dwordx4: 64 lanes x 16 bytes to consecutive LDS addresses) a ring of STAGES stages deep:
 // the copies of later stages run while a stage is multiplied, waited for by count, one barrier a stage.
@@ -388,8 +447,15 @@ __global__ __launch_bounds__(WAVES * 64) void dense_gemm_direct_kernel(GemmParam
         for (int j = 0; j < NT; ++j) acc[i][j] = mma(fw[j], fa[i], acc[i][j]);
     }
   }
-  emit_tile<__bf16, MT, NT, GATED>(a, acc, place.m_first, place.m_rows, place.n_first, wm * (BM / WM),
-                                   wn * (BN / WN), lane);
+  if (a.epilogue == DenseEpilogue::kAdd || a.epilogue == DenseEpilogue::kStoreF32) {
+    emit_tile<__bf16, MT, NT, GATED>(a, acc, place.m_first, place.m_rows, place.n_first, wm * (BM / WM),
+                                     wn * (BN / WN), lane);
+    return;
+  }
+  __syncthreads();  // the stages' LDS is free
+  static_assert(16 * (NT * 16 + 8) * 2 * WAVES <= STAGES * ROWS * 128, "a wave's output rows fit");
+  emit_rows<MT, NT, GATED>(a, acc, place.m_first, place.m_rows, place.n_first, wm * (BM / WM), wn * (BN / WN), lane,
+                           stage_rows + wave * 16 * (NT * 16 + 8));
 }
 
 template <int BM, int BN, int WM, int WAVES, int STAGES, bool GATED, bool ROUTED>
