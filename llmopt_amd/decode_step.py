@@ -144,8 +144,8 @@ class DecodeStep:
     def __init__(self, runtime: Runtime, config: DecodeConfig, weights: dict, batch: int, pool: Buffer,
                  slots: Buffer, slot_offsets, past_lengths, new_slots, positions, max_context=None,
                  slots_host=None, reference_entries: bool = False, fused: bool | None = None,
-                 projecting: bool | None = None, fused_qkv: bool | None = None):
-        """max_context: the longest context any later step will have (sizes the attention launch;
+                 projecting: bool | None = None, fused_qkv: bool | None = None, device_weights: dict | None = None):
+        """device_weights: buffers another step uploaded (`device`), to share.  max_context: the longest context any later step will have (sizes the attention launch;
         default: the longest now).  slots_host: the host copy of the slot table, with room behind
         every sequence's slots for the tokens `advance` will add.  reference_entries (batch 1):
         rotation, cache pack and attention as the reference's own three kernels
@@ -202,7 +202,7 @@ class DecodeStep:
         self.trig = b(np.concatenate([cos, sin]))
         self.cos = self.trig.view(0, cos.nbytes)
         self.sin = self.trig.view(cos.nbytes, sin.nbytes)
-        self.device = {
+        self.device = device_weights if device_weights is not None else {
             "embedding": b(weights["embedding"]),
             "final_norm": b(weights["final_norm"]),
             "lm_head": tuple(b(a) for a in weights["lm_head"]),
@@ -403,10 +403,14 @@ class DecodeStep:
         """After a step: every sequence is one token longer.  Rewrites the device buffers the next
         step reads - context lengths, the new token's slot (the next entry of the sequence's slot
         table) and the rotary rows of the next position."""
+        self.seek(self.host_lengths + 1, self.host_positions + 1)
+
+    def seek(self, lengths, positions) -> None:
+        """Makes the next step that of sequences with these context lengths and next positions."""
         if self.slots_host is None:
             raise ValueError("advance needs the host copy of the slot table")
-        self.host_lengths += 1
-        self.host_positions += 1
+        self.host_lengths[:] = lengths
+        self.host_positions[:] = positions
         if int(self.host_lengths.max()) > self.max_past:
             raise ValueError("context grew beyond max_context")
         self.past_lengths.write(self.host_lengths)

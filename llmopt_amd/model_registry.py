@@ -17,6 +17,7 @@ import os
 
 from .layered_model import LayeredModel
 from .native import Runtime
+from .w4a16_model import W4a16Model
 
 _ARCHITECTURES = {}
 
@@ -51,3 +52,4 @@ def load_model(directory: str, runtime: Runtime | None = None, **options):
 
 
 register("Barovik", LayeredModel)
+register("W4A16Transformer", W4a16Model)
