@@ -11,7 +11,8 @@
 //    head, 64 keys a stage through LDS; keys before the portion come from the ring, the others from the
 //    portion's own rows.  S^T = K Q^T leaves every lane four consecutive keys of one query row, which is
 //    the B operand of O^T += V^T P^T up to a permutation of the contraction index that the V^T operand
-//    follows: probabilities never leave their lane.  Caps of at most kFixedMaxCap bound the exponent, so
+//    follows: probabilities never leave their lane (bf16: as a high and a low part, so that the weights keep
+//    float32 accuracy in the product).  Caps of at most kFixedMaxCap bound the exponent, so
 //    the running maximum (and the rescaling) is dropped for a constant one.
 //  * chunk_decode_kernel: one token.  A workgroup takes kSplitKeys keys of one key / value head for all
 //    query heads on it, which are the operand columns; chunk_merge_kernel joins the splits when the ring is
@@ -243,13 +244,13 @@ __global__ __launch_bounds__(256, ND * 2 + NE <= 16 || sizeof(T) == 2 ? 2 : 1) v
     }
 #pragma unroll
     for (int ks = 0; ks < 2; ++ks) {
-      Frag<T> fp[QT];
+      WideFrag<T> fp[QT];  // the weights keep float32 accuracy
 #pragma unroll
       for (int t = 0; t < QT; ++t)
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          fp[t][r] = (T)score[2 * ks][t][r];
-          fp[t][4 + r] = (T)score[2 * ks + 1][t][r];
+          fp[t].set(r, score[2 * ks][t][r]);
+          fp[t].set(4 + r, score[2 * ks + 1][t][r]);
         }
 #pragma unroll
       for (int e = 0; e < NE; ++e) {
@@ -257,7 +258,7 @@ __global__ __launch_bounds__(256, ND * 2 + NE <= 16 || sizeof(T) == 2 ? 2 : 1) v
         const auto first = four_keys(keys, SV, lane), second = four_keys(keys + 16 * SV, SV, lane);
         const Frag<T> fv = __builtin_shufflevector(first, second, 0, 1, 2, 3, 4, 5, 6, 7);
 #pragma unroll
-        for (int t = 0; t < QT; ++t) out[e][t] = mma(fv, fp[t], out[e][t]);
+        for (int t = 0; t < QT; ++t) out[e][t] = mma_wide_b(fv, fp[t], out[e][t]);
         if (e % 4 == 3) __builtin_amdgcn_sched_barrier(0);
       }
     }
@@ -387,7 +388,7 @@ __global__ __launch_bounds__(256) void chunk_decode_kernel(ChunkAttentionArgs a,
     __syncthreads();
 #pragma unroll
     for (int w = 0; w < 4; ++w) best = fmaxf(best, lds_top[w * 16 + column]);
-    Frag<T> fp;
+    WideFrag<T> fp;
     float total = 0.0f;
 #pragma unroll
     for (int kt = 0; kt < 2; ++kt)
@@ -395,7 +396,7 @@ __global__ __launch_bounds__(256) void chunk_decode_kernel(ChunkAttentionArgs a,
       for (int r = 0; r < 4; ++r) {
         const float p = exp2_raw(score[kt][r] - best);
         total += p;
-        fp[kt * 4 + r] = (T)p;
+        fp.set(kt * 4 + r, p);
       }
     total += __shfl_xor(total, 16, 64);
     total += __shfl_xor(total, 32, 64);
@@ -406,7 +407,7 @@ __global__ __launch_bounds__(256) void chunk_decode_kernel(ChunkAttentionArgs a,
       const T *keys = lds_v + quad * 4 * SV + e * 16;
       const auto first = four_keys(keys, SV, lane), second = four_keys(keys + 16 * SV, SV, lane);
       const Frag<T> fv = __builtin_shufflevector(first, second, 0, 1, 2, 3, 4, 5, 6, 7);
-      out[e] = mma(fv, fp, f32x4{0.0f, 0.0f, 0.0f, 0.0f});
+      out[e] = mma_wide_b(fv, fp, f32x4{0.0f, 0.0f, 0.0f, 0.0f});
     }
     __syncthreads();  // every read of the values is done
 #pragma unroll
