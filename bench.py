@@ -702,9 +702,40 @@ def layered_work(model, m, context):
     return flops, weights + 2 * c.width * c.vocabulary + state
 
 
+def verify_layered(runtime):
+    """A small decoder with the timed one's layers, prompt and decoding, against the float64 restatement
+    (every expert chosen: no close call)."""
+    from llmopt_amd.layered_model import LayeredConfig, LayeredModel
+    from llmopt_amd.safetensors_file import from_bfloat16
+    from oracle import hybrid_model
+    config = layered_config("1024")
+    config.update(width=256, vocab=500)
+    for layer in config["layers"]:
+        m = layer["mixer"]
+        m.update(heads=8, vdim=64)
+        if layer["type"] == "attention":
+            m.update(kv_heads=2, dim=64, scale=0.125, mask={"size": 48})
+            layer["mlp"].update(router={"experts": 4, "top": 4}, expert={"ff": 128}, shared={"ff": 192})
+        else:
+            layer["mlp"]["ff"] = 512
+    parsed = LayeredConfig.parse(config)
+    rng = np.random.default_rng(SEED + 12)
+    patterns = parsed.random_tensors(rng)
+    model = LayeredModel(runtime, parsed, patterns, slots=1, max_context=256)
+    tokens = rng.integers(0, 500, 140).tolist()
+    sequence = model.open()
+    got = np.concatenate([model.step(sequence, tokens[:130], range(130))] +
+                         [model.step(sequence, [t], [0]) for t in tokens[130:]]).astype(np.float64)
+    weights = {name: from_bfloat16(array).reshape(array.shape) for name, array in patterns.items()}
+    want = hybrid_model.forward(config, weights, tokens)[0]
+    return float(np.linalg.norm(got - want) / np.linalg.norm(want))
+
+
 def bench_layered(runtime, sizes, prompts=(512, 2048, 8192), context=2000):
     """Prefill (one portion, logits of its last token) and decode (one token after `context`, a HIP graph) of
-    the layered decoders, and the same of the W4A16 transformer.  Medians of graph replays, in turn."""
+    the layered decoders, and the same of the W4A16 transformer.  Medians of graph replays, in turn.  Checked
+    outside the timed regions: a small decoder of the same layers against the restatement, and at every size the
+    decoded token's logits against those of the same token at the end of a prompt."""
     from llmopt_amd.decode_step import DecodeConfig, DecodeStep, random_w4
     from llmopt_amd.layered_model import LayeredConfig, LayeredModel
     from llmopt_amd.native import DispatchList
@@ -712,6 +743,7 @@ def bench_layered(runtime, sizes, prompts=(512, 2048, 8192), context=2000):
     rng = np.random.default_rng(SEED + 11)
     median = lambda values: sorted(values)[len(values) // 2]
     results = []
+    restated = verify_layered(runtime)
     for size in sizes:
         z = LAYERED_SIZES[size]
         print("layered", size, file=sys.stderr, flush=True)
@@ -757,10 +789,17 @@ def bench_layered(runtime, sizes, prompts=(512, 2048, 8192), context=2000):
                           "TFLOPs": round(step.flops() / other_ms / 1e9, 1),
                           "mfma_frac": round(step.flops() / other_ms / 1e9 / MFMA_F16_PEAK_TFLOPS, 4)}})
             del step, pool
+        tokens = rng.integers(0, LAYERED_VOCABULARY, context).tolist() + [1]
         sequence = model.open()
-        model.step(sequence, rng.integers(0, LAYERED_VOCABULARY, context))
+        at_once = model.step(sequence, tokens, [context]).astype(np.float64)
+        model.close(sequence)
+        sequence = model.open()
+        model.step(sequence, tokens[:context])
         plan = model.decode_plan()
         plan.execute(1, sequence)  # leaves the step words of a token behind the context
+        difference = float(np.linalg.norm(model.logits_row() - at_once[0]) / np.linalg.norm(at_once))
+        entry["verified"] = bool(restated <= 2e-2 and difference <= 0.1)
+        entry["rel_l2_restatement"], entry["rel_l2_decode_against_prompt"] = (float("%.3g" % v) for v in (restated, difference))
         graph = runtime.begin_batch()
         graph.dispatch_all(DispatchList(plan.dispatches))
         ms = median(graph.commit_profiled_each(repeats=9))
@@ -959,9 +998,11 @@ def main():
         runtime.close()
         return
     if args.layered:
-        print(json.dumps({"layered": bench_layered(runtime, args.layered.split(","),
-                                                   tuple(int(m) for m in args.layered_prompts.split(",")))}))
+        layered = bench_layered(runtime, args.layered.split(","), tuple(int(m) for m in args.layered_prompts.split(",")))
         runtime.close()
+        if not all(entry["verified"] for entry in layered):
+            sys.exit("bench.py: outputs of timed cases differ beyond tolerance: %s" % layered)
+        print(json.dumps({"layered": layered}))
         return
     gemv = bench_gemv(runtime, args.steps, args.warmup, serial_only=args.serial_only)
     # the sweep's time by kernel; `roofline` is the kernel with the largest share
