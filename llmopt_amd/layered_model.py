@@ -10,7 +10,6 @@ whose step words carry position and slot, so that it serves every sequence.
 """
 from __future__ import annotations
 
-import json
 import os
 import struct
 from dataclasses import dataclass
