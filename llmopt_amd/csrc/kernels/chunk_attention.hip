@@ -1,11 +1,12 @@
-// Grouped-query attention over chunks of positions, with a tanh cap on the scores and a learned sink in
-// the softmax denominator.
+// Grouped-query attention over chunks of positions or a sliding window, with a tanh cap on the scores and a
+// learned sink in the softmax denominator (both optional).
 //
-//   score(i, j) = cap tanh(scale q_i . k_j / cap),  visible when j <= i and i / chunk == j / chunk
+//   score(i, j) = cap tanh(scale q_i . k_j / cap),  visible when j <= i and i / chunk == j / chunk,
+//                                                   or when 0 <= i - j < window
 //   out_i = sum_j exp(score) v_j / (sum_j exp(score) + exp(sink))
 //
 // Keys and values live in a ring per sequence slot and head: position p in row p % capacity, capacity >=
-// chunk, so that a ring of one chunk holds everything later tokens can see.
+// chunk or window, so that a ring of one holds everything later tokens can see.
 //
 //  * chunk_prefill_kernel: a portion of a prompt.  Four waves walk the keys of 64 * QT query rows of one
 //    head, 64 keys a stage through LDS; keys before the portion come from the ring, the others from the
@@ -16,7 +17,9 @@
 //    the running maximum (and the rescaling) is dropped for a constant one.
 //  * chunk_decode_kernel: one token.  A workgroup takes kSplitKeys keys of one key / value head for all
 //    query heads on it, which are the operand columns; chunk_merge_kernel joins the splits when the ring is
-//    longer than one.
+//    longer than one.  Over a raw float32 row it norms and rotates the group's queries and the token's own
+//    key first (in LDS) and leaves key and value in the ring; the own key and value never come from there.
+//  * rotate_heads_kernel: the same norm and rotation for a portion of a prompt, in place.
 #include <algorithm>
 
 #include "dense.h"
@@ -31,8 +34,11 @@ constexpr uint32_t kSplitKeys = 128;
 constexpr float kFixedMaxCap = 40.0f;
 constexpr float kLog2e = 1.4426950408889634f;
 
-__device__ __forceinline__ uint32_t chunk_start(uint32_t position, uint32_t chunk) {
-  return chunk ? position - position % chunk : 0;
+// The first position that `position` sees; never falls from one position to the next.
+__device__ __forceinline__ uint32_t first_seen(uint32_t position, const ChunkCache &cache) {
+  if (cache.span == 0) return 0;
+  if (cache.sliding) return position + 1 > cache.span ? position + 1 - cache.span : 0;
+  return position - position % cache.span;
 }
 
 // Values of four keys (rows of the stage) at the lane's column: what the V^T operand takes.  bf16: the
@@ -80,14 +86,14 @@ __global__ __launch_bounds__(256, ND * 2 + NE <= 16 || sizeof(T) == 2 ? 2 : 1) v
   const uint32_t p0 = a.state[kStatePosition], slot = a.state[kStateSlot];
   const uint32_t row_first = tile * 64 * QT;
   const uint32_t row_end = min(row_first + 64 * QT, a.m);
-  const uint32_t ld = a.heads * a.dim + a.kv_heads * (a.dim + a.vdim);
+  const uint32_t ld = a.ld;
   const T *qkv = static_cast<const T *>(a.qkv);
   const T *fresh_k = qkv + a.heads * a.dim + group * a.dim;
   const T *fresh_v = qkv + a.heads * a.dim + a.kv_heads * a.dim + group * a.vdim;
   const size_t ring = ((size_t)slot * a.kv_heads + group) * a.cache.capacity;
   const T *cache_k = static_cast<const T *>(a.cache.keys) + ring * a.dim;
   const T *cache_v = static_cast<const T *>(a.cache.values) + ring * a.vdim;
-  const bool vec = a.dim % 8 == 0 && a.vdim % 8 == 0;
+  const bool vec = a.dim % 8 == 0 && a.vdim % 8 == 0 && ld % 8 == 0;
 
   // queries of this wave: operand columns
   Frag<T> fq[QT][ND];
@@ -96,7 +102,7 @@ __global__ __launch_bounds__(256, ND * 2 + NE <= 16 || sizeof(T) == 2 ? 2 : 1) v
   for (int t = 0; t < QT; ++t) {
     const uint32_t r = min(row_first + (wave * QT + t) * 16 + column, a.m - 1);
     query[t] = p0 + r;
-    low[t] = chunk_start(query[t], a.cache.chunk);
+    low[t] = first_seen(query[t], a.cache);
 #pragma unroll
     for (int d = 0; d < ND; ++d) {
       const int k = d * 32 + quad * 8;
@@ -105,8 +111,8 @@ __global__ __launch_bounds__(256, ND * 2 + NE <= 16 || sizeof(T) == 2 ? 2 : 1) v
   }
   const uint32_t wave_first = p0 + min(row_first + wave * QT * 16, a.m - 1);
   const uint32_t wave_last = p0 + min(row_first + (wave + 1) * QT * 16 - 1, a.m - 1);
-  const uint32_t wave_low = chunk_start(wave_first, a.cache.chunk);
-  const uint32_t wave_low_last = chunk_start(wave_last, a.cache.chunk);
+  const uint32_t wave_low = first_seen(wave_first, a.cache);
+  const uint32_t wave_low_last = first_seen(wave_last, a.cache);
 
   // Exponents are taken to base two.  capped: score = cap tanh(scale s / cap), with
   // tanh z = 1 - 2 / (1 + e^(2 z)); fixed: the cap bounds it, and the maximum is a constant.
@@ -127,7 +133,7 @@ __global__ __launch_bounds__(256, ND * 2 + NE <= 16 || sizeof(T) == 2 ? 2 : 1) v
     for (int t = 0; t < QT; ++t) out[e][t] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
 
   const uint32_t last = p0 + row_end - 1;
-  const uint32_t key_begin = chunk_start(p0 + row_first, a.cache.chunk);
+  const uint32_t key_begin = first_seen(p0 + row_first, a.cache);
 
   // a stage travels global -> registers while the one before it is multiplied
   Frag<T> reg_k[K_LOADS], reg_v[V_LOADS];
@@ -269,15 +275,15 @@ __global__ __launch_bounds__(256, ND * 2 + NE <= 16 || sizeof(T) == 2 ? 2 : 1) v
     float sum = total[t];
     sum += __shfl_xor(sum, 16, 64);
     sum += __shfl_xor(sum, 32, 64);
-    const float inverse = 1.0f / sum;
+    const float inverse = a.out_scale / sum;
     const uint32_t r = row_first + (wave * QT + t) * 16 + column;
     if (r >= a.m) continue;
-    T *target = static_cast<T *>(a.out) + (size_t)r * a.heads * a.vdim + head * a.vdim;
+    T *target = static_cast<T *>(a.out) + (size_t)r * a.ld_out + head * a.vdim;
 #pragma unroll
     for (int e = 0; e < NE; ++e) {
       const uint32_t c = e * 16 + quad * 4;
       typedef T x4 __attribute__((ext_vector_type(4)));
-      if (vec && c < a.vdim) {
+      if (vec && a.ld_out % 4 == 0 && c < a.vdim) {
         x4 packed;
 #pragma unroll
         for (int i = 0; i < 4; ++i) packed[i] = (T)(out[e][t][i] * inverse);
@@ -297,7 +303,7 @@ __global__ __launch_bounds__(256) void chunk_cache_write_kernel(ChunkAttentionAr
   const uint32_t position = a.state[kStatePosition] + r, slot = a.state[kStateSlot];
   const uint32_t row = position % a.cache.capacity;
   const uint32_t n_k = a.kv_heads * a.dim, n_v = a.kv_heads * a.vdim;
-  const T *source = static_cast<const T *>(a.qkv) + (size_t)r * (a.heads * a.dim + n_k + n_v) + a.heads * a.dim;
+  const T *source = static_cast<const T *>(a.qkv) + (size_t)r * a.ld + a.heads * a.dim;
   T *keys = static_cast<T *>(a.cache.keys), *values = static_cast<T *>(a.cache.values);
   for (uint32_t c = threadIdx.x; c < n_k + n_v; c += 256) {
     if (c < n_k)
@@ -317,13 +323,90 @@ constexpr int decode_lds_floats() {
   return 4 * 32 * value_stride<T, NE>() * (int)sizeof(T) / 4 + 2 * 4 * 16;
 }
 
+// Norm and rotation of head vectors, a wave a vector, lane l holding components l + 64 i.
+template <int PARTS>
+struct HeadVector {
+  float v[PARTS];
+  // exchange(v, partner, half): every rotated component's partner, c + half or c - half.
+  template <typename Exchange>
+  __device__ __forceinline__ void norm_and_rotate(const HeadRotation &r, const uint16_t *norm, uint32_t dim,
+                                                  uint32_t position, int lane, Exchange exchange) {
+    float sum = 0.0f;
+#pragma unroll
+    for (int i = 0; i < PARTS; ++i) sum += v[i] * v[i];
+    const float inverse = 1.0f / sqrtf(wave_sum(sum) / (float)dim + r.epsilon);
+    float partner[PARTS];
+    const uint32_t half = r.dims / 2;
+#pragma unroll
+    for (int i = 0; i < PARTS; ++i) {
+      const uint32_t c = lane + 64 * i;
+      v[i] *= inverse * (c < dim ? (float)reinterpret_cast<const __bf16 *>(norm)[c] : 0.0f);
+    }
+    exchange(v, partner, half);
+#pragma unroll
+    for (int i = 0; i < PARTS; ++i) {
+      const uint32_t c = lane + 64 * i;
+      if (c >= r.dims) continue;
+      float cosine, sine;
+      turn(position, r.frequencies[c < half ? c : c - half], cosine, sine);
+      v[i] = c < half ? v[i] * cosine - partner[i] * sine : v[i] * cosine + partner[i] * sine;
+    }
+  }
+};
+
+// The partner of every rotated component through `row`, floats of the wave's own in LDS.
+template <int PARTS>
+struct ThroughLds {
+  float *row;
+  uint32_t dims;
+  int lane;
+  __device__ __forceinline__ void operator()(const float (&v)[PARTS], float (&partner)[PARTS], uint32_t half) const {
+#pragma unroll
+    for (int i = 0; i < PARTS; ++i) row[lane + 64 * i] = v[i];
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+    __builtin_amdgcn_wave_barrier();
+#pragma unroll
+    for (int i = 0; i < PARTS; ++i) {
+      const uint32_t c = lane + 64 * i;
+      partner[i] = c < dims ? row[c < half ? c + half : c - half] : 0.0f;
+    }
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");  // read before the row is written again
+    __builtin_amdgcn_wave_barrier();
+  }
+};
+
+// Vectors 0 .. heads + kv_heads - 1 of every row: the queries, then the keys.
+template <typename T, int PARTS>
+__global__ __launch_bounds__(256) void rotate_heads_kernel(ChunkAttentionArgs a) {
+  __shared__ float rows[4][PARTS * 64];
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+  const uint32_t vector = blockIdx.y * 4 + wave, r = blockIdx.x;
+  if (vector >= a.heads + a.kv_heads) return;
+  T *head = const_cast<T *>(static_cast<const T *>(a.qkv)) + (size_t)r * a.ld + (size_t)vector * a.dim;
+  HeadVector<PARTS> h;
+#pragma unroll
+  for (int i = 0; i < PARTS; ++i) h.v[i] = lane + 64 * i < a.dim ? to_f32(head[lane + 64 * i]) : 0.0f;
+  h.norm_and_rotate(a.rotation, vector < a.heads ? a.rotation.q_norm : a.rotation.k_norm, a.dim,
+                    a.state[kStatePosition] + r, lane, ThroughLds<PARTS>{rows[wave], a.rotation.dims, lane});
+#pragma unroll
+  for (int i = 0; i < PARTS; ++i)
+    if (lane + 64 * i < a.dim) head[lane + 64 * i] = (T)h.v[i];
+}
+
+// LDS of a decode workgroup that starts from a raw row: queries [16][ND * 32 + pad], the own key, the own
+// value, a float row for every wave.
 template <typename T, int ND, int NE>
+constexpr int raw_row_lds_bytes() {
+  return (17 * (ND * 32 + 16 / (int)sizeof(T)) + NE * 16) * (int)sizeof(T) + 4 * (ND <= 2 ? 64 : ND * 32) * 4;
+}
+
+template <typename T, int ND, int NE, bool RAW>
 __global__ __launch_bounds__(256) void chunk_decode_kernel(ChunkAttentionArgs a, uint32_t splits) {
   constexpr int EP = NE * 16, SV = value_stride<T, NE>(), V_PIECES = EP / 8;
   extern __shared__ __attribute__((aligned(16))) char lds[];
   const uint32_t position = a.state[kStatePosition], slot = a.state[kStateSlot];
   const uint32_t group = blockIdx.x, split = blockIdx.y, per = a.heads / a.kv_heads;
-  const uint32_t begin = chunk_start(position, a.cache.chunk) + split * kSplitKeys;
+  const uint32_t begin = first_seen(position, a.cache) + split * kSplitKeys;
   if (begin > position) return;
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, column = lane & 15, quad = lane >> 4;
   // a wave's own rows: the values [32][SV], then its sums [16][EP] in their place
@@ -354,13 +437,60 @@ __global__ __launch_bounds__(256) void chunk_decode_kernel(ChunkAttentionArgs a,
   const float cap = a.softcap * kLog2e;
   const float inner = capped ? 2.0f * a.scale / a.softcap * kLog2e : a.scale * kLog2e;
 
+  // a raw row: the first sixteen queries and the own key and value
+  constexpr int SQ = ND * 32 + 16 / (int)sizeof(T), PARTS = ND <= 2 ? 1 : ND / 2;
+  T *lds_q = reinterpret_cast<T *>(lds + decode_lds_floats<T, NE>() * 4), *own_k = lds_q + 16 * SQ, *own_v = own_k + SQ;
+  float *exchange = reinterpret_cast<float *>(own_v + EP) + wave * PARTS * 64;
+  auto stage_vectors = [&](uint32_t h0, uint32_t count, bool key) {
+    for (uint32_t n = wave; n < count + (key ? 1 : 0); n += 4) {
+      const bool query = n < count;
+      const float *source = a.row + (query ? (size_t)(group * per + h0 + n) * a.dim : (size_t)(a.heads + group) * a.dim);
+      HeadVector<PARTS> h;
+#pragma unroll
+      for (int i = 0; i < PARTS; ++i) h.v[i] = lane + 64 * i < a.dim ? source[lane + 64 * i] : 0.0f;
+      h.norm_and_rotate(a.rotation, query ? a.rotation.q_norm : a.rotation.k_norm, a.dim, position, lane,
+                        ThroughLds<PARTS>{exchange, a.rotation.dims, lane});
+      T *target = query ? lds_q + n * SQ : own_k;
+#pragma unroll
+      for (int i = 0; i < PARTS; ++i)
+        if (lane + 64 * i < ND * 32) target[lane + 64 * i] = (T)h.v[i];  // (zeros behind the head's end)
+    }
+  };
+  if (RAW) {
+    stage_vectors(0, min(16u, per), true);
+    const float *value = a.row + (size_t)(a.heads + a.kv_heads) * a.dim + (size_t)group * a.vdim;
+    for (uint32_t c = tid; c < EP; c += 256) own_v[c] = (T)(c < a.vdim ? value[c] : 0.0f);
+    __syncthreads();
+    if (begin + kSplitKeys > position) {  // this workgroup's keys end with the own one
+      const size_t at = ring + position % a.cache.capacity;
+      for (uint32_t c = tid; c < a.dim; c += 256) static_cast<T *>(a.cache.keys)[at * a.dim + c] = own_k[c];
+      for (uint32_t c = tid; c < a.vdim; c += 256) static_cast<T *>(a.cache.values)[at * a.vdim + c] = own_v[c];
+    }
+#pragma unroll
+    for (int kt = 0; kt < 2; ++kt)
+      if (wave_begin + kt * 16 + column >= position)
+#pragma unroll
+        for (int d = 0; d < ND; ++d) fk[kt][d] = *reinterpret_cast<const Frag<T> *>(own_k + d * 32 + quad * 8);
+#pragma unroll
+    for (int i = 0; i < NE; ++i) {
+      const int index = i * 64 + lane;
+      if (wave_begin + index / V_PIECES >= position)
+        reg_v[i] = *reinterpret_cast<const Frag<T> *>(own_v + (index % V_PIECES) * 8);
+    }
+  }
+
   for (uint32_t h0 = 0; h0 < per; h0 += 16) {
     const uint32_t head = group * per + min(h0 + column, per - 1);
     Frag<T> fq[ND];
+    if (RAW && h0 > 0) {
+      stage_vectors(h0, min(16u, per - h0), false);
+      __syncthreads();
+    }
 #pragma unroll
     for (int d = 0; d < ND; ++d)
-      fq[d] = load_piece(static_cast<const T *>(a.qkv) + (size_t)head * a.dim + d * 32 + quad * 8,
-                         (int)a.dim - (d * 32 + quad * 8), vec);
+      fq[d] = RAW ? *reinterpret_cast<const Frag<T> *>(lds_q + min((uint32_t)column, per - 1 - h0) * SQ + d * 32 + quad * 8)
+                  : load_piece(static_cast<const T *>(a.qkv) + (size_t)head * a.dim + d * 32 + quad * 8,
+                               (int)a.dim - (d * 32 + quad * 8), vec);
     f32x4 score[2];
     float best = -1e30f;
 #pragma unroll
@@ -433,7 +563,8 @@ __global__ __launch_bounds__(256) void chunk_decode_kernel(ChunkAttentionArgs a,
           sum *= mine;
           all = all * mine + exp2_raw(sink - most);
         }
-        static_cast<T *>(a.out)[target * a.vdim + c] = (T)(sum / all);
+        if (a.out_row) a.out_row[target * a.vdim + c] = sum / all * a.out_scale;
+        else static_cast<T *>(a.out)[target * a.vdim + c] = (T)(sum / all * a.out_scale);
       } else {
         float *partial = static_cast<float *>(a.workspace) + ((size_t)target * splits + split) * (a.vdim + 2);
         partial[c] = sum;
@@ -453,7 +584,7 @@ __global__ __launch_bounds__(256) void chunk_merge_kernel(ChunkAttentionArgs a, 
   extern __shared__ __attribute__((aligned(16))) float shared[];
   float *best = shared, *total = shared + splits;
   const uint32_t head = blockIdx.x, position = a.state[kStatePosition];
-  const uint32_t live = min(splits, (position - chunk_start(position, a.cache.chunk)) / kSplitKeys + 1);
+  const uint32_t live = min(splits, (position - first_seen(position, a.cache)) / kSplitKeys + 1);
   const uint32_t stride = a.vdim + 2;
   const float *partial = static_cast<const float *>(a.workspace) + (size_t)head * splits * stride;
   const float sink = a.sink ? (float)reinterpret_cast<const __bf16 *>(a.sink)[head] * kLog2e : -INFINITY;
@@ -483,23 +614,25 @@ __global__ __launch_bounds__(256) void chunk_merge_kernel(ChunkAttentionArgs a, 
     denominator = fmaf(total[s], weight, denominator);
     if (c < a.vdim) sum = fmaf(partial[s * stride + c], weight, sum);
   }
-  if (c < a.vdim) static_cast<T *>(a.out)[head * a.vdim + c] = (T)(sum / denominator);
+  if (c >= a.vdim) return;
+  if (a.out_row) a.out_row[head * a.vdim + c] = sum / denominator * a.out_scale;
+  else static_cast<T *>(a.out)[head * a.vdim + c] = (T)(sum / denominator * a.out_scale);
 }
 
 uint32_t decode_splits(const ChunkAttentionArgs &a) {
-  const uint32_t longest = a.cache.chunk ? std::min(a.cache.chunk, a.cache.capacity) : a.cache.capacity;
+  const uint32_t longest = a.cache.span ? std::min(a.cache.span, a.cache.capacity) : a.cache.capacity;
   return (longest + kSplitKeys - 1) / kSplitKeys;
 }
 
-template <typename T, int ND, int NE>
+template <typename T, int ND, int NE, bool RAW>
 hipError_t run_decode(const ChunkAttentionArgs &a, hipStream_t stream) {
   static bool allowed[kMaxDevices] = {};
-  constexpr int bytes = decode_lds_floats<T, NE>() * 4;
+  constexpr int bytes = decode_lds_floats<T, NE>() * 4 + (RAW ? raw_row_lds_bytes<T, ND, NE>() : 0);
   const uint32_t splits = decode_splits(a);
   if (bytes > 64 * 1024)
-    if (hipError_t status = allow_dynamic_lds(reinterpret_cast<const void *>(chunk_decode_kernel<T, ND, NE>), bytes, allowed))
+    if (hipError_t status = allow_dynamic_lds(reinterpret_cast<const void *>(chunk_decode_kernel<T, ND, NE, RAW>), bytes, allowed))
       return status;
-  chunk_decode_kernel<T, ND, NE><<<dim3(a.kv_heads, splits), 256, bytes, stream>>>(a, splits);
+  chunk_decode_kernel<T, ND, NE, RAW><<<dim3(a.kv_heads, splits), 256, bytes, stream>>>(a, splits);
   if (hipError_t status = hipGetLastError()) return status;
   if (splits > 1) chunk_merge_kernel<T><<<a.heads, 256, splits * 8, stream>>>(a, splits);
   return hipGetLastError();
@@ -527,7 +660,8 @@ hipError_t run_prefill(const ChunkAttentionArgs &a, hipStream_t stream) {
 
 template <typename T, int ND, int NE>
 hipError_t run_attention(const ChunkAttentionArgs &a, hipStream_t stream) {
-  return a.m == 1 ? run_decode<T, ND, NE>(a, stream) : run_prefill<T, ND, NE>(a, stream);
+  if (a.m > 1) return run_prefill<T, ND, NE>(a, stream);
+  return a.row ? run_decode<T, ND, NE, true>(a, stream) : run_decode<T, ND, NE, false>(a, stream);
 }
 
 template <typename T, int ND>
@@ -559,6 +693,18 @@ bool chunk_attention_ok(const ChunkAttentionArgs &a) {
 
 hipError_t launch_chunk_attention(const ChunkAttentionArgs &a, hipStream_t stream) {
   return a.f32 ? pick_attention<float>(a, stream) : pick_attention<__bf16>(a, stream);
+}
+
+hipError_t launch_rotate_heads(const ChunkAttentionArgs &a, hipStream_t stream) {
+  const dim3 grid(a.m, (a.heads + a.kv_heads + 3) / 4);
+  const int parts = a.dim <= 64 ? 1 : a.dim <= 128 ? 2 : 4;
+  auto run = [&](auto kernel) {
+    kernel<<<grid, 256, 0, stream>>>(a);
+    return hipGetLastError();
+  };
+  if (a.f32)
+    return run(parts == 1 ? rotate_heads_kernel<float, 1> : parts == 2 ? rotate_heads_kernel<float, 2> : rotate_heads_kernel<float, 4>);
+  return run(parts == 1 ? rotate_heads_kernel<__bf16, 1> : parts == 2 ? rotate_heads_kernel<__bf16, 2> : rotate_heads_kernel<__bf16, 4>);
 }
 
 hipError_t launch_chunk_cache_write(const ChunkAttentionArgs &a, hipStream_t stream) {

@@ -1,6 +1,6 @@
 // Host-visible launch interface of the kernels over bfloat16 weights: linears with the epilogues a
-// layered decoder needs, chunked attention with a softmax sink, the Mamba-2 recurrence, and routed
-// experts.  Plain structs and device pointers; launchers are asynchronous on the stream and assume
+// layered decoder needs, attention over chunks or a sliding window, the Mamba-2 recurrence, the gated
+// delta rule, and routed experts.  Plain structs and device pointers; launchers are asynchronous on the stream and assume
 // validated sizes.  `f32` selects float activations (else bfloat16); weights are bfloat16 in both.
 #pragma once
 
@@ -15,7 +15,7 @@ constexpr uint32_t kStatePosition = 0, kStateSlot = 1, kStateWords = 2;
 
 enum class DenseEpilogue : uint32_t {
   kStore = 0,     // out[r, c] (activation type)
-  kStoreF32 = 1,  // out_f32[r, c]
+  kStoreF32 = 1,  // out_f32[r, c] (softcap > 0: softcap tanh(result / softcap))
   kAdd = 2,       // stream[r, c] += result * (row_gate ? sigmoid(row_gate[r * row_gate_stride]) : 1)
   kGated = 3,     // out[r, c] = act(gate) * up
   kQkv = 4,       // kStore, with the value columns mixed with another layer's values
@@ -39,6 +39,8 @@ struct DenseLinearArgs {
   uint32_t m, n, k, ldx;
   DenseEpilogue epilogue;
   uint32_t activation;
+  float limit;           // kGated, clamped activation
+  float softcap;         // kStoreF32; 0: none
   void *out;
   float *out_f32;        // kStoreF32, kSplit, and the stream of kAdd
   uint32_t ld_out, ld_f32;
@@ -68,6 +70,23 @@ struct DenseNormArgs {
 };
 hipError_t launch_dense_norm(const DenseNormArgs &args, hipStream_t stream);
 
+// A sublayer's output joins the stream behind its norm:
+//   stream_out[r, :] = x[row, :] + scale y[row, :] / rms(y[row, :]) * (offset + add_weight)
+// with row = rows_index ? rows_index[r] : r; y == null: stream_out = x.  operand (activation type) is the new
+// stream, or with norm_weight its norm, / rms * (offset + norm_weight).
+struct NormAddArgs {
+  bool f32;
+  const float *x, *y;          // f32 [*, width]
+  const uint16_t *add_weight;  // bf16 [width]
+  const uint16_t *norm_weight; // may be null
+  float *stream_out;           // f32 [rows, width], may be null
+  void *operand;               // may be null
+  const uint32_t *rows_index;
+  uint32_t rows, width;
+  float epsilon, offset, scale;
+};
+hipError_t launch_norm_add(const NormAddArgs &args, hipStream_t stream);
+
 struct DenseEmbeddingArgs {
   const int64_t *tokens;
   const uint16_t *embed;  // bf16 [vocabulary, width]
@@ -83,12 +102,14 @@ enum class GemvEpilogue : uint32_t {
   kStore = 0, kStoreF32 = 1, kAdd = 2, kGated = 3,
   kQkv = 4,    // q to out; mixed k, v straight to their cache rows
   kSsmIn = 5,  // z as it is, x | B | C through the convolution and silu, dt through softplus: all to out_f32
+  kConvIn = 6,  // columns inner .. inner + channels through the convolution and silu, the others as they are
 };
 
 struct ChunkCache {
   void *keys, *values;  // [slot][kv_heads][capacity][dim] / [...][vdim], activation type
   uint32_t capacity;    // rows per head; position p lives in row p % capacity
-  uint32_t chunk;       // positions of one chunk (capacity >= chunk); 0: no chunks
+  uint32_t span;        // positions of one chunk or window (capacity >= span); 0: all positions
+  bool sliding;         // span: the position itself and the span - 1 before it, else chunks of span
 };
 
 struct DenseGemvArgs {
@@ -99,10 +120,16 @@ struct DenseGemvArgs {
   const uint16_t *norm_weight;
   uint32_t norm_groups;
   float epsilon;
+  // a pending sublayer output joins the f32 row first (see NormAddArgs); the new row goes to stream_out
+  const float *pending;
+  const uint16_t *pending_weight;
+  float *stream_out;
+  float pending_scale, norm_offset;
   const uint16_t *w, *w_up;
   uint32_t n, k;
   GemvEpilogue epilogue;
   uint32_t activation;
+  float limit, softcap;
   void *out;
   float *out_f32;
   // kQkv
@@ -110,7 +137,7 @@ struct DenseGemvArgs {
   uint32_t n_q, n_k, dim, vdim, kv_heads;
   ChunkCache cache;
   ValueMix mix;
-  // kSsmIn
+  // kSsmIn, kConvIn
   const uint16_t *conv, *conv_bias, *dt_bias;
   float *conv_state;  // f32 [slot][taps][channels], position p in row p % taps
   uint32_t inner, channels, taps;
@@ -120,11 +147,27 @@ hipError_t launch_dense_gemv(const DenseGemvArgs &args, hipStream_t stream);
 
 // ---- attention ---------------------------------------------------------------------------------------
 
-// q | k | v rows of m new tokens at positions state[0] .. + m - 1; earlier keys of the first token's
-// chunk come from the cache.  score = cap tanh(scale q k / cap); the sink joins the denominator only.
+// Norm per head (weights over dim, shared by the heads) and rotation of queries and keys, in this order:
+// component i < dims / 2 turns with component i + dims / 2 by position * frequencies[i].
+struct HeadRotation {
+  const uint16_t *q_norm, *k_norm;  // bf16 [dim]
+  const double *frequencies;        // [dims / 2]
+  uint32_t dims;                    // 0: no rotation
+  float epsilon;
+};
+
+// q | k | v rows of m new tokens at positions state[0] .. + m - 1; earlier keys that the first token sees
+// come from the cache.  score = cap tanh(scale q k / cap); the sink joins the denominator only.
 struct ChunkAttentionArgs {
   bool f32;
-  const void *qkv;  // [m, heads * dim + kv_heads * (dim + vdim)]; one token: only q is read
+  const void *qkv;  // [m, ld]: heads * dim, kv_heads * dim, kv_heads * vdim; one token: only q is read
+  uint32_t ld, ld_out;
+  float out_scale;
+  // one token with row: the raw float32 q | k | v; its norm, rotation and cache rows are part of the launch,
+  // and the output is float32 in out_row
+  const float *row;
+  HeadRotation rotation;
+  float *out_row;
   ChunkCache cache;
   const uint16_t *sink;  // bf16 [heads], may be null
   const uint32_t *state;
@@ -139,6 +182,8 @@ bool chunk_attention_ok(const ChunkAttentionArgs &args);
 hipError_t launch_chunk_attention(const ChunkAttentionArgs &args, hipStream_t stream);
 // k, v of the step's tokens into their cache rows (those that the ring still holds afterwards).
 hipError_t launch_chunk_cache_write(const ChunkAttentionArgs &args, hipStream_t stream);
+// Norm and rotation of the q and k columns, in place.
+hipError_t launch_rotate_heads(const ChunkAttentionArgs &args, hipStream_t stream);
 
 // ---- Mamba-2 ------------------------------------------------------------------------------------------
 
@@ -162,6 +207,41 @@ constexpr uint32_t kSsmChunk = 64;
 size_t ssm_workspace_bytes(const SsmArgs &args);
 hipError_t launch_ssm_step(const SsmArgs &args, hipStream_t stream);
 hipError_t launch_ssm_prefill(const SsmArgs &args, hipStream_t stream);
+
+// ---- gated delta rule --------------------------------------------------------------------------------------
+
+// Per head, with unit keys and queries (queries also / sqrt(dim)), decay per key channel, state S [dim][vdim]:
+//   S <- diag(g) S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q
+//   out = o / rms(o) * norm * sigmoid(gate) * out_scale
+// g = exp(-exp(a_log) softplus(decay + dt_bias)).  q, k (kv_heads) and v pass a convolution and silu first.
+struct DeltaArgs {
+  bool f32;
+  uint32_t m, heads, kv_heads, dim, vdim, taps;
+  const uint32_t *step;  // state words
+  float epsilon, out_scale;
+  const uint16_t *conv, *dt_bias, *a_log, *norm;  // conv [q | k | v channels][taps]
+  float *conv_state;     // [slot][taps][channels]
+  float *state;          // [slot][heads][dim][vdim]
+  // more than one token
+  const void *projected;  // activation type, row stride ld: q | k | v before the convolution
+  uint32_t ld;
+  const float *beta;      // f32 [m, heads], before the sigmoid
+  const float *decay;     // f32 [m, heads * dim]
+  const void *gate;       // activation type [m, heads * vdim], before the sigmoid
+  void *out;              // activation type, row stride ld_out
+  uint32_t ld_out;
+  void *workspace;
+  size_t workspace_bytes;
+  // one token: float32 rows; decay = w_decay decay_in, gate = w_gate gate_in inside the launch
+  const float *row, *row_beta, *decay_in, *gate_in;  // row: q | k | v behind the convolution and silu
+  const uint16_t *w_decay, *w_gate;                  // [heads * dim][decay_rank], [heads * vdim][gate_rank]
+  uint32_t decay_rank, gate_rank;
+  float *out_row;
+};
+constexpr uint32_t kDeltaChunk = 64, kDeltaMaxWidth = 256, kDeltaMaxRank = 4096;
+size_t delta_workspace_bytes(const DeltaArgs &args);
+hipError_t launch_delta_step(const DeltaArgs &args, hipStream_t stream);
+hipError_t launch_delta_prefill(const DeltaArgs &args, hipStream_t stream);
 
 // ---- routed experts -------------------------------------------------------------------------------------
 

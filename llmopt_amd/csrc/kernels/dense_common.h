@@ -1,5 +1,5 @@
 // Shared device helpers of the kernels over bfloat16 weights (dense_gemm.hip, dense_gemv.hip,
-// chunk_attention.hip, ssm.hip, moe.hip).  Every kernel is a template over the element type T of the
+// chunk_attention.hip, ssm.hip, delta.hip, moe.hip).  Every kernel is a template over the element type T of the
 // activations: __bf16 (products on the bfloat16 matrix cores) or float (products on the float32
 // matrix cores, v_mfma_f32_16x16x4_f32: no reduced precision anywhere).  Accumulation is float32 in both.
 #pragma once
@@ -78,6 +78,14 @@ __device__ __forceinline__ f32x4 mma_wide_b(bf16x8 a, const WideFrag<__bf16> &b,
   return mma(a, b.lo, mma(a, b.hi, c));
 }
 
+// Both operands wide: everything but the product of the two low parts.
+__device__ __forceinline__ f32x4 mma_wide_both(const WideFrag<float> &a, const WideFrag<float> &b, f32x4 c) {
+  return mma(a.v, b.v, c);
+}
+__device__ __forceinline__ f32x4 mma_wide_both(const WideFrag<__bf16> &a, const WideFrag<__bf16> &b, f32x4 c) {
+  return mma(a.hi, b.hi, mma(a.lo, b.hi, mma(a.hi, b.lo, c)));
+}
+
 // Eight consecutive elements from p, of which `count` (possibly <= 0 or > 8) exist; the rest are zero.
 // vec: p is aligned to the whole piece and pieces are never partial (count >= 8 or count <= 0).
 template <typename T>
@@ -113,10 +121,27 @@ __device__ __forceinline__ float tanh_f32(float z) {
 __device__ __forceinline__ float softplus_f32(float z) { return z > 20.0f ? z : log1pf(expf(z)); }
 
 // Activation of a gated feed-forward.
-enum GateActivation : uint32_t { kGateSilu = 0, kGateGeluTanh = 1 };
+enum GateActivation : uint32_t { kGateSilu = 0, kGateGeluTanh = 1, kGateClamped = 2 };
 __device__ __forceinline__ float gate_activation(float z, uint32_t kind) {
   if (kind == kGateGeluTanh) return 0.5f * z * (1.0f + tanh_f32(0.7978845608028654f * (z + 0.044715f * z * z * z)));
   return silu_f32(z);
+}
+
+// act(gate) up; clamped: both halves limited, a steeper sigmoid, and one more than the up half.
+__device__ __forceinline__ float gated_value(float gate, float up, uint32_t kind, float limit) {
+  if (kind == kGateClamped) {
+    const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
+    return g * sigmoid_f32(1.702f * g) * (u + 1.0f);
+  }
+  return gate_activation(gate, kind) * up;
+}
+__device__ __forceinline__ float soft_capped(float z, float cap) { return cap > 0.0f ? cap * tanh_f32(z / cap) : z; }
+
+// Cosine and sine of position * frequency: the angle is reduced to one turn before it is rounded to float32.
+__device__ __forceinline__ void turn(uint32_t position, double frequency, float &cosine, float &sine) {
+  constexpr double kTurn = 6.283185307179586476925;
+  const double angle = (double)position * frequency;
+  sincosf((float)(angle - kTurn * rint(angle / kTurn)), &sine, &cosine);
 }
 
 // Sum over the 64 lanes of a wave, in every lane.

@@ -76,6 +76,10 @@ __device__ __forceinline__ void emit(const DenseLinearArgs &a, uint32_t r, uint3
       store4(static_cast<T *>(a.out) + (size_t)r * a.ld_out + c, v, count, (a.ld_out & 3) == 0);
       return;
     case DenseEpilogue::kStoreF32:
+      if (a.softcap > 0.0f) {
+#pragma unroll
+        for (int i = 0; i < 4; ++i) v[i] = soft_capped(v[i], a.softcap);
+      }
       store4(a.out_f32 + (size_t)r * a.ld_f32 + c, v, count, (a.ld_f32 & 3) == 0);
       return;
     case DenseEpilogue::kAdd: {
@@ -156,7 +160,7 @@ __device__ __forceinline__ void emit_tile(const DenseLinearArgs &a, const f32x4 
         if (c >= a.n) continue;
         f32x4 v;
 #pragma unroll
-        for (int e = 0; e < 4; ++e) v[e] = gate_activation(acc[i][j][e], a.activation) * acc[i][j + 1][e];
+        for (int e = 0; e < 4; ++e) v[e] = gated_value(acc[i][j][e], acc[i][j + 1][e], a.activation, a.limit);
         emit<T>(a, r, c, v);
       }
     } else {
@@ -319,7 +323,7 @@ __device__ __forceinline__ void emit_rows(const DenseLinearArgs &a, const f32x4 
       f32x4 v;
       if (GATED) {
 #pragma unroll
-        for (int e = 0; e < 4; ++e) v[e] = gate_activation(acc[i][2 * j][e], a.activation) * acc[i][2 * j + 1][e];
+        for (int e = 0; e < 4; ++e) v[e] = gated_value(acc[i][2 * j][e], acc[i][2 * j + 1][e], a.activation, a.limit);
       } else {
         v = acc[i][j];
         if (a.epilogue == DenseEpilogue::kQkv && r_in_tile < m_rows) mix_values(a, r, c, v);
@@ -581,6 +585,88 @@ __global__ __launch_bounds__(256) void dense_norm_vec_kernel(DenseNormArgs a) {
   }
 }
 
+// A workgroup a row.  VEC: eight values a thread and piece in registers (width % 8 == 0, at most 8 pieces),
+// else the row's parts are read again from cache.
+template <typename T, bool VEC>
+__global__ __launch_bounds__(256) void norm_add_kernel(NormAddArgs a) {
+  __shared__ float scratch[4];
+  const uint32_t r = blockIdx.x, source = a.rows_index ? a.rows_index[r] : r;
+  const float *x = a.x + (size_t)source * a.width, *y = a.y ? a.y + (size_t)source * a.width : nullptr;
+  const __bf16 *add = reinterpret_cast<const __bf16 *>(a.add_weight), *norm = reinterpret_cast<const __bf16 *>(a.norm_weight);
+  float *out = a.stream_out ? a.stream_out + (size_t)r * a.width : nullptr;
+  T *operand = a.operand ? static_cast<T *>(a.operand) + (size_t)r * a.width : nullptr;
+  if (VEC) {
+    f32x8 v[8], z[8];
+    float sum = 0.0f;
+#pragma unroll
+    for (int q = 0; q < 8; ++q) {
+      const uint32_t i = (q * 256 + threadIdx.x) * 8;
+      if (i >= a.width) break;
+      v[q] = *reinterpret_cast<const f32x8 *>(x + i);
+      if (y) {
+        z[q] = *reinterpret_cast<const f32x8 *>(y + i);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) sum += z[q][e] * z[q][e];
+      }
+    }
+    if (y) {
+      sum = block_sum<4>(sum, scratch);
+      const float factor = a.scale / sqrtf(sum / (float)a.width + a.epsilon);
+#pragma unroll
+      for (int q = 0; q < 8; ++q) {
+        const uint32_t i = (q * 256 + threadIdx.x) * 8;
+        if (i >= a.width) break;
+        const bf16x8 w = *reinterpret_cast<const bf16x8 *>(add + i);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) v[q][e] = fmaf(z[q][e] * factor, a.offset + (float)w[e], v[q][e]);
+      }
+    }
+    float inverse = 1.0f;
+    if (norm) {
+      sum = 0.0f;
+#pragma unroll
+      for (int q = 0; q < 8; ++q) {
+        if ((q * 256 + threadIdx.x) * 8 >= a.width) break;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) sum += v[q][e] * v[q][e];
+      }
+      inverse = 1.0f / sqrtf(block_sum<4>(sum, scratch) / (float)a.width + a.epsilon);
+    }
+#pragma unroll
+    for (int q = 0; q < 8; ++q) {
+      const uint32_t i = (q * 256 + threadIdx.x) * 8;
+      if (i >= a.width) break;
+      if (out) *reinterpret_cast<f32x8 *>(out + i) = v[q];
+      if (!operand) continue;
+      if (norm) {
+        const bf16x8 w = *reinterpret_cast<const bf16x8 *>(norm + i);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) v[q][e] *= inverse * (a.offset + (float)w[e]);
+      }
+      *reinterpret_cast<Frag<T> *>(operand + i) = convert_frag<T>(v[q]);
+    }
+    return;
+  }
+  float factor = 0.0f;
+  if (y) {
+    float sum = 0.0f;
+    for (uint32_t i = threadIdx.x; i < a.width; i += 256) sum += y[i] * y[i];
+    factor = a.scale / sqrtf(block_sum<4>(sum, scratch) / (float)a.width + a.epsilon);
+  }
+  auto value = [&](uint32_t i) { return y ? fmaf(y[i] * factor, a.offset + (float)add[i], x[i]) : x[i]; };
+  float inverse = 1.0f;
+  if (norm) {
+    float sum = 0.0f;
+    for (uint32_t i = threadIdx.x; i < a.width; i += 256) sum += value(i) * value(i);
+    inverse = 1.0f / sqrtf(block_sum<4>(sum, scratch) / (float)a.width + a.epsilon);
+  }
+  for (uint32_t i = threadIdx.x; i < a.width; i += 256) {
+    const float v = value(i);
+    if (out) out[i] = v;
+    if (operand) operand[i] = (T)(norm ? v * inverse * (a.offset + (float)norm[i]) : v);
+  }
+}
+
 __global__ __launch_bounds__(256) void dense_embedding_kernel(DenseEmbeddingArgs a) {
   const uint32_t t = blockIdx.x;
   const int64_t token = a.tokens[t];
@@ -611,6 +697,18 @@ hipError_t launch_dense_norm(const DenseNormArgs &a, hipStream_t stream) {
   if (bytes > 60 * 1024) return hipErrorInvalidValue;
   if (a.f32) dense_norm_kernel<float><<<a.rows, 256, bytes, stream>>>(a);
   else dense_norm_kernel<__bf16><<<a.rows, 256, bytes, stream>>>(a);
+  return hipGetLastError();
+}
+
+hipError_t launch_norm_add(const NormAddArgs &a, hipStream_t stream) {
+  const bool vec = a.width % 8 == 0 && a.width <= 8 * 256 * 8;
+  if (a.f32) {
+    if (vec) norm_add_kernel<float, true><<<a.rows, 256, 0, stream>>>(a);
+    else norm_add_kernel<float, false><<<a.rows, 256, 0, stream>>>(a);
+  } else {
+    if (vec) norm_add_kernel<__bf16, true><<<a.rows, 256, 0, stream>>>(a);
+    else norm_add_kernel<__bf16, false><<<a.rows, 256, 0, stream>>>(a);
+  }
   return hipGetLastError();
 }
 

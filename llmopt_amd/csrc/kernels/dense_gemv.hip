@@ -55,9 +55,92 @@ __device__ __forceinline__ void stage_normed_row(const DenseGemvArgs &a, float *
     if (i < k) {
       f32x4 out;
 #pragma unroll
-      for (int e = 0; e < 4; ++e) out[e] = v[q][e] * inverse * (float)w[q][e];
+      for (int e = 0; e < 4; ++e) out[e] = v[q][e] * inverse * (a.norm_offset + (float)w[q][e]);
       *reinterpret_cast<f32x4 *>(xs + staged_index(i, plane)) = out;
     }
+  }
+  __syncthreads();
+}
+
+// The f32 row x with a pending sublayer output added behind its norm (the first workgroup stores the new row),
+// normalised itself where the launch carries a norm weight.  A row of at most PIECES * 1024 values.
+template <int PIECES, typename Ahead>
+__device__ __forceinline__ void stage_pending_row(const DenseGemvArgs &a, float *xs, uint32_t plane, float *scratch,
+                                                  Ahead ahead) {
+  const uint32_t k = a.k;
+  const float *x = static_cast<const float *>(a.x);
+  const __bf16 *add = reinterpret_cast<const __bf16 *>(a.pending_weight);
+  const __bf16 *weight = reinterpret_cast<const __bf16 *>(a.norm_weight);
+  f32x4 v[PIECES], y[PIECES];
+  bf16x4 w[PIECES];
+  float sum = 0.0f;
+#pragma unroll
+  for (int q = 0; q < PIECES; ++q) {
+    const uint32_t i = (q * kWaves * 64 + threadIdx.x) * 4;
+    v[q] = y[q] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+    w[q] = bf16x4{0, 0, 0, 0};
+    if (i < k) {
+      v[q] = *reinterpret_cast<const f32x4 *>(x + i);
+      y[q] = *reinterpret_cast<const f32x4 *>(a.pending + i);
+      w[q] = *reinterpret_cast<const bf16x4 *>(add + i);
+    }
+  }
+  ahead();
+#pragma unroll
+  for (int q = 0; q < PIECES; ++q)
+    sum += y[q][0] * y[q][0] + y[q][1] * y[q][1] + y[q][2] * y[q][2] + y[q][3] * y[q][3];
+  const float factor = a.pending_scale / sqrtf(block_sum<kWaves>(sum, scratch) / (float)k + a.epsilon);
+  sum = 0.0f;
+#pragma unroll
+  for (int q = 0; q < PIECES; ++q)
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      v[q][e] = fmaf(y[q][e] * factor, a.norm_offset + (float)w[q][e], v[q][e]);
+      sum += v[q][e] * v[q][e];
+    }
+  if (blockIdx.x == 0 && a.stream_out) {
+#pragma unroll
+    for (int q = 0; q < PIECES; ++q) {
+      const uint32_t i = (q * kWaves * 64 + threadIdx.x) * 4;
+      if (i < k) *reinterpret_cast<f32x4 *>(a.stream_out + i) = v[q];
+    }
+  }
+  float inverse = 1.0f;
+  if (weight) inverse = 1.0f / sqrtf(block_sum<kWaves>(sum, scratch) / (float)k + a.epsilon);
+#pragma unroll
+  for (int q = 0; q < PIECES; ++q) {
+    const uint32_t i = (q * kWaves * 64 + threadIdx.x) * 4;
+    if (i < k) {
+      if (weight) {
+        const bf16x4 own = *reinterpret_cast<const bf16x4 *>(weight + i);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[q][e] *= inverse * (a.norm_offset + (float)own[e]);
+      }
+      *reinterpret_cast<f32x4 *>(xs + staged_index(i, plane)) = v[q];
+    }
+  }
+  __syncthreads();
+}
+
+// The same for any length, through the staged row.
+__device__ __forceinline__ void stage_pending_any(const DenseGemvArgs &a, float *xs, uint32_t plane, float *scratch) {
+  const uint32_t k = a.k;
+  const float *x = static_cast<const float *>(a.x);
+  float sum = 0.0f;
+  for (uint32_t i = threadIdx.x; i < k; i += kWaves * 64) sum += a.pending[i] * a.pending[i];
+  const float factor = a.pending_scale / sqrtf(block_sum<kWaves>(sum, scratch) / (float)k + a.epsilon);
+  sum = 0.0f;
+  for (uint32_t i = threadIdx.x; i < k; i += kWaves * 64) {
+    const float w = a.norm_offset + (float)reinterpret_cast<const __bf16 *>(a.pending_weight)[i];
+    const float v = fmaf(a.pending[i] * factor, w, x[i]);
+    if (blockIdx.x == 0 && a.stream_out) a.stream_out[i] = v;
+    sum += v * v;
+    xs[staged_index(i, plane)] = v;
+  }
+  if (a.norm_weight) {
+    const float inverse = 1.0f / sqrtf(block_sum<kWaves>(sum, scratch) / (float)k + a.epsilon);
+    for (uint32_t i = threadIdx.x; i < k; i += kWaves * 64)
+      xs[staged_index(i, plane)] *= inverse * (a.norm_offset + (float)reinterpret_cast<const __bf16 *>(a.norm_weight)[i]);
   }
   __syncthreads();
 }
@@ -71,6 +154,13 @@ __device__ __forceinline__ void stage_activation(const DenseGemvArgs &a, float *
   const __bf16 *weight = reinterpret_cast<const __bf16 *>(a.norm_weight);
   // whole pieces behind the row's end read as zeros
   for (uint32_t i = k + threadIdx.x; i < ((k + 7) & ~7u); i += kWaves * 64) xs[staged_index(i, plane)] = 0.0f;
+  if (a.pending) {
+    if ((k & 3) == 0 && k <= 2 * 4 * kWaves * 64) return stage_pending_row<2>(a, xs, plane, scratch, ahead);
+    if ((k & 3) == 0 && k <= 4 * 4 * kWaves * 64) return stage_pending_row<4>(a, xs, plane, scratch, ahead);
+    if ((k & 3) == 0 && k <= 8 * 4 * kWaves * 64) return stage_pending_row<8>(a, xs, plane, scratch, ahead);
+    ahead();
+    return stage_pending_any(a, xs, plane, scratch);
+  }
   if (weight == nullptr) {
     if ((k & 7) == 0 && k <= 8 * 8 * kWaves * 64) {
       f32x8 v[8];
@@ -117,7 +207,7 @@ __device__ __forceinline__ void stage_activation(const DenseGemvArgs &a, float *
     sum = block_sum<kWaves>(sum, scratch);
     const float inverse = 1.0f / sqrtf(sum / (float)part + a.epsilon);
     for (uint32_t i = g * part + threadIdx.x; i < (g + 1) * part; i += kWaves * 64)
-      xs[staged_index(i, plane)] = x[i] * inverse * (float)weight[i];
+      xs[staged_index(i, plane)] = x[i] * inverse * (a.norm_offset + (float)weight[i]);
   }
   __syncthreads();
 }
@@ -186,19 +276,23 @@ __device__ __forceinline__ float bf16_at(const uint16_t *p, size_t i) {
   return (float)reinterpret_cast<const __bf16 *>(p)[i];
 }
 
+// Channel c's input v of the short convolution into its ring; the output behind silu.
+__device__ __forceinline__ float conv_step(const DenseGemvArgs &a, uint32_t c, float v) {
+  const uint32_t position = a.state[kStatePosition], slot = a.state[kStateSlot];
+  float *ring = a.conv_state + (size_t)slot * a.taps * a.channels + c;
+  float sum = (a.conv_bias ? bf16_at(a.conv_bias, c) : 0.0f) + bf16_at(a.conv, (size_t)c * a.taps + a.taps - 1) * v;
+  for (uint32_t back = 1; back < a.taps; ++back)
+    if (back <= position)
+      sum = fmaf(bf16_at(a.conv, (size_t)c * a.taps + a.taps - 1 - back),
+                 ring[(size_t)((position - back) % a.taps) * a.channels], sum);
+  ring[(size_t)(position % a.taps) * a.channels] = v;
+  return silu_f32(sum);
+}
+
 // Row n of the recurrent layer's input projection.
 __device__ __forceinline__ void ssm_in_store(const DenseGemvArgs &a, uint32_t n, float v) {
   if (n >= a.inner && n < a.inner + a.channels) {
-    const uint32_t c = n - a.inner;
-    const uint32_t position = a.state[kStatePosition], slot = a.state[kStateSlot];
-    float *ring = a.conv_state + (size_t)slot * a.taps * a.channels + c;
-    float sum = bf16_at(a.conv_bias, c) + bf16_at(a.conv, (size_t)c * a.taps + a.taps - 1) * v;
-    for (uint32_t back = 1; back < a.taps; ++back)
-      if (back <= position)
-        sum = fmaf(bf16_at(a.conv, (size_t)c * a.taps + a.taps - 1 - back),
-                   ring[(size_t)((position - back) % a.taps) * a.channels], sum);
-    ring[(size_t)(position % a.taps) * a.channels] = v;
-    v = silu_f32(sum);
+    v = conv_step(a, n - a.inner, v);
   } else if (n >= a.inner + a.channels) {
     v = softplus_f32(v + bf16_at(a.dt_bias, n - a.inner - a.channels));
   }
@@ -209,14 +303,17 @@ template <typename T>
 __device__ __forceinline__ void gemv_epilogue(const DenseGemvArgs &a, uint32_t n, float v, float up) {
   switch (a.epilogue) {
     case GemvEpilogue::kStore: static_cast<T *>(a.out)[n] = (T)v; return;
-    case GemvEpilogue::kStoreF32: a.out_f32[n] = v; return;
+    case GemvEpilogue::kStoreF32: a.out_f32[n] = soft_capped(v, a.softcap); return;
     case GemvEpilogue::kAdd: a.out_f32[n] += v; return;
-    case GemvEpilogue::kGated: a.out_f32[n] = gate_activation(v, a.activation) * up; return;
+    case GemvEpilogue::kGated: a.out_f32[n] = gated_value(v, up, a.activation, a.limit); return;
     case GemvEpilogue::kQkv:
       if (n < a.n_q) static_cast<T *>(a.out)[n] = (T)v;
       else cache_store<T>(a, n, v);
       return;
     case GemvEpilogue::kSsmIn: ssm_in_store(a, n, v); return;
+    case GemvEpilogue::kConvIn:
+      a.out_f32[n] = n >= a.inner && n < a.inner + a.channels ? conv_step(a, n - a.inner, v) : v;
+      return;
   }
 }
 

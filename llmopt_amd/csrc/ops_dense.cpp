@@ -8,68 +8,13 @@
 // What moves from step to step - the position of the step's first token and the sequence's state slot -
 // is read from two device words (`step words`: u32 position, u32 slot), so that one captured list
 // serves every step and every slot.
-#include <cmath>
 #include <cstring>
 
-#include "kernels/dense.h"
 #include "kernels/kernels.h"
-#include "runtime.h"
+#include "ops_dense.h"
 
 namespace llmopt {
 namespace {
-
-const uint16_t *as_bf16(const BoundBuffer &b) { return reinterpret_cast<const uint16_t *>(b.device); }
-float *as_f32(const BoundBuffer &b) { return reinterpret_cast<float *>(b.device); }
-const uint32_t *as_u32(const BoundBuffer &b) { return reinterpret_cast<const uint32_t *>(b.device); }
-
-int launched(hipError_t status, const char *name) {
-  if (status != hipSuccess) return fail(LLMOPT_ERR_FAILURE, "%s launch failed: %s", name, hipGetErrorString(status));
-  return LLMOPT_OK;
-}
-
-size_t round_up_256(size_t bytes) { return (bytes + 255) & ~(size_t)255; }
-
-bool valid_epsilon(float epsilon) { return std::isfinite(epsilon) && epsilon >= 0.0f; }
-
-int require_positive(const DispatchRecord &record, std::initializer_list<uint32_t> values) {
-  for (uint32_t value : values)
-    if (value == 0) return fail(LLMOPT_ERR_INVALID, "%s requires positive sizes", record.name.c_str());
-  return LLMOPT_OK;
-}
-
-int require_sizes(const DispatchRecord &record, std::initializer_list<std::pair<int, uint64_t>> sizes) {
-  for (const auto &size : sizes) {
-    char name[32];
-    snprintf(name, sizeof name, "operand %d", size.first);
-    if (int status = require_buffer_size(record.buffers[size.first], size.second, name)) return status;
-  }
-  return LLMOPT_OK;
-}
-
-// Scratch of one entry, cut into aligned parts.
-class Scratch {
- public:
-  size_t want(size_t bytes) {
-    const size_t at = total_;
-    total_ += round_up_256(bytes);
-    return at;
-  }
-  bool get(llmopt_hip_context *context) {
-    base_ = static_cast<uint8_t *>(context_workspace(context, total_));
-    return base_ != nullptr;
-  }
-  template <typename P>
-  P *at(size_t offset) const {
-    return reinterpret_cast<P *>(base_ + offset);
-  }
-
- private:
-  size_t total_ = 0;
-  uint8_t *base_ = nullptr;
-};
-
-template <bool F32>
-constexpr size_t kElement = F32 ? 4 : 2;
 
 template <bool F32>
 hipError_t norm_rows(const float *x, const uint16_t *weight, void *out, uint32_t rows, uint32_t width, float epsilon,
@@ -103,18 +48,6 @@ DenseGemvArgs normed_gemv(bool f32, const float *x, const uint16_t *norm, float 
   return a;
 }
 
-DenseLinearArgs linear(bool f32, const void *x, const uint16_t *w, uint32_t m, uint32_t n, uint32_t k) {
-  DenseLinearArgs a = {};
-  a.f32 = f32;
-  a.x = x;
-  a.w = w;
-  a.m = m;
-  a.n = n;
-  a.k = k;
-  a.ldx = k;
-  return a;
-}
-
 // ---- embedding, logits ---------------------------------------------------------------------------------
 
 // {u32 m, vocabulary, width; f32 scale}; tokens i64, embedding, stream f32.
@@ -138,7 +71,7 @@ int embedding_scaled(llmopt_hip_context *context, const DispatchRecord &record) 
 }
 
 // {u32 rows, width, vocabulary; f32 epsilon; u32 m}; stream f32 [m, width], row indices u32 [rows] (each
-// below m), norm weight, head, logits f32 [rows, vocabulary].  m == 1: the indices are not read.
+// below m), norm weight, head, logits f32 [rows, vocabulary].  One row of one: the indices are not read.
 template <bool F32>
 int rms_logits(llmopt_hip_context *context, const DispatchRecord &record) {
   if (int status = require_buffer_count(record, 5)) return status;
@@ -167,7 +100,7 @@ int rms_logits(llmopt_hip_context *context, const DispatchRecord &record) {
   if (!scratch.get(context)) return LLMOPT_ERR_FAILURE;
   if (int status = launched(norm_rows<F32>(as_f32(record.buffers[0]), as_bf16(record.buffers[2]),
                                            scratch.at<void>(normed), rows, width, epsilon,
-                                           m == 1 ? nullptr : as_u32(record.buffers[1]), context->stream),
+                                           m == 1 && rows == 1 ? nullptr : as_u32(record.buffers[1]), context->stream),
                             name))
     return status;
   DenseLinearArgs a = linear(F32, scratch.at<void>(normed), as_bf16(record.buffers[3]), rows, vocabulary, width);
@@ -282,7 +215,7 @@ int chunk_attention(llmopt_hip_context *context, const DispatchRecord &record) {
   a.softcap = param_f32(record, 40);
   if (int status = require_positive(record, {a.m, a.heads, a.kv_heads, a.dim, a.vdim, a.cache.capacity, slots}))
     return status;
-  if (a.cache.chunk > a.cache.capacity || a.heads % a.kv_heads != 0 || !std::isfinite(a.scale) || !(a.softcap >= 0.0f))
+  if (a.cache.span > a.cache.capacity || a.heads % a.kv_heads != 0 || !std::isfinite(a.scale) || !(a.softcap >= 0.0f))
     return fail(LLMOPT_ERR_INVALID, "%s input metadata is inconsistent", name);
   if (!chunk_attention_ok(a))
     return fail(LLMOPT_ERR_INVALID, "%s takes heads of at most 256 values", name);
@@ -299,6 +232,9 @@ int chunk_attention(llmopt_hip_context *context, const DispatchRecord &record) {
   a.sink = has_sink ? as_bf16(record.buffers[1]) : nullptr;
   a.state = as_u32(record.buffers[2]);
   a.out = record.buffers[5].device;
+  a.ld = n;
+  a.ld_out = a.heads * a.vdim;
+  a.out_scale = 1.0f;
   a.workspace_bytes = chunk_attention_workspace_bytes(a);
   if (a.workspace_bytes) {
     a.workspace = context_workspace(context, a.workspace_bytes);

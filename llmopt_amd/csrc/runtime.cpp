@@ -52,6 +52,7 @@ void register_cache_kernels(std::vector<KernelEntryPoint> &table);
 void register_attention_kernels(std::vector<KernelEntryPoint> &table);
 void register_glue_kernels(std::vector<KernelEntryPoint> &table);
 void register_dense_kernels(std::vector<KernelEntryPoint> &table);
+void register_parallel_kernels(std::vector<KernelEntryPoint> &table);
 
 const std::vector<KernelEntryPoint> &kernel_table() {
   static const std::vector<KernelEntryPoint> table = [] {
@@ -61,6 +62,7 @@ const std::vector<KernelEntryPoint> &kernel_table() {
     register_attention_kernels(entries);
     register_glue_kernels(entries);
     register_dense_kernels(entries);
+    register_parallel_kernels(entries);
     return entries;
   }();
   return table;

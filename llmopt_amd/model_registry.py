@@ -15,7 +15,7 @@ from __future__ import annotations
 import json
 import os
 
-from .layered_model import LayeredModel
+from .layered_model import DESIGNS, LayeredModel
 from .native import Runtime
 from .w4a16_model import W4a16Model
 
@@ -51,5 +51,6 @@ def load_model(directory: str, runtime: Runtime | None = None, **options):
     return model_class(config).load(runtime or Runtime(), directory, config, **options)
 
 
-register("Barovik", LayeredModel)
+for _design in DESIGNS:
+    register(_design, LayeredModel)
 register("W4A16Transformer", W4a16Model)

@@ -7,7 +7,8 @@ position 0, where the kernels take state and history as zero, and rings only han
 sequence itself has written.
 
 A key / value ring keeps `capacity` positions per head (position p in row p % capacity).  Attention over
-chunks needs one chunk; attention over the whole sequence needs the longest context the pool is made for.
+chunks or a sliding window needs one of them; attention over the whole sequence needs the longest context the
+pool is made for.
 """
 from __future__ import annotations
 
@@ -26,20 +27,20 @@ class RingShape:
     kv_heads: int
     dim: int
     vdim: int
-    chunk: int     # 0: the whole sequence
+    span: int      # chunk or window; 0: the whole sequence
     capacity: int
 
     @staticmethod
-    def of(kv_heads: int, dim: int, vdim: int, chunk: int, max_context: int) -> "RingShape":
-        # positions below max_context never leave the first chunk when that is at least as long
-        if chunk == 0 or chunk >= max_context:
+    def of(kv_heads: int, dim: int, vdim: int, span: int, max_context: int) -> "RingShape":
+        # positions below max_context never leave the first chunk or window when that is at least as long
+        if span == 0 or span >= max_context:
             return RingShape(kv_heads, dim, vdim, 0, max_context)
-        return RingShape(kv_heads, dim, vdim, chunk, chunk)
+        return RingShape(kv_heads, dim, vdim, span, span)
 
 
 @dataclass(frozen=True)
 class RecurrentShape:
-    """Convolution inputs and state of one recurrent layer."""
+    """Convolution inputs and state (state x vdim values per head) of one recurrent layer."""
     heads: int
     vdim: int
     state: int
@@ -60,16 +61,18 @@ class StatePool:
         self.slots, self.max_context = slots, max_context
         self._free = list(range(slots))[::-1]
         self._live: set[int] = set()
-        self.regions = []  # per layer: (keys, values) or (convolution ring, state)
         self.bytes = 0
-        for shape in shapes:
-            if isinstance(shape, RingShape):
-                rows = slots * shape.kv_heads * shape.capacity * element_bytes
-                sizes = (rows * shape.dim, rows * shape.vdim)
-            else:
-                sizes = (slots * shape.taps * shape.channels * 4, slots * shape.heads * shape.vdim * shape.state * 4)
-            self.bytes += sum(sizes)
-            self.regions.append(tuple(runtime.create_buffer(size) for size in sizes))
+        # per layer, for each of its shapes: (keys, values) or (convolution ring, state)
+        self.regions = [tuple(self._region(runtime, shape, element_bytes) for shape in layer) for layer in shapes]
+
+    def _region(self, runtime: Runtime, shape, element_bytes: int) -> tuple:
+        if isinstance(shape, RingShape):
+            rows = self.slots * shape.kv_heads * shape.capacity * element_bytes
+            sizes = (rows * shape.dim, rows * shape.vdim)
+        else:
+            sizes = (self.slots * shape.taps * shape.channels * 4, self.slots * shape.heads * shape.vdim * shape.state * 4)
+        self.bytes += sum(sizes)
+        return tuple(runtime.create_buffer(size) for size in sizes)
 
     @property
     def free_slots(self) -> int:

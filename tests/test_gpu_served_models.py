@@ -77,4 +77,4 @@ def test_command_line(folder, capsys):
     runtime = model_registry.Runtime()
     assert [int(t) for t in capsys.readouterr().out.split()] == generate_by_steps(runtime, weights, prompt, 4)
     assert cli.main(["models"]) == 0
-    assert capsys.readouterr().out.split() == ["Barovik", "W4A16Transformer"]
+    assert capsys.readouterr().out.split() == ["Barovik", "Koketar", "W4A16Transformer"]

@@ -82,7 +82,7 @@ def test_state_pool():
     assert RingShape.of(2, 8, 4, 16, 100) == RingShape(2, 8, 4, 16, 16)
     assert RingShape.of(2, 8, 4, 0, 100) == RingShape.of(2, 8, 4, 100, 100) == RingShape(2, 8, 4, 0, 100)
     runtime = FakeRuntime()
-    pool = StatePool(runtime, [RingShape.of(2, 8, 4, 16, 100)], slots=2, max_context=100, element_bytes=2)
+    pool = StatePool(runtime, [(RingShape.of(2, 8, 4, 16, 100),)], slots=2, max_context=100, element_bytes=2)
     assert runtime.sizes == [2 * 2 * 16 * 2 * 8, 2 * 2 * 16 * 2 * 4]
     a, b = pool.open(), pool.open()
     assert a.slot != b.slot and pool.free_slots == 0
