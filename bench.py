@@ -668,20 +668,21 @@ class TiledWeights:
         return name in self.shapes
 
     def __getitem__(self, name):
-        shape = self.shapes[name]
+        shape = tuple(PARALLEL_RANK if size is None else size for size in self.shapes[name])
         kind = name.rsplit(".", 1)[-1]
         if "norm" in kind:
             return self.convert(np.ones(shape))
-        gain = 0.5 if kind in ("A_log", "dt_bias", "D", "b", "sink", "conv", "embed") or not shape else shape[-1] ** -0.5
+        small = kind in ("A_log", "dt_bias", "D", "b", "sink") and len(shape) < 2 or kind in ("conv", "embed") or not shape
+        gain = 0.5 if small else shape[-1] ** -0.5
         return np.resize(self.convert(self.block * np.float32(gain)), shape)
 
 
 def layered_work(model, m, context):
     """Algorithmic flops of the products of a prefill of m tokens, and the bytes one decode step reads and
     writes: weights it uses, keys and values of the chunk, recurrent state."""
-    from llmopt_amd.layered_model import AttentionMixer, DenseFfn
+    from llmopt_amd.layered_model import AttentionMixer, DenseFfn, ParallelMixer
     c, flops, weights, state = model.config, 0.0, 0, 0
-    for layer in c.layers:
+    for layer, d in zip(c.layers, model.layers):
         x, f = layer.mixer, layer.ffn
         if isinstance(x, AttentionMixer):
             columns, inner = x.columns, x.heads * x.vdim
@@ -689,12 +690,26 @@ def layered_work(model, m, context):
             keys = sum(n * (n + 1) / 2 for n in [chunk] * (m // chunk) + [m % chunk])
             flops += 2.0 * x.heads * (x.dim + x.vdim) * keys
             state += 2 * x.kv_heads * (x.dim + x.vdim) * (context % chunk + 1)
+        elif isinstance(x, ParallelMixer):
+            columns, inner, a, r = d["columns"].total, x.out, x.left, x.right
+            window = min(a.window or m, m)
+            keys = window * (window + 1) / 2 + (m - window) * window
+            flops += 2.0 * a.heads * (a.dim + a.vdim) * keys
+            state += 2 * a.kv_heads * (a.dim + a.vdim) * min(context + 1, a.window or context + 1)
+            # the recurrence in chunks of 64: three products with the state, two of a chunk's own tokens, the solves
+            flops += m * r.heads * (6.0 * r.dim * r.vdim + 64 * (2.0 * r.dim + r.vdim) + 64 * (r.dim + r.vdim))
+            state += 8 * r.heads * r.dim * r.vdim
+            low = r.heads * (r.dim * d["ranks"][0] + r.vdim * d["ranks"][1])
+            flops += 2.0 * m * low
+            weights += 2 * low
         else:
             columns, inner = x.columns, x.inner
             flops += m * (4.0 * x.inner * x.state + 2.0 * 64 * (x.inner + x.groups * x.state))
             state += 8 * x.inner * x.state
         flops += 2.0 * m * c.width * (columns + inner)
         weights += 2 * c.width * (columns + inner)
+        if f is None:
+            continue
         used = f.ff if isinstance(f, DenseFfn) else f.top * f.ff + f.shared_ff
         router = 0 if isinstance(f, DenseFfn) else f.experts + 1
         flops += 2.0 * m * c.width * (3 * used + router)
@@ -731,6 +746,139 @@ def verify_layered(runtime):
     return float(np.linalg.norm(got - want) / np.linalg.norm(want))
 
 
+def time_prompt(runtime, model, tokens):
+    """Milliseconds of a whole prompt in one portion with the logits of its last token, from graph replays."""
+    from llmopt_amd.native import DispatchList
+    m = len(tokens)
+    sequence = model.open()
+    logits = model.step(sequence, tokens, [m - 1])
+    model.close(sequence)
+    graph = runtime.begin_batch()
+    dispatches, stream = model._lists[m]
+    graph.dispatch_all(dispatches)
+    index = runtime.buffer_of_bytes(np.array([m - 1], np.uint32))
+    out = runtime.create_buffer(model.vocabulary * 4)
+    graph.dispatch_all(DispatchList([model._logits(1, m, model._work, stream, index, out)]))
+    return sorted(graph.commit_profiled_each(repeats=5))[2], bool(np.isfinite(logits).all())
+
+
+def time_token(runtime, model, tokens):
+    """One token behind len(tokens) - 1 others as a graph replay and as a retained plan (milliseconds), its logits' distance
+    from the same token's at the end of a prompt, and the plan's records."""
+    from llmopt_amd.native import DispatchList
+    context = len(tokens) - 1
+    sequence = model.open()
+    at_once = model.step(sequence, tokens, [context]).astype(np.float64)
+    model.close(sequence)
+    sequence = model.open()
+    model.step(sequence, tokens[:context])
+    plan = model.decode_plan()
+    plan.execute(tokens[-1], sequence)  # leaves the step words of a token behind the context
+    difference = float(np.linalg.norm(model.logits_row() - at_once[0]) / np.linalg.norm(at_once))
+    graph = runtime.begin_batch()
+    graph.dispatch_all(DispatchList(plan.dispatches))
+    ms = sorted(graph.commit_profiled_each(repeats=9))[4]
+    started = time.perf_counter()
+    for _ in range(20):
+        plan.execute(1, sequence)
+    wall = (time.perf_counter() - started) / 20 * 1e3
+    model.close(sequence)
+    return ms, wall, difference, len(plan.dispatches)
+
+
+# The Koketar design (window attention and the gated delta rule side by side, dense feed-forwards) at the sizes of real
+# models' layers, and beside it the same parts one after another: a Barovik decoder whose every second layer is a
+# recurrent mixer with the same state and whose others are the same attention and feed-forward.
+PARALLEL_SIZES = {
+    "1024": dict(width=1024, heads=16, kv_heads=4, dim=64, window=2048, delta_heads=8, state=128, ff=4096, layers=4),
+    "2048": dict(width=2048, heads=16, kv_heads=4, dim=128, window=2048, delta_heads=16, state=128, ff=8192, layers=4),
+    "4096": dict(width=4096, heads=32, kv_heads=8, dim=128, window=4096, delta_heads=32, state=128, ff=14336, layers=2),
+}
+PARALLEL_RANK = 128
+
+
+def parallel_configs(size):
+    z = PARALLEL_SIZES[size]
+    attention = {"heads": z["heads"], "kv_heads": z["kv_heads"], "dim": z["dim"], "vdim": z["dim"], "scale": z["dim"] ** -0.5}
+    left = {**attention, "mask": {"size": z["window"]},
+            "rot": {"base": 1e6, "dims": z["dim"], "scaling": {"factor": 4.0}}}
+    right = {"heads": z["delta_heads"], "kv_heads": z["delta_heads"], "dim": z["state"], "vdim": z["state"], "conv": 4}
+    layer = {"type": "parallel", "mlp": {"kind": "dense", "ff": z["ff"], "limit": 7.0},
+             "mixer": {"left": left, "right": right, "left_scale": 0.5, "right_scale": 0.5}}
+    common = {"vocab": LAYERED_VOCABULARY, "width": z["width"], "norm": {"eps": 1e-6}}
+    own = {**common, "architecture": "Koketar", "residual_mult": 0.5, "logit_softcap": 30.0, "layers": [layer] * z["layers"]}
+    recurrent = {"type": "mamba2", "mlp": None,
+                 "mixer": {"heads": 2 * z["delta_heads"], "vdim": z["state"] // 2, "state": z["state"], "groups": 1, "conv": 4,
+                           "norm_groups": 1}}
+    attending = {"type": "attention", "mlp": {"kind": "dense", "ff": z["ff"]},
+                 "mixer": {**attention, "softcap": 30.0, "v_mix": False, "mask": {"size": z["window"]}}}
+    like = {**common, "architecture": "Barovik", "embedding": {"scale": 1.0}, "layers": [recurrent, attending] * z["layers"]}
+    return own, like
+
+
+def verify_parallel(runtime):
+    """A small decoder of the timed one's layers, prompt and decoding, against the float64 restatement."""
+    from llmopt_amd.layered_model import LayeredConfig, LayeredModel
+    from llmopt_amd.safetensors_file import from_bfloat16
+    from oracle import parallel_model
+    config, _ = parallel_configs("1024")
+    config.update(width=256, vocab=500, layers=config["layers"][:2])
+    for layer in config["layers"]:
+        layer["mixer"]["left"].update(heads=8, kv_heads=2, mask={"size": 48})
+        layer["mixer"]["right"].update(heads=2, kv_heads=2)
+        layer["mlp"]["ff"] = 512
+    parsed = LayeredConfig.parse(config)
+    rng = np.random.default_rng(SEED + 13)
+    patterns = parsed.random_tensors(rng)
+    model = LayeredModel(runtime, parsed, patterns, slots=1, max_context=256)
+    tokens = rng.integers(0, 500, 140).tolist()
+    sequence = model.open()
+    got = np.concatenate([model.step(sequence, tokens[:130], range(130))] +
+                         [model.step(sequence, [t], [0]) for t in tokens[130:]]).astype(np.float64)
+    weights = {name: from_bfloat16(array).reshape(array.shape) for name, array in patterns.items()}
+    want = parallel_model.forward(config, weights, tokens)[0]
+    return float(np.linalg.norm(got - want) / np.linalg.norm(want))
+
+
+def bench_parallel(runtime, sizes, prompts=(512, 2048, 8192), context=2000):
+    """Prefill and decode of the Koketar design beside the Barovik decoder of the same parts, timed in turn; checked outside
+    the timed regions like bench_layered."""
+    from llmopt_amd.layered_model import LayeredConfig, LayeredModel
+    rng = np.random.default_rng(SEED + 14)
+    restated, results = verify_parallel(runtime), []
+    for size in sizes:
+        print("parallel", size, file=sys.stderr, flush=True)
+        entry = {"width": PARALLEL_SIZES[size]["width"], "prefill": [], "decode": {},
+                 "rel_l2_restatement": float("%.3g" % restated)}
+        models = []
+        for config in map(LayeredConfig.parse, parallel_configs(size)):
+            models.append(LayeredModel(runtime, config, TiledWeights(config.tensor_shapes(), rng), slots=2, max_context=16384))
+        finite = True
+        for m in prompts:
+            row = {"tokens": m}
+            for name, model in zip(("koketar", "barovik"), models):
+                ms, fine = time_prompt(runtime, model, rng.integers(0, LAYERED_VOCABULARY, m))
+                flops, _ = layered_work(model, m, context)
+                finite = finite and fine
+                row[name] = {"ms": round(ms, 4), "tokens_per_s": round(m / ms * 1e3), "TFLOPs": round(flops / ms / 1e9, 1),
+                             "mfma_frac": round(flops / ms / 1e9 / MFMA_F16_PEAK_TFLOPS, 4)}
+            entry["prefill"].append(row)
+        entry["verified"] = finite and restated <= 2e-2
+        for name, model in zip(("koketar", "barovik"), models):
+            tokens = rng.integers(0, LAYERED_VOCABULARY, context).tolist() + [1]
+            ms, wall, difference, records = time_token(runtime, model, tokens)
+            _, step_bytes = layered_work(model, 1, context)
+            entry["verified"] = bool(entry["verified"] and difference <= 0.1)
+            entry["decode"][name] = {
+                "context": context, "ms": round(ms, 4), "tokens_per_s": round(1e3 / ms, 1), "plan_wall_ms": round(wall, 4),
+                "bytes": int(step_bytes), "GBps": round(step_bytes / ms / 1e6, 1),
+                "hbm_frac": round(step_bytes / ms / 1e6 / HBM_PEAK_GBS, 4), "records": records,
+                "rel_l2_decode_against_prompt": float("%.3g" % difference)}
+        results.append(entry)
+        del models
+    return results
+
+
 def bench_layered(runtime, sizes, prompts=(512, 2048, 8192), context=2000):
     """Prefill (one portion, logits of its last token) and decode (one token after `context`, a HIP graph) of
     the layered decoders, and the same of the W4A16 transformer.  Medians of graph replays, in turn.  Checked
@@ -738,7 +886,6 @@ def bench_layered(runtime, sizes, prompts=(512, 2048, 8192), context=2000):
     decoded token's logits against those of the same token at the end of a prompt."""
     from llmopt_amd.decode_step import DecodeConfig, DecodeStep, random_w4
     from llmopt_amd.layered_model import LayeredConfig, LayeredModel
-    from llmopt_amd.native import DispatchList
     from llmopt_amd.prefill_step import PrefillStep
     rng = np.random.default_rng(SEED + 11)
     median = lambda values: sorted(values)[len(values) // 2]
@@ -764,15 +911,7 @@ def bench_layered(runtime, sizes, prompts=(512, 2048, 8192), context=2000):
         device_weights = None
         for m in prompts:
             tokens = rng.integers(0, LAYERED_VOCABULARY, m)
-            sequence = model.open()
-            logits = model.step(sequence, tokens, [m - 1])
-            model.close(sequence)
-            graph = runtime.begin_batch()
-            graph.dispatch_all(model._lists[m])
-            index = runtime.buffer_of_bytes(np.array([m - 1], np.uint32))
-            out = runtime.create_buffer(LAYERED_VOCABULARY * 4)
-            graph.dispatch_all(DispatchList([model._logits(1, m, model._work, index, out)]))
-            ms = median(graph.commit_profiled_each(repeats=5))
+            ms, finite = time_prompt(runtime, model, tokens)
             flops, _ = layered_work(model, m, context)
             pool = runtime.create_buffer((m + 1) * other.token_stride)
             step = PrefillStep(runtime, other, weights, m, pool, runtime.buffer_of_bytes(np.arange(m + 1, dtype=np.uint32)),
@@ -783,31 +922,16 @@ def bench_layered(runtime, sizes, prompts=(512, 2048, 8192), context=2000):
             step.record(graph)
             other_ms = median(graph.commit_profiled_each(repeats=5))
             entry["prefill"].append({
-                "tokens": m, "ms": round(ms, 4), "tokens_per_s": round(m / ms * 1e3), "finite": bool(np.isfinite(logits).all()),
+                "tokens": m, "ms": round(ms, 4), "tokens_per_s": round(m / ms * 1e3), "finite": finite,
                 "TFLOPs": round(flops / ms / 1e9, 1), "mfma_frac": round(flops / ms / 1e9 / MFMA_F16_PEAK_TFLOPS, 4),
                 "w4a16": {"ms": round(other_ms, 4), "tokens_per_s": round(m / other_ms * 1e3),
                           "TFLOPs": round(step.flops() / other_ms / 1e9, 1),
                           "mfma_frac": round(step.flops() / other_ms / 1e9 / MFMA_F16_PEAK_TFLOPS, 4)}})
             del step, pool
         tokens = rng.integers(0, LAYERED_VOCABULARY, context).tolist() + [1]
-        sequence = model.open()
-        at_once = model.step(sequence, tokens, [context]).astype(np.float64)
-        model.close(sequence)
-        sequence = model.open()
-        model.step(sequence, tokens[:context])
-        plan = model.decode_plan()
-        plan.execute(1, sequence)  # leaves the step words of a token behind the context
-        difference = float(np.linalg.norm(model.logits_row() - at_once[0]) / np.linalg.norm(at_once))
+        ms, wall, difference, records = time_token(runtime, model, tokens)
         entry["verified"] = bool(restated <= 2e-2 and difference <= 0.1)
         entry["rel_l2_restatement"], entry["rel_l2_decode_against_prompt"] = (float("%.3g" % v) for v in (restated, difference))
-        graph = runtime.begin_batch()
-        graph.dispatch_all(DispatchList(plan.dispatches))
-        ms = median(graph.commit_profiled_each(repeats=9))
-        started = time.perf_counter()
-        for _ in range(20):
-            plan.execute(1, sequence)
-        wall = (time.perf_counter() - started) / 20 * 1e3
-        model.close(sequence)
         _, step_bytes = layered_work(model, 1, context)
         slots = np.arange(context + 64, dtype=np.uint32)
         step = DecodeStep(runtime, other, weights, 1, runtime.create_buffer(len(slots) * other.token_stride),
@@ -820,12 +944,12 @@ def bench_layered(runtime, sizes, prompts=(512, 2048, 8192), context=2000):
         entry["decode"] = {
             "context": context, "ms": round(ms, 4), "tokens_per_s": round(1e3 / ms, 1), "plan_wall_ms": round(wall, 4),
             "bytes": int(step_bytes), "GBps": round(step_bytes / ms / 1e6, 1),
-            "hbm_frac": round(step_bytes / ms / 1e6 / HBM_PEAK_GBS, 4), "records": len(plan.dispatches),
+            "hbm_frac": round(step_bytes / ms / 1e6 / HBM_PEAK_GBS, 4), "records": records,
             "w4a16": {"ms": round(other_ms, 4), "tokens_per_s": round(1e3 / other_ms, 1), "bytes": int(other_bytes),
                       "GBps": round(other_bytes / other_ms / 1e6, 1),
                       "hbm_frac": round(other_bytes / other_ms / 1e6 / HBM_PEAK_GBS, 4), "records": len(step.dispatches)}}
         results.append(entry)
-        del model, step, plan, graph, device_weights
+        del model, step, graph, device_weights
     return results
 
 
@@ -984,7 +1108,10 @@ def main():
     parser.add_argument("--layered", nargs="?", const=",".join(LAYERED_SIZES), metavar="SIZES",
                         help="only the layered decoders beside the W4A16 transformer, at these widths (default: "
                              + ",".join(LAYERED_SIZES) + ")")
-    parser.add_argument("--layered-prompts", default="512,2048,8192", help="prompt lengths of --layered")
+    parser.add_argument("--parallel", nargs="?", const=",".join(PARALLEL_SIZES), metavar="SIZES",
+                        help="only the Koketar design beside a Barovik decoder of the same parts, at these widths (default: "
+                             + ",".join(PARALLEL_SIZES) + ")")
+    parser.add_argument("--layered-prompts", default="512,2048,8192", help="prompt lengths of --layered and --parallel")
     parser.add_argument("--pmc-probe", action="store_true",
                         help="only the calibration copies and the cases of the GEMV sweep, for rocprofv3 --pmc")
     args = parser.parse_args()
@@ -997,12 +1124,14 @@ def main():
         print(json.dumps(pmc_probe(runtime)))
         runtime.close()
         return
-    if args.layered:
-        layered = bench_layered(runtime, args.layered.split(","), tuple(int(m) for m in args.layered_prompts.split(",")))
+    if args.layered or args.parallel:
+        prompts = tuple(int(m) for m in args.layered_prompts.split(","))
+        run, sizes, key = (bench_layered, args.layered, "layered") if args.layered else (bench_parallel, args.parallel, "parallel")
+        entries = run(runtime, sizes.split(","), prompts)
         runtime.close()
-        if not all(entry["verified"] for entry in layered):
-            sys.exit("bench.py: outputs of timed cases differ beyond tolerance: %s" % layered)
-        print(json.dumps({"layered": layered}))
+        if not all(entry["verified"] for entry in entries):
+            sys.exit("bench.py: outputs of timed cases differ beyond tolerance: %s" % entries)
+        print(json.dumps({key: entries}))
         return
     gemv = bench_gemv(runtime, args.steps, args.warmup, serial_only=args.serial_only)
     # the sweep's time by kernel; `roofline` is the kernel with the largest share

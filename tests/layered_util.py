@@ -36,10 +36,10 @@ def config(*layers, vocab=90, width=72, eps=1e-5, scale=1.5):
             "embedding": {"scale": scale}, "layers": list(layers)}
 
 
-def make_weights(cfg, seed=0, change=None):
+def make_weights(cfg, seed=0, change=None, **options):
     """(bfloat16 patterns, the same as float arrays); change(name, values) may replace a tensor's values."""
     parsed = LayeredConfig.parse(cfg)
-    patterns = parsed.random_tensors(np.random.default_rng(seed))
+    patterns = parsed.random_tensors(np.random.default_rng(seed), **options)
     if change is not None:
         for name, array in patterns.items():
             new = change(name, from_bfloat16(array))
