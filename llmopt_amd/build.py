@@ -41,6 +41,7 @@ PER_FILE = {
     "dense_attention.hip": ["-mllvm", "-amdgpu-mfma-vgpr-form=1"],
     "q8_attention.hip": ["-mllvm", "-amdgpu-mfma-vgpr-form=1"],
     "chunk_attention.hip": ["-mllvm", "-amdgpu-mfma-vgpr-form=1"],
+    "delta.hip": ["-mllvm", "-amdgpu-mfma-vgpr-form=1"],
 }
 
 

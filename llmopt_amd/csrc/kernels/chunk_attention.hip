@@ -323,6 +323,14 @@ constexpr int decode_lds_floats() {
   return 4 * 32 * value_stride<T, NE>() * (int)sizeof(T) / 4 + 2 * 4 * 16;
 }
 
+// Cosine and sine of every rotated pair at one position.
+struct Turn {
+  float cosine, sine;
+};
+__device__ __forceinline__ void fill_turns(const HeadRotation &r, uint32_t position, Turn *turns) {
+  for (uint32_t c = threadIdx.x; c < r.dims / 2; c += 256) turn(position, r.frequencies[c], turns[c].cosine, turns[c].sine);
+}
+
 // Norm and rotation of head vectors, a wave a vector, lane l holding components l + 64 i.
 template <int PARTS>
 struct HeadVector {
@@ -330,7 +338,7 @@ struct HeadVector {
   // exchange(v, partner, half): every rotated component's partner, c + half or c - half.
   template <typename Exchange>
   __device__ __forceinline__ void norm_and_rotate(const HeadRotation &r, const uint16_t *norm, uint32_t dim,
-                                                  uint32_t position, int lane, Exchange exchange) {
+                                                  const Turn *turns, int lane, Exchange exchange) {
     float sum = 0.0f;
 #pragma unroll
     for (int i = 0; i < PARTS; ++i) sum += v[i] * v[i];
@@ -347,9 +355,8 @@ struct HeadVector {
     for (int i = 0; i < PARTS; ++i) {
       const uint32_t c = lane + 64 * i;
       if (c >= r.dims) continue;
-      float cosine, sine;
-      turn(position, r.frequencies[c < half ? c : c - half], cosine, sine);
-      v[i] = c < half ? v[i] * cosine - partner[i] * sine : v[i] * cosine + partner[i] * sine;
+      const Turn t = turns[c < half ? c : c - half];
+      v[i] = c < half ? v[i] * t.cosine - partner[i] * t.sine : v[i] * t.cosine + partner[i] * t.sine;
     }
   }
 };
@@ -375,29 +382,43 @@ struct ThroughLds {
   }
 };
 
-// Vectors 0 .. heads + kv_heads - 1 of every row: the queries, then the keys.
+// A workgroup a row; its waves take vectors 0 .. heads + kv_heads - 1 (the queries, then the keys) in turn, the next one
+// requested ahead.
 template <typename T, int PARTS>
 __global__ __launch_bounds__(256) void rotate_heads_kernel(ChunkAttentionArgs a) {
   __shared__ float rows[4][PARTS * 64];
+  __shared__ Turn turns[PARTS * 32];
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
-  const uint32_t vector = blockIdx.y * 4 + wave, r = blockIdx.x;
-  if (vector >= a.heads + a.kv_heads) return;
-  T *head = const_cast<T *>(static_cast<const T *>(a.qkv)) + (size_t)r * a.ld + (size_t)vector * a.dim;
-  HeadVector<PARTS> h;
+  const uint32_t r = blockIdx.x, vectors = a.heads + a.kv_heads;
+  T *row = const_cast<T *>(static_cast<const T *>(a.qkv)) + (size_t)r * a.ld;
+  T ahead[PARTS];
+  auto request = [&](uint32_t vector) {
 #pragma unroll
-  for (int i = 0; i < PARTS; ++i) h.v[i] = lane + 64 * i < a.dim ? to_f32(head[lane + 64 * i]) : 0.0f;
-  h.norm_and_rotate(a.rotation, vector < a.heads ? a.rotation.q_norm : a.rotation.k_norm, a.dim,
-                    a.state[kStatePosition] + r, lane, ThroughLds<PARTS>{rows[wave], a.rotation.dims, lane});
+    for (int i = 0; i < PARTS; ++i)
+      if (lane + 64 * i < a.dim) ahead[i] = row[(size_t)vector * a.dim + lane + 64 * i];
+  };
+  request(min((uint32_t)wave, vectors - 1));
+  fill_turns(a.rotation, a.state[kStatePosition] + r, turns);
+  __syncthreads();
+  for (uint32_t vector = wave; vector < vectors; vector += 4) {
+    HeadVector<PARTS> h;
 #pragma unroll
-  for (int i = 0; i < PARTS; ++i)
-    if (lane + 64 * i < a.dim) head[lane + 64 * i] = (T)h.v[i];
+    for (int i = 0; i < PARTS; ++i) h.v[i] = lane + 64 * i < a.dim ? to_f32(ahead[i]) : 0.0f;
+    request(min(vector + 4, vectors - 1));
+    h.norm_and_rotate(a.rotation, vector < a.heads ? a.rotation.q_norm : a.rotation.k_norm, a.dim, turns, lane,
+                      ThroughLds<PARTS>{rows[wave], a.rotation.dims, lane});
+#pragma unroll
+    for (int i = 0; i < PARTS; ++i)
+      if (lane + 64 * i < a.dim) row[(size_t)vector * a.dim + lane + 64 * i] = (T)h.v[i];
+  }
 }
 
 // LDS of a decode workgroup that starts from a raw row: queries [16][ND * 32 + pad], the own key, the own
-// value, a float row for every wave.
+// value, a float row for every wave, the position's turns.
 template <typename T, int ND, int NE>
 constexpr int raw_row_lds_bytes() {
-  return (17 * (ND * 32 + 16 / (int)sizeof(T)) + NE * 16) * (int)sizeof(T) + 4 * (ND <= 2 ? 64 : ND * 32) * 4;
+  return (17 * (ND * 32 + 16 / (int)sizeof(T)) + NE * 16) * (int)sizeof(T) + 4 * (ND <= 2 ? 64 : ND * 32) * 4 +
+         ND * 16 * (int)sizeof(Turn);
 }
 
 template <typename T, int ND, int NE, bool RAW>
@@ -441,6 +462,7 @@ __global__ __launch_bounds__(256) void chunk_decode_kernel(ChunkAttentionArgs a,
   constexpr int SQ = ND * 32 + 16 / (int)sizeof(T), PARTS = ND <= 2 ? 1 : ND / 2;
   T *lds_q = reinterpret_cast<T *>(lds + decode_lds_floats<T, NE>() * 4), *own_k = lds_q + 16 * SQ, *own_v = own_k + SQ;
   float *exchange = reinterpret_cast<float *>(own_v + EP) + wave * PARTS * 64;
+  Turn *turns = reinterpret_cast<Turn *>(reinterpret_cast<float *>(own_v + EP) + 4 * PARTS * 64);
   auto stage_vectors = [&](uint32_t h0, uint32_t count, bool key) {
     for (uint32_t n = wave; n < count + (key ? 1 : 0); n += 4) {
       const bool query = n < count;
@@ -448,7 +470,7 @@ __global__ __launch_bounds__(256) void chunk_decode_kernel(ChunkAttentionArgs a,
       HeadVector<PARTS> h;
 #pragma unroll
       for (int i = 0; i < PARTS; ++i) h.v[i] = lane + 64 * i < a.dim ? source[lane + 64 * i] : 0.0f;
-      h.norm_and_rotate(a.rotation, query ? a.rotation.q_norm : a.rotation.k_norm, a.dim, position, lane,
+      h.norm_and_rotate(a.rotation, query ? a.rotation.q_norm : a.rotation.k_norm, a.dim, turns, lane,
                         ThroughLds<PARTS>{exchange, a.rotation.dims, lane});
       T *target = query ? lds_q + n * SQ : own_k;
 #pragma unroll
@@ -457,6 +479,8 @@ __global__ __launch_bounds__(256) void chunk_decode_kernel(ChunkAttentionArgs a,
     }
   };
   if (RAW) {
+    fill_turns(a.rotation, position, turns);
+    __syncthreads();
     stage_vectors(0, min(16u, per), true);
     const float *value = a.row + (size_t)(a.heads + a.kv_heads) * a.dim + (size_t)group * a.vdim;
     for (uint32_t c = tid; c < EP; c += 256) own_v[c] = (T)(c < a.vdim ? value[c] : 0.0f);
@@ -696,7 +720,7 @@ hipError_t launch_chunk_attention(const ChunkAttentionArgs &a, hipStream_t strea
 }
 
 hipError_t launch_rotate_heads(const ChunkAttentionArgs &a, hipStream_t stream) {
-  const dim3 grid(a.m, (a.heads + a.kv_heads + 3) / 4);
+  const dim3 grid(a.m);
   const int parts = a.dim <= 64 ? 1 : a.dim <= 128 ? 2 : 4;
   auto run = [&](auto kernel) {
     kernel<<<grid, 256, 0, stream>>>(a);

@@ -120,6 +120,13 @@ __device__ __forceinline__ float tanh_f32(float z) {
 }
 __device__ __forceinline__ float softplus_f32(float z) { return z > 20.0f ? z : log1pf(expf(z)); }
 
+// log(1 + e^z) from the hardware's exponential and logarithm: log(u) e / (u - 1) with u = 1 + e rounded takes the
+// rounding of u back out.
+__device__ __forceinline__ float softplus_fast_f32(float z) {
+  const float e = __expf(-fabsf(z)), u = 1.0f + e;
+  return fmaxf(z, 0.0f) + (u == 1.0f ? e : __logf(u) * e * __builtin_amdgcn_rcpf(u - 1.0f));
+}
+
 // Activation of a gated feed-forward.
 enum GateActivation : uint32_t { kGateSilu = 0, kGateGeluTanh = 1, kGateClamped = 2 };
 __device__ __forceinline__ float gate_activation(float z, uint32_t kind) {
@@ -145,9 +152,18 @@ __device__ __forceinline__ void turn(uint32_t position, double frequency, float 
 }
 
 // Sum over the 64 lanes of a wave, in every lane.
+template <int CONTROL>
+__device__ __forceinline__ float dpp_f32(float v) {
+  return __builtin_bit_cast(float, __builtin_amdgcn_mov_dpp(__builtin_bit_cast(int, v), CONTROL, 0xf, 0xf, true));
+}
 __device__ __forceinline__ float wave_sum(float v) {
-#pragma unroll
-  for (int mask = 32; mask >= 1; mask >>= 1) v += __shfl_xor(v, mask, 64);
+  // within rows of sixteen lanes: neighbours, pairs, halves, the row
+  v += dpp_f32<0xb1>(v);   // quad_perm [1, 0, 3, 2]
+  v += dpp_f32<0x4e>(v);   // quad_perm [2, 3, 0, 1]
+  v += dpp_f32<0x141>(v);  // row_half_mirror
+  v += dpp_f32<0x140>(v);  // row_mirror
+  v += __shfl_xor(v, 16, 64);
+  v += __shfl_xor(v, 32, 64);
   return v;
 }
 __device__ __forceinline__ float wave_max(float v) {
