@@ -145,44 +145,64 @@ __device__ __forceinline__ void stage_pending_any(const DenseGemvArgs &a, float 
   __syncthreads();
 }
 
-// Stages the f32 row x, normalised in `groups` parts by norm_weight when that is not null.  `ahead` is
-// called once the row has been requested (loads return in order: what it requests does not delay the row).
-template <typename T, typename Ahead>
+// How a launch stages its row.  One kernel each: a kernel's registers are those of its largest branch, and they decide
+// how many loads a CU keeps in flight.
+enum class Staging {
+  kPlainShort,    // rows of whole pieces of eight, at most 8192 values
+  kPlain,
+  kNormedShort,   // one norm over a row of whole pieces of four, at most 4096 values
+  kNormed,
+  kPendingShort,  // the same with a pending output
+  kPending,
+};
+
+inline Staging staging_of(const DenseGemvArgs &a) {
+  if (a.pending) return a.k % 4 == 0 && a.k <= 4096 ? Staging::kPendingShort : Staging::kPending;
+  if (a.norm_weight) return a.k % 4 == 0 && a.k <= 4096 && a.norm_groups == 1 ? Staging::kNormedShort : Staging::kNormed;
+  return a.k % 8 == 0 && a.k <= 8192 ? Staging::kPlainShort : Staging::kPlain;
+}
+
+template <typename T, int PIECES, typename Ahead>
+__device__ __forceinline__ void stage_plain_row(const DenseGemvArgs &a, float *xs, uint32_t plane, Ahead ahead) {
+  const uint32_t k = a.k;
+  f32x8 v[PIECES];
+#pragma unroll
+  for (int q = 0; q < PIECES; ++q) {
+    const uint32_t i = (q * kWaves * 64 + threadIdx.x) * 8;
+    if (i < k)
+      v[q] = a.x_is_f32 ? *reinterpret_cast<const f32x8 *>(static_cast<const float *>(a.x) + i)
+                        : convert_frag<float>(*reinterpret_cast<const Frag<T> *>(static_cast<const T *>(a.x) + i));
+  }
+  ahead();
+#pragma unroll
+  for (int q = 0; q < PIECES; ++q) {
+    const uint32_t i = (q * kWaves * 64 + threadIdx.x) * 8;
+    if (i < k) {
+      *reinterpret_cast<f32x4 *>(xs + (i >> 1)) = f32x4{v[q][0], v[q][1], v[q][2], v[q][3]};
+      *reinterpret_cast<f32x4 *>(xs + plane + (i >> 1)) = f32x4{v[q][4], v[q][5], v[q][6], v[q][7]};
+    }
+  }
+  __syncthreads();
+}
+
+// Stages the row x (f32, or the activation type where it is plain), normalised in `groups` parts by norm_weight.  `ahead`
+// is called once the row has been requested (loads return in order: what it requests does not delay the row).
+template <typename T, Staging STAGING, typename Ahead>
 __device__ __forceinline__ void stage_activation(const DenseGemvArgs &a, float *xs, uint32_t plane, float *scratch,
                                                  Ahead ahead) {
   const uint32_t k = a.k;
-  const __bf16 *weight = reinterpret_cast<const __bf16 *>(a.norm_weight);
   // whole pieces behind the row's end read as zeros
   for (uint32_t i = k + threadIdx.x; i < ((k + 7) & ~7u); i += kWaves * 64) xs[staged_index(i, plane)] = 0.0f;
-  if (a.pending) {
-    if ((k & 3) == 0 && k <= 2 * 4 * kWaves * 64) return stage_pending_row<2>(a, xs, plane, scratch, ahead);
-    if ((k & 3) == 0 && k <= 4 * 4 * kWaves * 64) return stage_pending_row<4>(a, xs, plane, scratch, ahead);
+  if (STAGING == Staging::kPlainShort) return stage_plain_row<T, 4>(a, xs, plane, ahead);
+  if (STAGING == Staging::kNormedShort) return stage_normed_row<4>(a, xs, plane, scratch, ahead);
+  if (STAGING == Staging::kPendingShort) return stage_pending_row<4>(a, xs, plane, scratch, ahead);
+  if (STAGING == Staging::kPending) {
     if ((k & 3) == 0 && k <= 8 * 4 * kWaves * 64) return stage_pending_row<8>(a, xs, plane, scratch, ahead);
     ahead();
     return stage_pending_any(a, xs, plane, scratch);
   }
-  if (weight == nullptr) {
-    if ((k & 7) == 0 && k <= 8 * 8 * kWaves * 64) {
-      f32x8 v[8];
-#pragma unroll
-      for (int q = 0; q < 8; ++q) {
-        const uint32_t i = (q * kWaves * 64 + threadIdx.x) * 8;
-        if (i < k)
-          v[q] = a.x_is_f32 ? *reinterpret_cast<const f32x8 *>(static_cast<const float *>(a.x) + i)
-                            : convert_frag<float>(*reinterpret_cast<const Frag<T> *>(static_cast<const T *>(a.x) + i));
-      }
-      ahead();
-#pragma unroll
-      for (int q = 0; q < 8; ++q) {
-        const uint32_t i = (q * kWaves * 64 + threadIdx.x) * 8;
-        if (i < k) {
-          *reinterpret_cast<f32x4 *>(xs + (i >> 1)) = f32x4{v[q][0], v[q][1], v[q][2], v[q][3]};
-          *reinterpret_cast<f32x4 *>(xs + plane + (i >> 1)) = f32x4{v[q][4], v[q][5], v[q][6], v[q][7]};
-        }
-      }
-      __syncthreads();
-      return;
-    }
+  if (STAGING == Staging::kPlain) {
+    if ((k & 7) == 0 && k <= 8 * 8 * kWaves * 64) return stage_plain_row<T, 8>(a, xs, plane, ahead);
     ahead();
     for (uint32_t i = threadIdx.x; i < k; i += kWaves * 64)
       xs[staged_index(i, plane)] =
@@ -190,17 +210,12 @@ __device__ __forceinline__ void stage_activation(const DenseGemvArgs &a, float *
     __syncthreads();
     return;
   }
-  const float *x = static_cast<const float *>(a.x);
-  const uint32_t part = k / a.norm_groups;
-  if (a.norm_groups == 1 && (k & 3) == 0 && k <= 4 * 4 * kWaves * 64) {
-    stage_normed_row<4>(a, xs, plane, scratch, ahead);
-    return;
-  }
-  if (a.norm_groups == 1 && (k & 3) == 0 && k <= 8 * 4 * kWaves * 64) {
-    stage_normed_row<8>(a, xs, plane, scratch, ahead);
-    return;
-  }
+  if (a.norm_groups == 1 && (k & 3) == 0 && k <= 8 * 4 * kWaves * 64)
+    return stage_normed_row<8>(a, xs, plane, scratch, ahead);
   ahead();
+  const float *x = static_cast<const float *>(a.x);
+  const __bf16 *weight = reinterpret_cast<const __bf16 *>(a.norm_weight);
+  const uint32_t part = k / a.norm_groups;
   for (uint32_t g = 0; g < a.norm_groups; ++g) {
     float sum = 0.0f;
     for (uint32_t i = g * part + threadIdx.x; i < (g + 1) * part; i += kWaves * 64) sum += x[i] * x[i];
@@ -317,7 +332,7 @@ __device__ __forceinline__ void gemv_epilogue(const DenseGemvArgs &a, uint32_t n
   }
 }
 
-template <typename T, int ROWS, bool GATED, bool VEC>
+template <typename T, int ROWS, bool GATED, bool VEC, Staging STAGING>
 __global__ __launch_bounds__(256) void dense_gemv_kernel(DenseGemvArgs a) {
   extern __shared__ __attribute__((aligned(16))) float xs[];
   __shared__ float scratch[kWaves];
@@ -332,7 +347,7 @@ __global__ __launch_bounds__(256) void dense_gemv_kernel(DenseGemvArgs a) {
     const uint32_t n = min(first + (GATED ? r / 2 : r), a.n - 1);
     stream.rows[r] = reinterpret_cast<const __bf16 *>(matrix) + (size_t)n * a.k;
   }
-  stage_activation<T>(a, xs, plane, scratch, [&] { stream.request(a.k, lane); });
+  stage_activation<T, STAGING>(a, xs, plane, scratch, [&] { stream.request(a.k, lane); });
   if (first >= a.n) return;
   stream.run(xs, plane, a.k, lane);
   const float(&sums)[ROWS] = stream.sums;
@@ -346,16 +361,29 @@ __global__ __launch_bounds__(256) void dense_gemv_kernel(DenseGemvArgs a) {
   if (lane < OUTPUTS && first + lane < a.n) gemv_epilogue<T>(a, first + lane, mine, up);
 }
 
-template <typename T, int ROWS, bool GATED, bool VEC>
-hipError_t run_gemv(const DenseGemvArgs &a, hipStream_t stream) {
+template <typename T, int ROWS, bool GATED, bool VEC, Staging STAGING>
+hipError_t run_staged(const DenseGemvArgs &a, hipStream_t stream) {
   static bool allowed[kMaxDevices] = {};
-  const void *kernel = reinterpret_cast<const void *>(dense_gemv_kernel<T, ROWS, GATED, VEC>);
+  const auto kernel = dense_gemv_kernel<T, ROWS, GATED, VEC, STAGING>;
   const uint32_t bytes = ((a.k + 7) / 8) * 32;
   if (bytes > 48 * 1024)
-    if (hipError_t status = allow_dynamic_lds(kernel, kGemvMaxK * 4, allowed)) return status;
+    if (hipError_t status = allow_dynamic_lds(reinterpret_cast<const void *>(kernel), kGemvMaxK * 4, allowed)) return status;
   const uint32_t per = kWaves * (GATED ? ROWS / 2 : ROWS);
-  dense_gemv_kernel<T, ROWS, GATED, VEC><<<(a.n + per - 1) / per, 256, bytes, stream>>>(a);
+  kernel<<<(a.n + per - 1) / per, 256, bytes, stream>>>(a);
   return hipGetLastError();
+}
+
+template <typename T, int ROWS, bool GATED, bool VEC>
+hipError_t run_gemv(const DenseGemvArgs &a, hipStream_t stream) {
+  switch (staging_of(a)) {
+    case Staging::kPlainShort: return run_staged<T, ROWS, GATED, VEC, Staging::kPlainShort>(a, stream);
+    case Staging::kPlain: return run_staged<T, ROWS, GATED, VEC, Staging::kPlain>(a, stream);
+    case Staging::kNormedShort: return run_staged<T, ROWS, GATED, VEC, Staging::kNormedShort>(a, stream);
+    case Staging::kNormed: return run_staged<T, ROWS, GATED, VEC, Staging::kNormed>(a, stream);
+    case Staging::kPendingShort: return run_staged<T, ROWS, GATED, VEC, Staging::kPendingShort>(a, stream);
+    case Staging::kPending: return run_staged<T, ROWS, GATED, VEC, Staging::kPending>(a, stream);
+  }
+  return hipErrorInvalidValue;
 }
 
 template <typename T>
@@ -406,7 +434,7 @@ __device__ __forceinline__ void select_experts(const float *logits, uint32_t exp
 // blockIdx.y: choice 0 .. top - 1, or `top`: the shared expert.  A wave owns kUpOutputs hidden values.
 constexpr int kUpOutputs = 4, kUpSteps = 2;
 
-template <typename T, bool VEC>
+template <bool VEC, Staging STAGING>
 __global__ __launch_bounds__(256) void moe_gemv_up_kernel(MoeGemvArgs a) {
   extern __shared__ __attribute__((aligned(16))) float lds[];
   __shared__ float scratch[kWaves];
@@ -426,7 +454,7 @@ __global__ __launch_bounds__(256) void moe_gemv_up_kernel(MoeGemvArgs a) {
   const uint32_t first = (blockIdx.x * kWaves + wave) * kUpOutputs;
   RowStream<2 * kUpOutputs, VEC, kUpSteps> stream;
   // the choice is made, and its weights are requested, while the activation is on its way to LDS
-  stage_activation<T>(in, xs, plane, scratch, [&] {
+  stage_activation<float, STAGING>(in, xs, plane, scratch, [&] {
     uint32_t expert = 0;
     if (!shared) {
       select_experts<256>(a.logits, a.experts, a.top, z, ids, weights);
@@ -525,8 +553,10 @@ hipError_t launch_moe_gemv_up(const MoeGemvArgs &a, hipStream_t stream) {
   if (bytes > 60 * 1024) return hipErrorInvalidValue;
   const uint32_t widest = std::max(a.ff, a.shared_ff);
   const dim3 grid((widest + kUpOutputs * kWaves - 1) / (kUpOutputs * kWaves), a.top + (a.shared_ff ? 1 : 0));
-  if (a.width % 8 == 0) moe_gemv_up_kernel<float, true><<<grid, 256, bytes, stream>>>(a);
-  else moe_gemv_up_kernel<float, false><<<grid, 256, bytes, stream>>>(a);
+  const bool small = a.width % 4 == 0 && a.width <= 4096;
+  if (a.width % 8 != 0) moe_gemv_up_kernel<false, Staging::kNormed><<<grid, 256, bytes, stream>>>(a);
+  else if (small) moe_gemv_up_kernel<true, Staging::kNormedShort><<<grid, 256, bytes, stream>>>(a);
+  else moe_gemv_up_kernel<true, Staging::kNormed><<<grid, 256, bytes, stream>>>(a);
   return hipGetLastError();
 }
 
