@@ -15,7 +15,7 @@ constexpr uint32_t kStatePosition = 0, kStateSlot = 1, kStateWords = 2;
 
 enum class DenseEpilogue : uint32_t {
   kStore = 0,     // out[r, c] (activation type)
-  kStoreF32 = 1,  // out_f32[r, c] (softcap > 0: softcap tanh(result / softcap))
+  kStoreF32 = 1,  // out_f32[r, c]
   kAdd = 2,       // stream[r, c] += result * (row_gate ? sigmoid(row_gate[r * row_gate_stride]) : 1)
   kGated = 3,     // out[r, c] = act(gate) * up
   kQkv = 4,       // kStore, with the value columns mixed with another layer's values
@@ -40,7 +40,6 @@ struct DenseLinearArgs {
   DenseEpilogue epilogue;
   uint32_t activation;
   float limit;           // kGated, clamped activation
-  float softcap;         // kStoreF32; 0: none
   void *out;
   float *out_f32;        // kStoreF32, kSplit, and the stream of kAdd
   uint32_t ld_out, ld_f32;
@@ -87,6 +86,9 @@ struct NormAddArgs {
 };
 hipError_t launch_norm_add(const NormAddArgs &args, hipStream_t stream);
 
+// values <- cap tanh(values / cap), in place.  (In the products' epilogue it would cost every large tile registers.)
+hipError_t launch_soft_cap(float *values, uint64_t count, float cap, hipStream_t stream);
+
 struct DenseEmbeddingArgs {
   const int64_t *tokens;
   const uint16_t *embed;  // bf16 [vocabulary, width]
@@ -129,7 +131,8 @@ struct DenseGemvArgs {
   uint32_t n, k;
   GemvEpilogue epilogue;
   uint32_t activation;
-  float limit, softcap;
+  float limit;
+  float softcap;  // kStoreF32: softcap tanh(result / softcap); 0: none
   void *out;
   float *out_f32;
   // kQkv

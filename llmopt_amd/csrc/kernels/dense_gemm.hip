@@ -76,10 +76,6 @@ __device__ __forceinline__ void emit(const DenseLinearArgs &a, uint32_t r, uint3
       store4(static_cast<T *>(a.out) + (size_t)r * a.ld_out + c, v, count, (a.ld_out & 3) == 0);
       return;
     case DenseEpilogue::kStoreF32:
-      if (a.softcap > 0.0f) {
-#pragma unroll
-        for (int i = 0; i < 4; ++i) v[i] = soft_capped(v[i], a.softcap);
-      }
       store4(a.out_f32 + (size_t)r * a.ld_f32 + c, v, count, (a.ld_f32 & 3) == 0);
       return;
     case DenseEpilogue::kAdd: {
@@ -142,8 +138,17 @@ __device__ __forceinline__ bool place_tile(const GemmParams &p, TilePlace &t) {
   return true;
 }
 
+// GATED of the kernels: 0 no, 1 an activation of the gate alone, 2 the clamped pair.  (Apart: the epilogue's code is
+// repeated for every value of a tile, and an activation more costs the large tiles a few percent.)
+constexpr int kOneSided = 1, kClampedPair = 2;
+template <int GATED>
+__device__ __forceinline__ float gated(const DenseLinearArgs &a, float gate, float up) {
+  if (GATED == kClampedPair) return gated_value(gate, up, kGateClamped, a.limit);
+  return gate_activation(gate, a.activation) * up;
+}
+
 // A wave's accumulators: MT x NT groups of 16 x 16 from row `row_offset` and tile column `column_offset` on.
-template <typename T, int MT, int NT, bool GATED>
+template <typename T, int MT, int NT, int GATED>
 __device__ __forceinline__ void emit_tile(const DenseLinearArgs &a, const f32x4 (&acc)[MT][NT], uint32_t m_first,
                                           uint32_t m_rows, uint32_t n_first, uint32_t row_offset,
                                           uint32_t column_offset, int lane) {
@@ -160,7 +165,7 @@ __device__ __forceinline__ void emit_tile(const DenseLinearArgs &a, const f32x4 
         if (c >= a.n) continue;
         f32x4 v;
 #pragma unroll
-        for (int e = 0; e < 4; ++e) v[e] = gated_value(acc[i][j][e], acc[i][j + 1][e], a.activation, a.limit);
+        for (int e = 0; e < 4; ++e) v[e] = gated<GATED>(a, acc[i][j][e], acc[i][j + 1][e]);
         emit<T>(a, r, c, v);
       }
     } else {
@@ -176,7 +181,7 @@ __device__ __forceinline__ void emit_tile(const DenseLinearArgs &a, const f32x4 
 // WM x WN waves; a wave owns (BM / WM) x (BN / WN).  Two LDS stages: the next one travels global -> registers
 // while this one is multiplied, one barrier a stage; LDS rows carry 16 bytes of padding, so that the sixteen
 // rows an operand read touches start in different banks.
-template <typename T, int BM, int BN, int WM, bool GATED, bool ROUTED, bool VEC, int WAVES = 4>
+template <typename T, int BM, int BN, int WM, int GATED, bool ROUTED, bool VEC, int WAVES = 4>
 __global__ __launch_bounds__(WAVES * 64) void dense_gemm_kernel(GemmParams p) {
   constexpr int WN = WAVES / WM, PASS = WAVES * 8;
   constexpr int MT = BM / WM / 16, NT = BN / WN / 16;
@@ -291,7 +296,7 @@ GemmParams gemm_params(const DenseLinearArgs &a, dim3 *grid) {
   return p;
 }
 
-template <typename T, int BM, int BN, int WM, bool GATED, bool ROUTED, bool VEC, int WAVES = 4>
+template <typename T, int BM, int BN, int WM, int GATED, bool ROUTED, bool VEC, int WAVES = 4>
 hipError_t run_gemm(const DenseLinearArgs &a, hipStream_t stream) {
   constexpr int bytes = gemm_lds_bytes<T, BM, BN>();
   static bool allowed[kMaxDevices] = {};
@@ -306,7 +311,7 @@ hipError_t run_gemm(const DenseLinearArgs &a, hipStream_t stream) {
 }
 
 // The bf16 outputs of a wave, 16 rows at a time through its own LDS rows, so that a store covers whole lines.
-template <int MT, int NT, bool GATED>
+template <int MT, int NT, int GATED>
 __device__ __forceinline__ void emit_rows(const DenseLinearArgs &a, const f32x4 (&acc)[MT][NT], uint32_t m_first,
                                           uint32_t m_rows, uint32_t n_first, uint32_t row_offset,
                                           uint32_t column_offset, int lane, __bf16 *rows) {
@@ -323,7 +328,7 @@ __device__ __forceinline__ void emit_rows(const DenseLinearArgs &a, const f32x4 
       f32x4 v;
       if (GATED) {
 #pragma unroll
-        for (int e = 0; e < 4; ++e) v[e] = gated_value(acc[i][2 * j][e], acc[i][2 * j + 1][e], a.activation, a.limit);
+        for (int e = 0; e < 4; ++e) v[e] = gated<GATED>(a, acc[i][2 * j][e], acc[i][2 * j + 1][e]);
       } else {
         v = acc[i][j];
         if (a.epilogue == DenseEpilogue::kQkv && r_in_tile < m_rows) mix_values(a, r, c, v);
@@ -369,7 +374,7 @@ __device__ __forceinline__ void copy_to_lds(const __bf16 *source, uint32_t lds_a
   asm volatile("s_mov_b32 m0, %1\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %0, off" : : "v"(source), "s"(lds_address) : "memory");
 }
 
-template <int BM, int BN, int WM, int WAVES, int STAGES, bool GATED, bool ROUTED>
+template <int BM, int BN, int WM, int WAVES, int STAGES, int GATED, bool ROUTED>
 __global__ __launch_bounds__(WAVES * 64) void dense_gemm_direct_kernel(GemmParams p) {
   constexpr int WN = WAVES / WM;
   constexpr int MT = BM / WM / 16, NT = BN / WN / 16;
@@ -462,7 +467,7 @@ __global__ __launch_bounds__(WAVES * 64) void dense_gemm_direct_kernel(GemmParam
                            stage_rows + wave * 16 * (NT * 16 + 8));
 }
 
-template <int BM, int BN, int WM, int WAVES, int STAGES, bool GATED, bool ROUTED>
+template <int BM, int BN, int WM, int WAVES, int STAGES, int GATED, bool ROUTED>
 hipError_t run_direct(const DenseLinearArgs &a, hipStream_t stream) {
   constexpr int bytes = STAGES * (BM + BN) * 128;
   static bool allowed[kMaxDevices] = {};
@@ -476,13 +481,13 @@ hipError_t run_direct(const DenseLinearArgs &a, hipStream_t stream) {
 }
 
 // Rows whose length is no multiple of the stage, and float32 rows: through registers.
-template <typename T, int BM, bool GATED, bool ROUTED>
+template <typename T, int BM, int GATED, bool ROUTED>
 hipError_t run_registers(const DenseLinearArgs &a, hipStream_t stream) {
   if (a.k % 8 == 0 && a.ldx % 8 == 0) return run_gemm<T, BM, 64, 2, GATED, ROUTED, true>(a, stream);
   return run_gemm<T, BM, 64, 2, GATED, ROUTED, false>(a, stream);
 }
 
-template <bool GATED>
+template <int GATED>
 hipError_t pick_routed(const DenseLinearArgs &a, hipStream_t stream) {
   const bool direct = !a.f32 && a.k % kStageK == 0 && a.ldx % 8 == 0;
   if (a.tile == 128) return direct ? run_direct<128, 128, 2, 4, 2, GATED, true>(a, stream) : hipErrorInvalidValue;
@@ -494,7 +499,7 @@ hipError_t pick_routed(const DenseLinearArgs &a, hipStream_t stream) {
 // 8192 x 4096 x 4096 937 / 827 with 256 x 256 / 128 x 128 tiles; 2048 x 8512 x 2048 500 / 680 / 643 with
 // 256 x 256 / 128 x 128 / 64 x 128; 2048 x 2048 x 8192 723 / 842 / 681 with 128 x 128 / 64 x 128 / 64 x 64;
 // 512 x 2048 x 4096 261 / 359 with 64 x 128 / 64 x 64; 64 x 4096 x 2048 80 / 89 with 64 x 64 / 32 x 64.
-template <bool GATED>
+template <int GATED>
 hipError_t pick_gemm(const DenseLinearArgs &a, hipStream_t stream) {
   if (a.f32) return run_registers<float, 32, GATED, false>(a, stream);
   const uint32_t columns = a.n * (GATED ? 2 : 1);
@@ -667,6 +672,11 @@ __global__ __launch_bounds__(256) void norm_add_kernel(NormAddArgs a) {
   }
 }
 
+__global__ __launch_bounds__(256) void soft_cap_kernel(float *values, uint64_t count, float cap) {
+  const uint64_t i = (uint64_t)blockIdx.x * 256 + threadIdx.x;
+  if (i < count) values[i] = soft_capped(values[i], cap);
+}
+
 __global__ __launch_bounds__(256) void dense_embedding_kernel(DenseEmbeddingArgs a) {
   const uint32_t t = blockIdx.x;
   const int64_t token = a.tokens[t];
@@ -679,9 +689,13 @@ __global__ __launch_bounds__(256) void dense_embedding_kernel(DenseEmbeddingArgs
 }  // namespace
 
 hipError_t launch_dense_gemm(const DenseLinearArgs &a, hipStream_t stream) {
-  const bool gated = a.epilogue == DenseEpilogue::kGated;
-  if (a.tile_expert) return gated ? pick_routed<true>(a, stream) : pick_routed<false>(a, stream);
-  return gated ? pick_gemm<true>(a, stream) : pick_gemm<false>(a, stream);
+  const bool pair = a.epilogue == DenseEpilogue::kGated, clamped = a.activation == kGateClamped;
+  if (a.tile_expert) {
+    if (pair && clamped) return hipErrorInvalidValue;
+    return pair ? pick_routed<kOneSided>(a, stream) : pick_routed<0>(a, stream);
+  }
+  if (!pair) return pick_gemm<0>(a, stream);
+  return clamped ? pick_gemm<kClampedPair>(a, stream) : pick_gemm<kOneSided>(a, stream);
 }
 
 hipError_t launch_dense_norm(const DenseNormArgs &a, hipStream_t stream) {
@@ -697,6 +711,11 @@ hipError_t launch_dense_norm(const DenseNormArgs &a, hipStream_t stream) {
   if (bytes > 60 * 1024) return hipErrorInvalidValue;
   if (a.f32) dense_norm_kernel<float><<<a.rows, 256, bytes, stream>>>(a);
   else dense_norm_kernel<__bf16><<<a.rows, 256, bytes, stream>>>(a);
+  return hipGetLastError();
+}
+
+hipError_t launch_soft_cap(float *values, uint64_t count, float cap, hipStream_t stream) {
+  soft_cap_kernel<<<(uint32_t)((count + 255) / 256), 256, 0, stream>>>(values, count, cap);
   return hipGetLastError();
 }
 

@@ -142,10 +142,11 @@ int pending_logits(llmopt_hip_context *context, const DispatchRecord &record) {
   if (int status = launched(launch_norm_add(norm, context->stream), name)) return status;
   DenseLinearArgs a = linear(F32, scratch.at<void>(normed), head, rows, vocabulary, width);
   a.epilogue = DenseEpilogue::kStoreF32;
-  a.softcap = softcap;
   a.out_f32 = as_f32(record.buffers[7]);
   a.ld_f32 = vocabulary;
-  return launched(launch_dense_gemm(a, context->stream), name);
+  if (int status = launched(launch_dense_gemm(a, context->stream), name)) return status;
+  if (softcap == 0.0f) return LLMOPT_OK;
+  return launched(launch_soft_cap(a.out_f32, (uint64_t)rows * vocabulary, softcap, context->stream), name);
 }
 
 // {u32 m, width, n, split, conv_first, conv_channels, taps, slots, pending; f32 epsilon, offset, scale}; stream, y, its

@@ -57,12 +57,13 @@ def window_attention(q, k, v, scale, size):
 
 def attention_mixer(h, m, w, eps):
     t, heads, kv, dim = h.shape[0], m["heads"], m["kv_heads"], m["dim"]
-    rot = m["rot"]
-    turn = (rot["dims"], rot["base"], rot["scaling"]["factor"])
+    rot, mask = m.get("rot") or {"dims": 0, "base": 1.0}, m.get("mask")
+    turn = (rot["dims"], rot["base"], rot["scaling"]["factor"] if rot.get("scaling") else 1.0)
     q = rms_unit((h @ w("q").T).reshape(t, heads, dim), eps) * w("q.norm")
     k = rms_unit((h @ w("k").T).reshape(t, kv, dim), eps) * w("k.norm")
     v = (h @ w("v").T).reshape(t, kv, m["vdim"])
-    out = window_attention(rotate(q, *turn), rotate(k, *turn), v, m["scale"], m["mask"]["size"])
+    out = window_attention(rotate(q, *turn), rotate(k, *turn), v, m["scale"],
+                           mask["size"] if mask else None)
     return out.reshape(t, -1) @ w("o").T
 
 

@@ -40,6 +40,8 @@ LEFT = {
     "window of one": window(size=1),
     "window of two": window(size=2, rotated=2),
     "no scaling, low base": window(base=10.0, factor=1.0, rotated=24),
+    "no window": {**window(), "mask": None},
+    "no rotation": {**window(), "rot": None},
     "wide values, several splits": window(heads=4, kv_heads=2, dim=72, vdim=128, size=150, scale=0.1, rotated=40),
 }
 RIGHT = {

@@ -8,11 +8,13 @@ import pytest
 
 from llmopt_amd import model_registry, sampling, trace_replay
 from llmopt_amd.engine import Engine
-from llmopt_amd.layered_model import AttentionMixer, DenseFfn, LayeredConfig, LayeredModel, Mamba2Mixer, RoutedFfn
+from llmopt_amd.layered_model import (DESIGNS, AttentionMixer, DeltaMixer, DenseFfn, JointColumns, LayeredConfig, LayeredModel,
+                                      Mamba2Mixer, RoutedFfn, Rotation, WindowMixer, _Tensors)
 from llmopt_amd.safetensors_file import (SafetensorsError, SafetensorsFile, from_bfloat16, to_bfloat16,
                                          write_safetensors)
 from llmopt_amd.sequence_state import RingShape, Sequence, StateError, StatePool
-from oracle import hybrid_model
+from oracle import hybrid_model, parallel_model
+from tests import parallel_util as pu
 from tests.layered_util import attention, config, dense, make_weights, mamba2, moe
 
 
@@ -257,3 +259,116 @@ def test_restatement_is_causal_and_chunked():
     _, weights = make_weights(only, 1)
     assert np.allclose(hybrid_model.forward(only, weights, tokens[5:10])[0],
                        hybrid_model.forward(only, weights, tokens)[0][5:10])
+
+
+# ---- the Koketar design --------------------------------------------------------------------------------
+
+def test_parallel_config_reads_every_size():
+    cfg = pu.config(pu.parallel(mlp=pu.dense(33, 2.5)), pu.parallel(pu.window(size=9, rotated=6, base=70.0, factor=1.5),
+                                                                    pu.delta(5, 1, 7, 9, 3), 0.25, 1.75))
+    parsed = LayeredConfig.parse(cfg)
+    assert parsed.design is DESIGNS["Koketar"] and parsed.residual_scale == 0.7 and parsed.logit_softcap == 12.0
+    first, second = parsed.layers
+    assert first.mixer.left == WindowMixer(6, 2, 24, 40, 0.3, 0.0, 21, Rotation(14, 5000.0, 3.0))
+    assert first.ffn == DenseFfn(33, 2, 2.5) and second.ffn is None
+    assert second.mixer.right == DeltaMixer(5, 1, 7, 9, 3)
+    assert (second.mixer.left_scale, second.mixer.right_scale) == (0.25, 1.75)
+    assert np.allclose(second.mixer.left.rotation.frequencies, [70.0 ** (-2 * i / 6) / 1.5 for i in range(3)])
+    shapes = parsed.tensor_shapes()
+    assert shapes["l1.mix.right.v.conv"] == (45, 3) and shapes["l1.mix.right.a2"] == (35, None)
+    assert shapes["l1.mix.left.o"] == (72, 240) and shapes["l0.mix.left.k.norm"] == (24,)
+    assert "head" not in shapes and "l1.norm2" not in shapes and "l0.norm2" in shapes
+    columns = JointColumns.of(second.mixer, 11, 6)
+    assert columns.conv == 272 and columns.decay == 272 + 64 and columns.gate == 336 + 16 and columns.split == 360
+    assert columns.total == 365
+    assert model_registry.model_class({"architecture": "Koketar"}) is LayeredModel
+
+
+@pytest.mark.parametrize("bad", [
+    pu.config(pu.parallel(pu.window(heads=5, kv_heads=2))),
+    pu.config(pu.parallel(right=pu.delta(heads=5, kv_heads=2))),
+    pu.config(pu.parallel(pu.window(rotated=7))),
+    pu.config(pu.parallel(pu.window(dim=8, rotated=10))),
+    pu.config(pu.parallel(mlp=pu.dense(8, None))),
+    pu.config(pu.parallel(mlp=moe())),
+    pu.config(attention()),
+    config(pu.parallel()),
+])
+def test_parallel_config_refuses(bad):
+    with pytest.raises(ValueError):
+        LayeredConfig.parse(bad)
+
+
+def test_a_design_without_options_of_its_mechanisms():
+    cfg = pu.config(pu.parallel(mlp=pu.dense()), softcap=None)
+    left = cfg["layers"][0]["mixer"]["left"]
+    del left["mask"]
+    del left["rot"]["scaling"]
+    parsed = LayeredConfig.parse(cfg)
+    assert parsed.logit_softcap == 0.0 and parsed.layers[0].mixer.left.window == 0
+    assert parsed.layers[0].mixer.left.rotation == Rotation(14, 5000.0, 1.0)
+
+
+def test_ranks_come_from_the_weights(tmp_path):
+    parsed = LayeredConfig.parse(pu.config(pu.parallel()))
+    patterns = parsed.random_tensors(np.random.default_rng(0), rank=5)
+    path = str(tmp_path / "w.safetensors")
+    write_safetensors(path, patterns)
+    for source in (patterns, SafetensorsFile(path)):
+        tensors = _Tensors(parsed, source)
+        assert tensors["l0.mix.right.a1"].shape == (5, 72) and tensors["l0.mix.right.g2"].shape == (112, 5)
+    wrong = dict(patterns, **{"l0.mix.right.a2": patterns["l0.mix.right.a2"][:-1]})
+    with pytest.raises(ValueError):
+        _Tensors(parsed, wrong)["l0.mix.right.a2"]
+
+
+def test_restated_window_and_rotation():
+    t, rng = 9, np.random.default_rng(3)
+    v, k = rng.standard_normal((t, 1, 3)), rng.standard_normal((t, 1, 4))
+    out = parallel_model.window_attention(np.zeros((t, 2, 4)), k, v, 1.0, 4)
+    for i in range(t):
+        assert np.allclose(out[i, 1], v[max(0, i - 3):i + 1, 0].mean(0))
+    # a rotation keeps lengths, leaves the rest alone, and makes products depend on distances
+    x = rng.standard_normal((1, 1, 6)).repeat(t, axis=0)
+    turned = parallel_model.rotate(x, 4, 30.0, 2.0)
+    assert np.allclose(turned[:, :, 4:], x[:, :, 4:]) and np.allclose(turned[0], x[0])
+    assert np.allclose((turned ** 2).sum(-1), (x ** 2).sum(-1))
+    products = turned[:, 0] @ turned[:, 0].T
+    assert np.allclose(products[5, 2], products[8, 5]) and not np.allclose(products[5, 2], products[5, 3])
+
+
+def test_restated_delta_rule_closed_forms():
+    """Without decay and with full write strength a key holds what was written to it last; a channel's decay acts on what
+    its key component wrote."""
+    e = np.eye(3)
+    k = np.array([e[0], e[1], e[0]])[:, None]
+    v = np.arange(6.0).reshape(3, 1, 2) + 1.0
+    ones = np.ones((3, 1, 3))
+    out = parallel_model.delta_scan(np.array([e[0], e[0], e[0] + e[1]])[:, None], k, v, ones, np.ones((3, 1)))
+    assert np.allclose(out[:, 0], [v[0, 0], v[0, 0], v[2, 0] + v[1, 0]])
+    decay = ones * np.array([0.5, 0.25, 1.0])
+    out = parallel_model.delta_scan(np.array([e[0] + e[1]] * 3)[:, None], k[:2].repeat([1, 2], axis=0), v, decay,
+                                    np.ones((3, 1)))
+    assert np.allclose(out[2, 0], 0.25 * v[0, 0] + v[2, 0])
+
+
+def test_restated_convolution_norms_and_feed_forward():
+    x = np.arange(1.0, 6.0)[:, None]
+    assert parallel_model.short_conv(x, np.array([[1.0, 10.0]]))[:, 0].tolist() == [10.0, 21.0, 32.0, 43.0, 54.0]
+    assert np.allclose(parallel_model.offset_rms_norm(np.full((1, 4), 3.0), np.array([0.0, 1.0, -1.0, 0.5]), 0.0),
+                       [[1.0, 2.0, 0.0, 1.5]])
+    assert np.allclose(np.linalg.norm(parallel_model.unit(np.array([[3.0, 4.0]]))), 1.0)
+    one = np.ones((1, 1))
+    out = [parallel_model.clamped_ffn(np.array([[z]]), one, one, one, 2.0)[0, 0] for z in (-9.0, 1.0, 9.0)]
+    gate = lambda g: g / (1.0 + np.exp(-1.702 * g))
+    assert np.allclose(out, [gate(-9.0) * -1.0, gate(1.0) * 2.0, gate(2.0) * 3.0])
+
+
+def test_restated_parallel_model_is_causal():
+    cfg = pu.config(pu.parallel(pu.window(size=5), mlp=pu.dense()), pu.parallel())
+    _, weights = make_weights(cfg, 1)
+    tokens = np.random.default_rng(2).integers(0, 90, 14)
+    whole, streams = parallel_model.forward(cfg, weights, tokens)
+    part, part_streams = parallel_model.forward(cfg, weights, tokens[:9])
+    assert np.allclose(part, whole[:9]) and np.allclose(part_streams, streams[:, :9])
+    assert np.abs(whole).max() <= 12.0
